@@ -3,13 +3,16 @@
 // with a factor per query position f(i) = 1 + coef * ln(floor((i + 1) / every) + 1) (or 1) and a
 // distance bias per query head (or none).  Keys at positions [first, i] of the row's request,
 // first = max(0, i - window + 1) with a window, else 0; with `keep_first` the keys at positions
-// [0, keep_first) stay visible after the window has passed them.  `sink_one`: the softmax's denominator
-// holds a one more (a key whose score is 0 and that has no value).  Values may be wider or narrower than keys.
+// [0, keep_first) stay visible after the window has passed them.  The softmax's denominator may hold one
+// more term, a key that has no value: of score 0 (`sink_one`) or of a learned score per head (`sink`, neither
+// scaled nor bent).  With `softcap` c a scaled score s becomes c * tanh(s / c) before the bias.  Values may be
+// wider or narrower than keys.
 //
 // Cache layout: K [pages, layers, kv_heads, page_tokens, head_dim],
 // V [pages, layers, kv_heads, v_dim, page_tokens].
 //
-// kv_store writes a step's keys and values to their rows' places in the pages.  The general
+// kv_store writes a step's keys and values to their rows' places in the pages; with v_eps > 0 every head's
+// value is divided by sqrt(mean(v^2) + v_eps) on the way.  The general
 // attention kernel is one wavefront per (row, query head), 64 keys a round, a lane scores one key;
 // maximum, normaliser and sums are 32-bit, in an order that depends on the row's own position only.
 #include "common.h"
@@ -34,7 +37,7 @@ template <typename T>
 __global__ void kv_store_kernel(const T* __restrict__ k, int ldk, const T* __restrict__ v, int ldv, T* __restrict__ k_pool,
                                 T* __restrict__ v_pool, const int* __restrict__ table, int table_stride,
                                 const int* __restrict__ token_slot, const int* __restrict__ positions, int kv_heads, int head_dim,
-                                int v_dim, int page_tokens, int n_layers, int layer) {
+                                int v_dim, int page_tokens, int n_layers, int layer, float v_eps) {
     const int t = blockIdx.x, g = blockIdx.y;
     const int pos = positions[t];
     const int page = table[static_cast<size_t>(token_slot[t]) * table_stride + pos / page_tokens], in_page = pos % page_tokens;
@@ -43,6 +46,16 @@ __global__ void kv_store_kernel(const T* __restrict__ k, int ldk, const T* __res
     for (int d = threadIdx.x; d < head_dim; d += blockDim.x) kd[d] = ks[d];
     T* vd = v_pool + ba_v_offset(page, n_layers, layer, kv_heads, g, page_tokens, v_dim) + in_page;
     const T* vs = v + static_cast<size_t>(t) * ldv + static_cast<size_t>(g) * v_dim;
+    if (v_eps > 0.f) {
+        float sq = 0.f;
+        for (int d = threadIdx.x; d < v_dim; d += blockDim.x) {
+            const float x = to_float(vs[d]);
+            sq = fmaf(x, x, sq);
+        }
+        const float inv = 1.0f / sqrtf(wave_sum(sq) / static_cast<float>(v_dim) + v_eps);      // (a block is one wavefront)
+        for (int d = threadIdx.x; d < v_dim; d += blockDim.x) vd[static_cast<size_t>(d) * page_tokens] = from_float<T>(to_float(vs[d]) * inv);
+        return;
+    }
     for (int d = threadIdx.x; d < v_dim; d += blockDim.x) vd[static_cast<size_t>(d) * page_tokens] = vs[d];
 }
 
@@ -54,7 +67,7 @@ __global__ __launch_bounds__(CELEG_WAVE) void biased_attention_kernel(
     int table_stride, const int* __restrict__ token_slot, const int* __restrict__ positions, const float* __restrict__ r1,
     const float* __restrict__ r2, const T* __restrict__ gate, int ldg, T* __restrict__ out, int ldo, int q_heads, int kv_heads,
     int head_dim, int v_dim, int page_tokens, int n_layers, int layer, float scale, float coef, int every, int window,
-    int keep_first, int sink_one) {
+    int keep_first, int sink_one, const float* __restrict__ sink, float softcap) {
     extern __shared__ float lds[];  // head_dim floats of q, then 64 weights
     float* qs = lds;
     float* ps = lds + head_dim;
@@ -73,8 +86,9 @@ __global__ __launch_bounds__(CELEG_WAVE) void biased_attention_kernel(
     float acc[BA_MAX_V_CHUNKS];
 #pragma unroll
     for (int j = 0; j < BA_MAX_V_CHUNKS; ++j) acc[j] = 0.f;
-    // (the extra one of the denominator: a key of score 0 seen before all others)
-    float top = sink_one ? 0.f : -INFINITY, total = sink_one ? 1.f : 0.f;
+    // (the denominator's extra term: a key of score 0, or of the head's own number, seen before all others)
+    const bool extra = sink || sink_one;
+    float top = sink ? sink[h] : sink_one ? 0.f : -INFINITY, total = extra ? 1.f : 0.f;
 
     // the kept first keys that the window has passed, then the window (or everything)
     const int kept = min(keep_first, first);
@@ -89,6 +103,7 @@ __global__ __launch_bounds__(CELEG_WAVE) void biased_attention_kernel(
                 float dot = 0.f;
                 for (int d = 0; d < head_dim; ++d) dot = fmaf(qs[d], to_float(kp[d]), dot);
                 score = dot * s;
+                if (softcap > 0.f) score = softcap * tanhf(score / softcap);
                 if (r1) score -= b1 * logf(1.0f + b2 * static_cast<float>(pos - key));
             }
             const float new_top = fmaxf(top, wave_max(score));     // (the round holds at least one visible key)
@@ -135,17 +150,17 @@ __global__ __launch_bounds__(CELEG_WAVE) void biased_attention_kernel(
 
 extern "C" int celeg_kv_store(const void* k, int ldk, const void* v, int ldv, int dtype, void* k_pool, void* v_pool, const int* table,
                               int table_stride, const int* token_slot, const int* positions, int n_tokens, int kv_heads, int head_dim,
-                              int v_dim, int page_tokens, int n_layers, int layer, hipStream_t stream) {
+                              int v_dim, int page_tokens, int n_layers, int layer, float v_eps, hipStream_t stream) {
     if (n_tokens <= 0) return 0;
     dim3 grid(n_tokens, kv_heads), block(CELEG_WAVE);
     if (dtype == CELEG_F32)
         hipLaunchKernelGGL(kv_store_kernel<float>, grid, block, 0, stream, static_cast<const float*>(k), ldk,
                            static_cast<const float*>(v), ldv, static_cast<float*>(k_pool), static_cast<float*>(v_pool), table,
-                           table_stride, token_slot, positions, kv_heads, head_dim, v_dim, page_tokens, n_layers, layer);
+                           table_stride, token_slot, positions, kv_heads, head_dim, v_dim, page_tokens, n_layers, layer, v_eps);
     else
         hipLaunchKernelGGL(kv_store_kernel<bf16>, grid, block, 0, stream, static_cast<const bf16*>(k), ldk,
                            static_cast<const bf16*>(v), ldv, static_cast<bf16*>(k_pool), static_cast<bf16*>(v_pool), table,
-                           table_stride, token_slot, positions, kv_heads, head_dim, v_dim, page_tokens, n_layers, layer);
+                           table_stride, token_slot, positions, kv_heads, head_dim, v_dim, page_tokens, n_layers, layer, v_eps);
     return CELEG_LAUNCH_RESULT();
 }
 
@@ -154,7 +169,8 @@ extern "C" int celeg_biased_attention(const void* q, int ldq, int dtype, const v
                                       int table_stride, const int* token_slot, const int* positions, const float* r1,
                                       const float* r2, const void* gate, int ldg, void* out, int ldo, int n_tokens, int q_heads,
                                       int kv_heads, int head_dim, int v_dim, int page_tokens, int n_layers, int layer, float scale,
-                                      float coef, int every, int window, int keep_first, int sink_one, hipStream_t stream) {
+                                      float coef, int every, int window, int keep_first, int sink_one, const float* sink,
+                                      float softcap, hipStream_t stream) {
     if (n_tokens <= 0) return 0;
     if (v_dim > BA_MAX_V_CHUNKS * CELEG_WAVE || q_heads % kv_heads) return static_cast<int>(hipErrorInvalidValue);
     dim3 grid(n_tokens, q_heads), block(CELEG_WAVE);
@@ -163,11 +179,13 @@ extern "C" int celeg_biased_attention(const void* q, int ldq, int dtype, const v
         hipLaunchKernelGGL(biased_attention_kernel<float>, grid, block, lds, stream, static_cast<const float*>(q), ldq,
                            static_cast<const float*>(k_pool), static_cast<const float*>(v_pool), table, table_stride, token_slot,
                            positions, r1, r2, static_cast<const float*>(gate), ldg, static_cast<float*>(out), ldo, q_heads,
-                           kv_heads, head_dim, v_dim, page_tokens, n_layers, layer, scale, coef, every, window, keep_first, sink_one);
+                           kv_heads, head_dim, v_dim, page_tokens, n_layers, layer, scale, coef, every, window, keep_first, sink_one, sink,
+                           softcap);
     else
         hipLaunchKernelGGL(biased_attention_kernel<bf16>, grid, block, lds, stream, static_cast<const bf16*>(q), ldq,
                            static_cast<const bf16*>(k_pool), static_cast<const bf16*>(v_pool), table, table_stride, token_slot,
                            positions, r1, r2, static_cast<const bf16*>(gate), ldg, static_cast<bf16*>(out), ldo, q_heads, kv_heads,
-                           head_dim, v_dim, page_tokens, n_layers, layer, scale, coef, every, window, keep_first, sink_one);
+                           head_dim, v_dim, page_tokens, n_layers, layer, scale, coef, every, window, keep_first, sink_one,
+                           sink, softcap);
     return CELEG_LAUNCH_RESULT();
 }

@@ -1,9 +1,12 @@
 // Softmax attention with a factor per query position and a distance bias per head, bfloat16, on
 // the matrix cores:
 //     score(i, j) = (q_i . k_j) * scale * f(i) - r1[h] * ln(1 + r2[h] * (i - j)),   weights = softmax over the visible j
-// Visible: j <= i, inside the window where there is one, or among the first `keep_first` positions.  With `sink_one`
-// the denominator holds a one more (a key of score 0 without a value, which the row meets before all others).
-// Keys of `D` numbers, values of `V` numbers a head (both multiples of 32 up to 128).
+// Visible: j <= i, inside the window where there is one, or among the first `keep_first` positions.  The
+// denominator may hold one more term, a key without a value that the row meets before all others: of score 0
+// (`sink_one`) or of a learned score per head (`sink`).  With `softcap` c a scaled score s is bent to
+// c * tanh(s / c) = c - 2 c / (exp(2 s / c) + 1) before the bias.
+// Keys of up to `D` numbers, values of up to `V` numbers a head (D, V multiples of 32 up to 128; smaller heads,
+// keys in multiples of 8 and values in multiples of 4, are staged with zeros behind them).
 // Cache layout: K [pages, layers, kv_heads, page_tokens, D], V [pages, layers, kv_heads, V, page_tokens].
 //
 // Scores are computed transposed (keys as the first operand of a 16x16x32 instruction): a lane
@@ -56,22 +59,23 @@ struct BfFetch {
     bf_u32x4 k[KCH], v[VCH];
     __device__ __forceinline__ void load(int tid, int kb, int pos_last, const bf16* __restrict__ k_pool, const bf16* __restrict__ v_pool,
                                          const int* __restrict__ pages, int page_shift, int page_mask, int page_tokens,
-                                         size_t head_index_stride, int kvh, size_t layer_index) {
+                                         size_t head_index_stride, int kvh, size_t layer_index, int kd, int vd) {
 #pragma unroll
         for (int i = 0; i < KCH; ++i) {
             const int c = tid + THREADS * i, key_in = c / (D / 8), part = c % (D / 8);
             const int key = min(kb + key_in, pos_last);
             const size_t head = (static_cast<size_t>(pages[key >> page_shift]) * head_index_stride + layer_index) + kvh;
-            k[i] = *reinterpret_cast<const bf_u32x4*>(k_pool + (head * page_tokens + (key & page_mask)) * D + 8 * part);
+            k[i] = bf_u32x4{0u, 0u, 0u, 0u};
+            if (8 * part < kd) k[i] = *reinterpret_cast<const bf_u32x4*>(k_pool + (head * page_tokens + (key & page_mask)) * kd + 8 * part);
         }
 #pragma unroll
         for (int i = 0; i < VCH; ++i) {
             const int c = tid + THREADS * i, d = c / (BF_KEYS / 8), part = c % (BF_KEYS / 8);
             const int key = kb + 8 * part;         // eight keys that lie side by side in one page
             bf_u32x4 val = {0u, 0u, 0u, 0u};
-            if (key <= pos_last) {
+            if (key <= pos_last && d < vd) {
                 const size_t head = (static_cast<size_t>(pages[key >> page_shift]) * head_index_stride + layer_index) + kvh;
-                val = *reinterpret_cast<const bf_u32x4*>(v_pool + (head * V + d) * page_tokens + (key & page_mask));
+                val = *reinterpret_cast<const bf_u32x4*>(v_pool + (head * vd + d) * page_tokens + (key & page_mask));
                 const int live = pos_last - key + 1;       // keys of this piece that exist
                 if (live < 8) {
                     if (live <= 6) val[3] = 0u; else val[3] &= 0x0000ffffu;
@@ -102,7 +106,7 @@ struct BfFetch {
 template <int D, int V>
 __device__ __forceinline__ void bf_block(const __bf16* ks, const __bf16* vs, const bf_bf16x8 (&qreg)[D / 32], BfRow<V / 16>& row, int kb,
                                          int my_pos, int window, int keep_first, bool kept_only, int r, int quad, float s2, float b1, float b2,
-                                         bool biased) {
+                                         bool biased, float cap2) {
     constexpr int KROW = D + 8, VROW = BF_KEYS + 8, KS = D / 32, DT = V / 16;
     bf_f32x4 sacc[4];
 #pragma unroll
@@ -115,6 +119,15 @@ __device__ __forceinline__ void bf_block(const __bf16* ks, const __bf16* vs, con
         }
     }
     float top = -INFINITY;
+    if (cap2 > 0.f) {
+        // bent scores: s2 holds 2 log2(e) scale f / c, cap2 is c log2(e)
+#pragma unroll
+        for (int kt = 0; kt < 4; ++kt)
+#pragma unroll
+            for (int i = 0; i < 4; ++i)
+                sacc[kt][i] = fmaf(-2.0f * cap2, __builtin_amdgcn_rcpf(bf_exp2(sacc[kt][i] * s2) + 1.0f), cap2);
+        s2 = 1.0f;
+    }
 #pragma unroll
     for (int kt = 0; kt < 4; ++kt)
 #pragma unroll
@@ -170,10 +183,11 @@ __device__ __forceinline__ void bf_block(const __bf16* ks, const __bf16* vs, con
 // a finished row: divided by its normaliser, times sigmoid(gate), stored
 template <int V>
 __device__ __forceinline__ void bf_store(const BfRow<V / 16>& row, float total, const bf16* __restrict__ gate_row, bf16* __restrict__ out_row,
-                                         int quad) {
+                                         int quad, int vd) {
     const float inv = 1.0f / total;
 #pragma unroll
     for (int dt = 0; dt < V / 16; ++dt) {
+        if (16 * dt + 4 * quad >= vd) continue;
         float g[4] = {1.f, 1.f, 1.f, 1.f};
         if (gate_row) {
             const bf_bf16x4 g4 = __builtin_bit_cast(bf_bf16x4, *reinterpret_cast<const bf_u32x2*>(gate_row + 16 * dt + 4 * quad));
@@ -196,10 +210,11 @@ struct BfArgs {
     const int* seq_start;
     const float* r1;
     const float* r2;
+    const float* sink;
     const bf16* gate;
     bf16* out;
-    int ldq, ldg, ldo, table_stride, n_seqs, q_heads, kv_heads, page_tokens, n_layers, layer, every, window, keep_first, sink_one;
-    float scale, coef;
+    int ldq, ldg, ldo, table_stride, n_seqs, q_heads, kv_heads, page_tokens, n_layers, layer, every, window, keep_first, sink_one, kd, vd;
+    float scale, coef, softcap;
 };
 
 // The key blocks of a tile whose lowest position is pos0: first the blocks that hold the kept first keys
@@ -221,6 +236,13 @@ struct BfBlocks {
     // the last key a block may touch: pages between the kept keys and the window may be gone
     __device__ __forceinline__ int last(int i, int pos_last, int keep) const { return i < n_kept ? keep - 1 : pos_last; }
 };
+
+// a row's factor on the products q.k (in powers of two) and, where scores are bent, the bend in those units
+__device__ __forceinline__ float bf_score_factor(const BfArgs& a, int pos, float& cap2) {
+    const float s = a.scale * bf_query_factor(pos, a.coef, a.every) * BF_LOG2E;
+    cap2 = a.softcap > 0.f ? a.softcap * BF_LOG2E : 0.f;
+    return a.softcap > 0.f ? 2.0f * s / a.softcap : s;
+}
 
 // which tile of `rows` rows: tiles of all requests of the step, one after the other
 __device__ __forceinline__ bool bf_find_tile(const BfArgs& a, int rows, int& tile, int& s, int& row0, int& n) {
@@ -253,18 +275,23 @@ __global__ __launch_bounds__(BF_WAVES * CELEG_WAVE) void biased_attention_rows_k
     const int my_pos = a.seq_start[s] + safe_row;
     const int wave_pos0 = a.seq_start[s] + first_row, wave_last = wave_pos0 + rows_here - 1;
     const int* pages = a.table + static_cast<size_t>(a.seq_slot[s]) * a.table_stride;
-    const float s2 = a.scale * BF_LOG2E * bf_query_factor(my_pos, a.coef, a.every);
+    float cap2;
+    const float s2 = bf_score_factor(a, my_pos, cap2);
     const bool biased = a.r1 != nullptr;
     const float b1 = biased ? a.r1[h] : 0.f, b2 = biased ? a.r2[h] : 0.f;
     bf_bf16x8 qreg[KS];
-    const bf16* qrow = a.q + static_cast<size_t>(row0 + safe_row) * a.ldq + static_cast<size_t>(h) * D;
+    const bf16* qrow = a.q + static_cast<size_t>(row0 + safe_row) * a.ldq + static_cast<size_t>(h) * a.kd;
 #pragma unroll
-    for (int st = 0; st < KS; ++st) qreg[st] = __builtin_bit_cast(bf_bf16x8, *reinterpret_cast<const bf_u32x4*>(qrow + 32 * st + 8 * quad));
+    for (int st = 0; st < KS; ++st) {
+        bf_u32x4 piece = {0u, 0u, 0u, 0u};
+        if (32 * st + 8 * quad < a.kd) piece = *reinterpret_cast<const bf_u32x4*>(qrow + 32 * st + 8 * quad);
+        qreg[st] = __builtin_bit_cast(bf_bf16x8, piece);
+    }
     BfRow<DT> row;
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt) row.acc[dt] = bf_f32x4{0.f, 0.f, 0.f, 0.f};
-    if (a.sink_one) {
-        row.top = 0.f;
+    if (a.sink_one || a.sink) {
+        row.top = a.sink ? a.sink[h] * BF_LOG2E : 0.f;
         row.sum = quad == 0 ? 1.f : 0.f;
     }
     const int page_shift = 31 - __builtin_clz(a.page_tokens), page_mask = a.page_tokens - 1;
@@ -273,7 +300,7 @@ __global__ __launch_bounds__(BF_WAVES * CELEG_WAVE) void biased_attention_rows_k
     const BfBlocks blocks(tile_pos0, a.window, a.keep_first);
     const int n_blocks = blocks.count(pos_last);
     pre.load(tid, blocks.start(0), blocks.last(0, pos_last, a.keep_first), a.k_pool, a.v_pool, pages, page_shift, page_mask, a.page_tokens,
-             head_index_stride, kvh, layer_index);
+             head_index_stride, kvh, layer_index, a.kd, a.vd);
     int turn = 0;
     for (int i = 0; i < n_blocks; ++i, turn ^= 1) {
         const int kb = blocks.start(i);
@@ -283,19 +310,19 @@ __global__ __launch_bounds__(BF_WAVES * CELEG_WAVE) void biased_attention_rows_k
         __syncthreads();
         if (i + 1 < n_blocks)
             pre.load(tid, blocks.start(i + 1), blocks.last(i + 1, pos_last, a.keep_first), a.k_pool, a.v_pool, pages, page_shift, page_mask,
-                     a.page_tokens, head_index_stride, kvh, layer_index);
+                     a.page_tokens, head_index_stride, kvh, layer_index, a.kd, a.vd);
         // blocks none of this wavefront's rows can see
         if (rows_here <= 0) continue;
         if (!blocks.kept(i) && (kb > wave_last || (a.window > 0 && kb >= a.keep_first && kb + BF_KEYS - 1 < wave_pos0 - a.window + 1))) continue;
-        bf_block<D, V>(ks, vs, qreg, row, kb, my_pos, a.window, a.keep_first, blocks.kept(i), r, quad, s2, b1, b2, biased);
+        bf_block<D, V>(ks, vs, qreg, row, kb, my_pos, a.window, a.keep_first, blocks.kept(i), r, quad, s2, b1, b2, biased, cap2);
     }
     float total = row.sum;
     total += __shfl_xor(total, 16, CELEG_WAVE);
     total += __shfl_xor(total, 32, CELEG_WAVE);
     if (r >= rows_here) return;
     const size_t at = static_cast<size_t>(row0 + my_row);
-    bf_store<V>(row, total, a.gate ? a.gate + at * a.ldg + static_cast<size_t>(h) * V : nullptr, a.out + at * a.ldo + static_cast<size_t>(h) * V,
-                quad);
+    bf_store<V>(row, total, a.gate ? a.gate + at * a.ldg + static_cast<size_t>(h) * a.vd : nullptr, a.out + at * a.ldo + static_cast<size_t>(h) * a.vd,
+                quad, a.vd);
 }
 
 template <int D, int V, int WAVES>
@@ -314,18 +341,23 @@ __global__ __launch_bounds__(WAVES * CELEG_WAVE) void biased_attention_tile_kern
     const int my_row = first_row + min(r, rows_here - 1);      // rows past the end repeat the last one (not stored)
     const int my_pos = a.seq_start[s] + my_row;
     const int* pages = a.table + static_cast<size_t>(a.seq_slot[s]) * a.table_stride;
-    const float s2 = a.scale * BF_LOG2E * bf_query_factor(my_pos, a.coef, a.every);
+    float cap2;
+    const float s2 = bf_score_factor(a, my_pos, cap2);
     const bool biased = a.r1 != nullptr;
     const float b1 = biased ? a.r1[h] : 0.f, b2 = biased ? a.r2[h] : 0.f;
     bf_bf16x8 qreg[KS];
-    const bf16* qrow = a.q + static_cast<size_t>(row0 + my_row) * a.ldq + static_cast<size_t>(h) * D;
+    const bf16* qrow = a.q + static_cast<size_t>(row0 + my_row) * a.ldq + static_cast<size_t>(h) * a.kd;
 #pragma unroll
-    for (int st = 0; st < KS; ++st) qreg[st] = __builtin_bit_cast(bf_bf16x8, *reinterpret_cast<const bf_u32x4*>(qrow + 32 * st + 8 * quad));
+    for (int st = 0; st < KS; ++st) {
+        bf_u32x4 piece = {0u, 0u, 0u, 0u};
+        if (32 * st + 8 * quad < a.kd) piece = *reinterpret_cast<const bf_u32x4*>(qrow + 32 * st + 8 * quad);
+        qreg[st] = __builtin_bit_cast(bf_bf16x8, piece);
+    }
     BfRow<DT> row;
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt) row.acc[dt] = bf_f32x4{0.f, 0.f, 0.f, 0.f};
-    if (a.sink_one && wave == 0) {        // (once a row: the first wavefront's share)
-        row.top = 0.f;
+    if ((a.sink_one || a.sink) && wave == 0) {        // (once a row: the first wavefront's share)
+        row.top = a.sink ? a.sink[h] * BF_LOG2E : 0.f;
         row.sum = quad == 0 ? 1.f : 0.f;
     }
     const int page_shift = 31 - __builtin_clz(a.page_tokens), page_mask = a.page_tokens - 1;
@@ -335,7 +367,7 @@ __global__ __launch_bounds__(WAVES * CELEG_WAVE) void biased_attention_tile_kern
     const int n_blocks = blocks.count(pos_last);
     if (wave < n_blocks)
         pre.load(lane, blocks.start(wave), blocks.last(wave, pos_last, a.keep_first), a.k_pool, a.v_pool, pages, page_shift, page_mask,
-                 a.page_tokens, head_index_stride, kvh, layer_index);
+                 a.page_tokens, head_index_stride, kvh, layer_index, a.kd, a.vd);
     for (int i = wave; i < n_blocks; i += WAVES) {
         __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
         __builtin_amdgcn_wave_barrier();
@@ -345,8 +377,8 @@ __global__ __launch_bounds__(WAVES * CELEG_WAVE) void biased_attention_tile_kern
         __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
         if (i + WAVES < n_blocks)
             pre.load(lane, blocks.start(i + WAVES), blocks.last(i + WAVES, pos_last, a.keep_first), a.k_pool, a.v_pool, pages, page_shift,
-                     page_mask, a.page_tokens, head_index_stride, kvh, layer_index);
-        bf_block<D, V>(ks, vs, qreg, row, blocks.start(i), my_pos, a.window, a.keep_first, blocks.kept(i), r, quad, s2, b1, b2, biased);
+                     page_mask, a.page_tokens, head_index_stride, kvh, layer_index, a.kd, a.vd);
+        bf_block<D, V>(ks, vs, qreg, row, blocks.start(i), my_pos, a.window, a.keep_first, blocks.kept(i), r, quad, s2, b1, b2, biased, cap2);
     }
     // the wavefronts' maxima, normalisers and sums meet in LDS (every wavefront's staging area is
     // free after the barrier); the first one joins them in the order of the wavefronts and stores
@@ -388,8 +420,8 @@ __global__ __launch_bounds__(WAVES * CELEG_WAVE) void biased_attention_tile_kern
     total += __shfl_xor(total, 32, CELEG_WAVE);
     if (r >= rows_here) return;
     const size_t at = static_cast<size_t>(row0 + my_row);
-    bf_store<V>(row, total, a.gate ? a.gate + at * a.ldg + static_cast<size_t>(h) * V : nullptr, a.out + at * a.ldo + static_cast<size_t>(h) * V,
-                quad);
+    bf_store<V>(row, total, a.gate ? a.gate + at * a.ldg + static_cast<size_t>(h) * a.vd : nullptr, a.out + at * a.ldo + static_cast<size_t>(h) * a.vd,
+                quad, a.vd);
 }
 
 constexpr int bf_block_bytes(int d, int v) { return (BF_KEYS * (d + 8) + v * (BF_KEYS + 8)) * 2; }
@@ -411,10 +443,10 @@ int bf_launch(int form, int max_tiles, const BfArgs& a, hipStream_t stream) {
 
 template <int D>
 int bf_launch_v(int v_dim, int form, int max_tiles, const BfArgs& a, hipStream_t stream) {
-    switch (v_dim) {
-        case 32: return bf_launch<D, 32>(form, max_tiles, a, stream);
-        case 64: return bf_launch<D, 64>(form, max_tiles, a, stream);
-        case 96: return bf_launch<D, 96>(form, max_tiles, a, stream);
+    switch ((v_dim + 31) / 32) {
+        case 1: return bf_launch<D, 32>(form, max_tiles, a, stream);
+        case 2: return bf_launch<D, 64>(form, max_tiles, a, stream);
+        case 3: return bf_launch<D, 96>(form, max_tiles, a, stream);
         default: return bf_launch<D, 128>(form, max_tiles, a, stream);
     }
 }
@@ -423,8 +455,7 @@ int bf_launch_v(int v_dim, int form, int max_tiles, const BfArgs& a, hipStream_t
 
 // sizes of keys and values a head that the matrix-core kernels take
 extern "C" int celeg_biased_attention_fast_ok(int head_dim, int v_dim) {
-    auto ok = [](int n) { return n == 32 || n == 64 || n == 96 || n == 128; };
-    return ok(head_dim) && ok(v_dim);
+    return head_dim > 0 && head_dim <= 128 && head_dim % 8 == 0 && v_dim > 0 && v_dim <= 128 && v_dim % 4 == 0;
 }
 
 // bfloat16 on the matrix cores; form 0: tiles of 16 rows whose key blocks the wavefronts share out
@@ -437,7 +468,7 @@ extern "C" int celeg_biased_attention_fast(int form, const void* q, int ldq, con
                                            int max_tiles, const float* r1, const float* r2, const void* gate, int ldg, void* out, int ldo,
                                            int q_heads, int kv_heads, int head_dim, int v_dim, int page_tokens, int n_layers, int layer,
                                            float scale, float coef, int every, int window, int keep_first, int sink_one,
-                                           hipStream_t stream) {
+                                           const float* sink, float softcap, hipStream_t stream) {
     if (max_tiles <= 0 || n_seqs <= 0) return 0;
     if (!celeg_biased_attention_fast_ok(head_dim, v_dim) || q_heads % kv_heads || page_tokens < 8 || (page_tokens & (page_tokens - 1)) ||
         ldq % 8 || ldo % 4 || (gate && ldg % 4) || (r1 == nullptr) != (r2 == nullptr))
@@ -468,12 +499,16 @@ extern "C" int celeg_biased_attention_fast(int form, const void* q, int ldq, con
     a.window = window;
     a.keep_first = window > 0 ? keep_first : 0;
     a.sink_one = sink_one;
+    a.sink = sink;
+    a.softcap = softcap;
+    a.kd = head_dim;
+    a.vd = v_dim;
     a.scale = scale;
     a.coef = coef;
-    switch (head_dim) {
-        case 32: return bf_launch_v<32>(v_dim, form, max_tiles, a, stream);
-        case 64: return bf_launch_v<64>(v_dim, form, max_tiles, a, stream);
-        case 96: return bf_launch_v<96>(v_dim, form, max_tiles, a, stream);
+    switch ((head_dim + 31) / 32) {
+        case 1: return bf_launch_v<32>(v_dim, form, max_tiles, a, stream);
+        case 2: return bf_launch_v<64>(v_dim, form, max_tiles, a, stream);
+        case 3: return bf_launch_v<96>(v_dim, form, max_tiles, a, stream);
         default: return bf_launch_v<128>(v_dim, form, max_tiles, a, stream);
     }
 }

@@ -1,4 +1,4 @@
-// Row-wise and element-wise kernels: embedding gather, RMSNorm (with the residual
+// Row-wise and element-wise kernels: embedding gather (of tokens, of pairs of tokens), RMSNorm (with the residual
 // addition folded in), SwiGLU, bias, dtype conversion, block-table updates.
 #include "common.h"
 
@@ -41,6 +41,66 @@ extern "C" int celeg_embed(const void* table, int table_dtype, const int* ids, f
     else
         hipLaunchKernelGGL(embed_kernel<bf16>, grid, block, 0, stream,
                            static_cast<const bf16*>(table), ids, out, width, vocab, scale);
+    return CELEG_LAUNCH_RESULT();
+}
+
+// ---------------------------------------------------------------- embedding of pairs
+// out[row, :] = table[id] + pairs[(previous id * mul_prev + id * mul_cur) mod buckets], the sequence's first
+// token (position 0) taking row `buckets` of pairs; the sum in 32-bit.  The previous token is the row before
+// in the request's portion, or the one its slot keeps from the step before; the block of a portion's
+// first row, the only one that reads it, leaves the portion's last token there.  Where xb is given, the
+// stream's bfloat16 copy (in the layout of the fused products' operands) and the row's sum of squares leave with it.
+template <typename TW>
+__global__ __launch_bounds__(256) void embed_pairs_kernel(const TW* __restrict__ table, const TW* __restrict__ pairs, const int* __restrict__ ids,
+                                                          const int* __restrict__ positions, const int* __restrict__ token_seq,
+                                                          const int* __restrict__ cu_seqlens, const int* __restrict__ token_slot,
+                                                          int* __restrict__ last, size_t last_stride, long long buckets, long long mul_prev,
+                                                          long long mul_cur, float* __restrict__ out, bf16* __restrict__ xb, int ldx,
+                                                          long long xb_k8, float* __restrict__ stats, int stats_ld, int width, int vocab) {
+    __shared__ float scratch[16];
+    const int row = blockIdx.x, seq = token_seq[row], first = cu_seqlens[seq];
+    const int id = ids[row];
+    int* mine = last + static_cast<size_t>(token_slot[row]) * last_stride;
+    const int before = positions[row] == 0 ? -1 : row > first ? ids[row - 1] : *mine;
+    if (row == first) {
+        __syncthreads();               // (every thread has read the token kept so far)
+        if (threadIdx.x == 0) *mine = ids[cu_seqlens[seq + 1] - 1];
+    }
+    const bool ok = id >= 0 && id < vocab;      // the host rejects other ids; never read out of bounds
+    long long bucket = buckets;
+    if (before >= 0 && ok) {
+        bucket = (before * mul_prev + id * mul_cur) % buckets;
+        if (bucket < 0) bucket += buckets;
+    }
+    const TW* src = table + static_cast<size_t>(ok ? id : 0) * width;
+    const TW* pair = pairs + static_cast<size_t>(bucket) * width;
+    float sum = 0.f;
+    for (int i = threadIdx.x; i < width; i += blockDim.x) {
+        const float v = ok ? to_float(src[i]) + to_float(pair[i]) : 0.f;
+        out[static_cast<size_t>(row) * width + i] = v;
+        if (xb) xb[static_cast<size_t>(row) * ldx + static_cast<size_t>(i >> 3) * xb_k8 + (i & 7)] = from_float<bf16>(v);
+        sum += v * v;
+    }
+    if (!stats) return;
+    sum = block_sum(sum, scratch);
+    if (threadIdx.x == 0) stats[static_cast<size_t>(row) * stats_ld] = sum;
+}
+
+extern "C" int celeg_embed_pairs(const void* table, const void* pairs, int table_dtype, const int* ids, const int* positions,
+                                 const int* token_seq, const int* cu_seqlens, const int* token_slot, int* last, size_t last_stride,
+                                 long long buckets, long long mul_prev, long long mul_cur, float* out, void* xb, int ldx, long long xb_k8,
+                                 float* stats, int stats_ld, int rows, int width, int vocab, hipStream_t stream) {
+    if (rows <= 0) return 0;
+    if (buckets <= 0 || (xb && !stats)) return static_cast<int>(hipErrorInvalidValue);
+    dim3 grid(rows), block(256);
+    if (table_dtype == CELEG_F32)
+        hipLaunchKernelGGL(embed_pairs_kernel<float>, grid, block, 0, stream, static_cast<const float*>(table), static_cast<const float*>(pairs),
+                           ids, positions, token_seq, cu_seqlens, token_slot, last, last_stride, buckets, mul_prev, mul_cur, out,
+                           static_cast<bf16*>(xb), ldx, xb_k8, stats, stats_ld, width, vocab);
+    else
+        hipLaunchKernelGGL(embed_pairs_kernel<bf16>, grid, block, 0, stream, static_cast<const bf16*>(table), static_cast<const bf16*>(pairs),
+                           ids, positions, token_seq, cu_seqlens, token_slot, last, last_stride, buckets, mul_prev, mul_cur, out,
+                           static_cast<bf16*>(xb), ldx, xb_k8, stats, stats_ld, width, vocab);
     return CELEG_LAUNCH_RESULT();
 }
 

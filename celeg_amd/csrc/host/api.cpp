@@ -986,7 +986,7 @@ public:
     bool graph_safe() const override { return part_.description().graph_safe; }
     WeightSpecs weight_specs() const override { return part_.description().weights; }
     void load(const PartTensors& t, Runtime&) override { part_.load(t); }
-    void forward(const int* token_ids, const Tensor& out, Runtime& rt, const StepBatch* batch) override {
+    void forward(const int* token_ids, const Tensor& out, Runtime& rt, const StepBatch* batch, const LayerCache&) override {
         celeg_forward_args args{};
         args.out = view_of(out);
         args.token_ids = token_ids;

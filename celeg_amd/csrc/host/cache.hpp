@@ -80,8 +80,10 @@ struct StateNeed {
 };
 
 // What a model's run order needs.  kv_of_step[i] = (group, layer in group, writes) for the
-// entries of the run order whose mixer uses keys and values; states lists (run-order entry, need).
+// entries of the run order whose mixer uses keys and values; states lists (run-order entry, need), the
+// embedding's state standing under the entry EMBEDDING, before all entries of the run order.
 struct CacheLayout {
+    static constexpr int EMBEDDING = -1;
     struct KvUse { int group, layer; bool writes; };
     std::vector<KVNeed> kv_groups;
     std::vector<int> group_layers;

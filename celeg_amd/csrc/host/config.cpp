@@ -1325,6 +1325,199 @@ ModelSpec vabuzen_build_spec(const Json& c) {
 
 }  // namespace
 
+// ---------------------------------------------------------------------------- Minilorn
+// A pre-norm decoder (RMS norms, plain sums) of three kinds of mixer, whose embedding adds a row of a second
+// table chosen by the pair (previous token, token).  config.json describes every layer by itself:
+//   {"architecture": "Minilorn", "vocab", "width", "norm": {"eps"},
+//    "embedding": {"bigram": {"buckets", "mul_prev", "mul_cur"}} (absent: the token's own row alone),
+//    "max_context" (an engine limit; optional),
+//    "layers": [{"type": "attention",
+//                "mixer": {"heads", "kv_heads" (absent: heads), "dim", "vdim" (absent: dim), "scale",
+//                          "q_temp": {"coef", "every"} (absent: none), "softcap" (absent: none)},
+//                "mlp": null | {"kind": "dense", "ff"}},
+//               {"type": "latent_attention",
+//                "mixer": {"heads", "dim", "rot_dim", "vdim", "q_rank", "kv_rank", "scale", "rot": {"base", "dims"}
+//                          (neighbouring values pair), "mask": {"size"} (absent: every earlier key)}, "mlp": ...},
+//               {"type": "mlstm", "mixer": {"heads", "dim", "vdim", "gate_cap"}, "mlp": ...}]}
+// Tensors: embed, bigram [buckets + 1, width], head, final.norm, l<i>.norm1, l<i>.norm2;
+// attention: l<i>.mix.{q, k, v, sink, o}; latent: l<i>.mix.{dq, dq.norm, uq, dkv, dkv.norm, uk, uv, o};
+// mlstm: l<i>.mix.{q, k, v, g, i, i.b, f, f.b, norm, o}; l<i>.mlp.{up, down, act}.
+namespace {
+
+Json minilorn_read_config(const Json& raw, const TensorShapes*) {
+    if (!raw.is_object()) throw ConfigError("config.json is not an object");
+    Json out = Json::object();
+    out.set("architecture", "Minilorn");
+    out.set("vocab", regipel_int(raw, "vocab", ""));
+    out.set("width", regipel_int(raw, "width", ""));
+    const double eps = regipel_number(regipel_object(raw, "norm", ""), "eps", "norm.");
+    if (!(eps > 0)) throw ConfigError("config.json: 'norm.eps' must be positive");
+    out.set("norm", Json::object().set("eps", eps));
+    Json bigram;
+    if (!raw["embedding"].is_null()) {
+        const Json& e = regipel_object(raw, "embedding", "");
+        if (!e["bigram"].is_null()) {
+            const Json& b = regipel_object(e, "bigram", "embedding.");
+            const std::string bw = "embedding.bigram.";
+            bigram = Json::object().set("buckets", regipel_int(b, "buckets", bw)).set("mul_prev", regipel_int(b, "mul_prev", bw, 0))
+                         .set("mul_cur", regipel_int(b, "mul_cur", bw, 0));
+        }
+    }
+    out.set("embedding", Json::object().set("bigram", bigram));
+    out.set("max_context", raw["max_context"].is_null() ? 131072LL : regipel_int(raw, "max_context", ""));
+    if (!raw["layers"].is_array() || raw["layers"].size() == 0) throw ConfigError("config.json: 'layers' must be a list of layers");
+    Json layers = Json::array();
+    int i = 0;
+    for (const Json& l : raw["layers"].items()) {
+        const std::string where = "layers[" + std::to_string(i++) + "].";
+        if (!l.is_object()) throw ConfigError("config.json: " + where + " must be an object");
+        const std::string type = l.get_string("type", "");
+        if (type != "attention" && type != "latent_attention" && type != "mlstm")
+            throw ConfigError("config.json: " + where + "'type' is '" + type + "'; known types are ['attention', 'latent_attention', 'mlstm']");
+        const Json& m = regipel_object(l, "mixer", where);
+        const std::string mw = where + "mixer.";
+        const long long heads = regipel_int(m, "heads", mw), dim = regipel_int(m, "dim", mw);
+        Json mixer = Json::object().set("heads", heads).set("dim", dim);
+        if (type == "attention") {
+            const long long kv_heads = m["kv_heads"].is_null() ? heads : regipel_int(m, "kv_heads", mw);
+            if (heads % kv_heads) throw ConfigError("config.json: " + mw + "'heads' must be a multiple of 'kv_heads'");
+            const long long vdim = m["vdim"].is_null() ? dim : regipel_int(m, "vdim", mw);
+            if (vdim > 256) throw ConfigError("config.json: " + mw + "'vdim' may be at most 256");
+            if (dim > 1024) throw ConfigError("config.json: " + mw + "'dim' may be at most 1024");
+            mixer.set("kv_heads", kv_heads).set("vdim", vdim).set("scale", regipel_number(m, "scale", mw));
+            Json q_temp, softcap;
+            if (!m["q_temp"].is_null()) {
+                const Json& t = regipel_object(m, "q_temp", mw);
+                q_temp = Json::object().set("coef", regipel_number(t, "coef", mw + "q_temp.")).set("every", regipel_int(t, "every", mw + "q_temp."));
+            }
+            if (!m["softcap"].is_null()) {
+                const double cap = regipel_number(m, "softcap", mw);
+                if (!(cap > 0)) throw ConfigError("config.json: " + mw + "'softcap' must be positive");
+                softcap = cap;
+            }
+            mixer.set("q_temp", q_temp).set("softcap", softcap);
+        } else if (type == "latent_attention") {
+            const long long rot_dim = regipel_int(m, "rot_dim", mw, 0);
+            mixer.set("rot_dim", rot_dim).set("vdim", regipel_int(m, "vdim", mw)).set("q_rank", regipel_int(m, "q_rank", mw))
+                .set("kv_rank", regipel_int(m, "kv_rank", mw)).set("scale", regipel_number(m, "scale", mw))
+                .set("rot", rot_dim > 0 ? vabuzen_rot(m, mw, rot_dim, "rot_dim") : Json());
+            if (mixer["kv_rank"].as_int() > 1024) throw ConfigError("config.json: " + mw + "'kv_rank' may be at most 1024");
+            Json mask;
+            if (!m["mask"].is_null()) mask = Json::object().set("size", regipel_int(regipel_object(m, "mask", mw), "size", mw + "mask."));
+            mixer.set("mask", mask);
+        } else {
+            const long long vdim = regipel_int(m, "vdim", mw);
+            if (dim > 256) throw ConfigError("config.json: " + mw + "'dim' may be at most 256");
+            if (vdim > 512) throw ConfigError("config.json: " + mw + "'vdim' may be at most 512");
+            const double cap = regipel_number(m, "gate_cap", mw);
+            if (!(cap > 0)) throw ConfigError("config.json: " + mw + "'gate_cap' must be positive");
+            mixer.set("vdim", vdim).set("gate_cap", cap);
+        }
+        Json mlp;
+        if (!l["mlp"].is_null()) {
+            const Json& f = regipel_object(l, "mlp", where);
+            const std::string fw = where + "mlp.", kind = f.get_string("kind", "");
+            if (kind != "dense") throw ConfigError("config.json: " + fw + "'kind' is '" + kind + "'; known kinds are ['dense']");
+            mlp = Json::object().set("kind", kind).set("ff", regipel_int(f, "ff", fw));
+        }
+        layers.push(Json::object().set("type", type).set("mixer", mixer).set("mlp", mlp));
+    }
+    out.set("layers", layers);
+    for (const char* key : {"bos_token_id", "eos_token_id"})
+        if (!raw[key].is_null()) out.set(key, raw[key]);
+    return out;
+}
+
+ModelSpec minilorn_build_spec(const Json& c) {
+    const long long W = c["width"].as_int();
+    const double eps = c["norm"]["eps"].as_double();
+    auto norm = [&](const std::string& name) {
+        PartSpec p;
+        p.kind = "rmsnorm";
+        p.params = Json::object().set("width", W).set("eps", eps);
+        p.tensors = {{"weight", name}};
+        return p;
+    };
+    ModelSpec spec;
+    int i = 0;
+    for (const Json& l : c["layers"].items()) {
+        const std::string p = "l" + std::to_string(i) + ".", type = l["type"].as_string();
+        const Json& m = l["mixer"];
+        LayerSpec layer;
+        layer.arrangement = "pre_norm";
+        layer.mixer.params = Json::object().set("width", W).set("heads", m["heads"]);
+        auto tensors = [&](std::initializer_list<const char*> roles) {
+            for (const char* role : roles) layer.mixer.tensors.emplace_back(role, p + "mix." + role);
+        };
+        if (type == "attention") {
+            layer.mixer.kind = "biased_attention";
+            layer.mixer.params.set("kv_heads", m["kv_heads"]).set("head_dim", m["dim"]).set("v_dim", m["vdim"]).set("scale", m["scale"])
+                .set("sink", true).set("value_norm", true).set("eps", eps);
+            if (!m["q_temp"].is_null()) layer.mixer.params.set("query_temperature", m["q_temp"]);
+            if (!m["softcap"].is_null()) layer.mixer.params.set("softcap", m["softcap"]);
+            tensors({"q", "k", "v", "sink", "o"});
+        } else if (type == "latent_attention") {
+            layer.mixer.kind = "latent_attention";
+            layer.mixer.params.set("dim", m["dim"]).set("rot_dim", m["rot_dim"]).set("vdim", m["vdim"]).set("q_rank", m["q_rank"])
+                .set("kv_rank", m["kv_rank"]).set("scale", m["scale"]).set("eps", eps).set("sink", false).set("gate", false);
+            if (!m["mask"].is_null()) layer.mixer.params.set("window", m["mask"]["size"]);
+            if (!m["rot"].is_null()) {
+                PartSpec rope;
+                rope.kind = "rope";
+                rope.params = Json::object().set("theta", m["rot"]["base"]).set("rotary_dim", m["rot"]["dims"])
+                                  .set("head_dim", m["rot_dim"]).set("pairing", "neighbours");
+                layer.mixer.params.set("position", rope.to_json());
+            }
+            tensors({"dq", "uq", "dkv", "uk", "uv", "o"});
+            layer.mixer.tensors.emplace_back("dq_norm", p + "mix.dq.norm");
+            layer.mixer.tensors.emplace_back("dkv_norm", p + "mix.dkv.norm");
+        } else {
+            layer.mixer.kind = "matrix_memory";
+            layer.mixer.params.set("dim", m["dim"]).set("vdim", m["vdim"]).set("gate_cap", m["gate_cap"]).set("eps", eps);
+            tensors({"q", "k", "v", "g", "i", "f", "norm", "o"});
+            layer.mixer.tensors.emplace_back("i_bias", p + "mix.i.b");
+            layer.mixer.tensors.emplace_back("f_bias", p + "mix.f.b");
+        }
+        layer.mixer_norm = norm(p + "norm1");
+        if (l["mlp"].is_null()) {
+            layer.ffn.kind = "none";
+            layer.ffn_norm.kind = "identity";
+        } else {
+            layer.ffn.kind = "mlp";
+            layer.ffn.params = Json::object().set("width", W).set("ff", l["mlp"]["ff"]).set("activation", "xielu").set("bias", false);
+            layer.ffn.tensors = {{"up", p + "mlp.up"}, {"down", p + "mlp.down"}, {"act", p + "mlp.act"}};
+            layer.ffn_norm = norm(p + "norm2");
+        }
+        spec.layers.push_back(std::move(layer));
+        spec.order.push_back(RunStep{i, {}, false, 0});
+        ++i;
+    }
+    spec.architecture = "Minilorn";
+    spec.vocab_size = static_cast<int>(c["vocab"].as_int());
+    spec.hidden_size = static_cast<int>(W);
+    spec.max_context = static_cast<int>(c["max_context"].as_int());
+    spec.embedding.kind = "embedding";
+    spec.embedding.params = Json::object().set("vocab", c["vocab"]).set("width", W);
+    spec.embedding.tensors = {{"table", "embed"}};
+    if (!c["embedding"]["bigram"].is_null()) {
+        spec.embedding.params.set("pairs", c["embedding"]["bigram"]);
+        spec.embedding.tensors.emplace_back("pairs", "bigram");
+    }
+    spec.head.kind = "linear_head";
+    spec.head.params = Json::object().set("vocab", c["vocab"]).set("width", W);
+    spec.head.tensors = {{"weight", "head"}};
+    spec.final_norm = norm("final.norm");
+    if (c["eos_token_id"].is_array())
+        for (const Json& e : c["eos_token_id"].items()) spec.eos_token_ids.push_back(static_cast<int>(e.as_int()));
+    else if (c["eos_token_id"].is_int())
+        spec.eos_token_ids.push_back(static_cast<int>(c["eos_token_id"].as_int()));
+    if (c["bos_token_id"].is_int()) spec.bos_token_id = static_cast<int>(c["bos_token_id"].as_int());
+    spec.validate();
+    return spec;
+}
+
+}  // namespace
+
 namespace {
 void register_builtin() {
     Architecture lfm2;
@@ -1363,6 +1556,13 @@ void register_builtin() {
     vabuzen.build_spec = vabuzen_build_spec;
     table()["Vabuzen"] = vabuzen;
     table()["vabuzen"] = vabuzen;
+    Architecture minilorn;
+    minilorn.name = "Minilorn";
+    minilorn.aliases = {"minilorn"};
+    minilorn.read_config = minilorn_read_config;
+    minilorn.build_spec = minilorn_build_spec;
+    table()["Minilorn"] = minilorn;
+    table()["minilorn"] = minilorn;
 }
 
 }  // namespace

@@ -17,6 +17,10 @@ extern "C" {
 int celeg_embed(const void* table, int table_dtype, const int* ids, float* out, int rows, int width, int vocab,
                 float scale, hipStream_t stream);
 int celeg_scale_f32(float* x, size_t total, float scale, hipStream_t stream);
+int celeg_embed_pairs(const void* table, const void* pairs, int table_dtype, const int* ids, const int* positions,
+                      const int* token_seq, const int* cu_seqlens, const int* token_slot, int* last, size_t last_stride,
+                      long long buckets, long long mul_prev, long long mul_cur, float* out, void* xb, int ldx, long long xb_k8,
+                      float* stats, int stats_ld, int rows, int width, int vocab, hipStream_t stream);
 int celeg_rmsnorm(void* x, int x_dtype, const void* delta, int delta_dtype, const float* w, void* out, int out_dtype,
                   const int* rows, int n_rows, int width, float eps, int write_back, hipStream_t stream);
 int celeg_swiglu(const void* gu, void* out, int dtype, int rows, int ff, hipStream_t stream);
@@ -38,14 +42,15 @@ int celeg_hyper_step(float* xs, const void* y, int y_dtype, const float* mix, co
 int celeg_latent_prepare(void* proj, int ld, int dtype, int q_off, int dkv_off, int heads, int dim, int rot, int rank,
                          const float* weight, float eps, const float* inv_freq, int rotary, int pairing,
                          const int* positions, const int* token_slot, const int* table, int table_stride, void* pool,
-                         int n_layers, int layer, int page_tokens, int write, int n_tokens, hipStream_t stream);
+                         int n_layers, int layer, int page_tokens, int write, int n_tokens, int cq_off, int q_rank,
+                         const float* q_weight, void* cq, hipStream_t stream);
 int celeg_headwise_linear(const void* x, int ldx, int x_head, const void* w, int dtype, int heads, int N, int K, void* out,
                           int ldo, int o_head, int tail, const void* gate, int ldg, int rows, int matrix_cores,
-                          hipStream_t stream);
+                          const float* tail_freq, int rotary, int pairing, const int* positions, hipStream_t stream);
 int celeg_latent_attention(const void* q, int ldq, const void* pool, int dtype, const int* table, int table_stride,
                            const int* token_slot, const int* positions, const float* sink, void* out, int ldo,
                            int n_tokens, int heads, int rank, int rot, int page_tokens, int n_layers, int layer,
-                           float scale, hipStream_t stream);
+                           float scale, int window, hipStream_t stream);
 // latent_fast.hip
 int celeg_latent_attention_fast_ok(int rank, int rot);
 int celeg_latent_attention_tile_rows(int rank, int rot);
@@ -53,7 +58,7 @@ int celeg_latent_attention_fast(int form, const void* q, int ldq, const void* po
                                 const int* cu_seqlens, const int* seq_slot, const int* seq_start, int n_seqs, int max_tiles,
                                 const int* token_slot, const int* positions, int n_single, const float* sink, void* out,
                                 int ldo, float* ws_o, float* ws_ml, int n_splits, int blocks_per_split, int heads, int rank,
-                                int rot, int page_tokens, int n_layers, int layer, float scale, hipStream_t stream);
+                                int rot, int page_tokens, int n_layers, int layer, float scale, int window, hipStream_t stream);
 // moe.hip
 int celeg_moe_route(const float* logits, int rows, int experts, int top, int score, int renorm, int groups, int keep,
                     float renorm_eps, float scale, int* ids, float* weights, hipStream_t stream);
@@ -173,7 +178,7 @@ int celeg_delta_gated_norm(const float* o, const float* w, const void* gate, int
                            int n_tokens, int H, int V, int act, hipStream_t stream);
 // layer_glue.hip
 int celeg_activation_bias(const void* x, int ldx, const float* bias, void* out, int ldo, int dtype, int rows, int cols, int act,
-                          hipStream_t stream);
+                          float p0, float p1, hipStream_t stream);
 int celeg_residual_sum(float* h, const void* a, int lda, const void* b, int ldb, void* copy, int dtype, int rows, int width,
                        hipStream_t stream);
 int celeg_token_gate(const void* z, int ldz, const void* table, int ld_table, int offset, const int* token_ids, void* g, int dtype,
@@ -192,19 +197,26 @@ int celeg_conv_rope_store(const void* proj, int ld, int dtype, const float* conv
 // biased_attention.hip
 int celeg_kv_store(const void* k, int ldk, const void* v, int ldv, int dtype, void* k_pool, void* v_pool, const int* table,
                    int table_stride, const int* token_slot, const int* positions, int n_tokens, int kv_heads, int head_dim, int v_dim,
-                   int page_tokens, int n_layers, int layer, hipStream_t stream);
+                   int page_tokens, int n_layers, int layer, float v_eps, hipStream_t stream);
 int celeg_biased_attention(const void* q, int ldq, int dtype, const void* k_pool, const void* v_pool, const int* table,
                            int table_stride, const int* token_slot, const int* positions, const float* r1, const float* r2,
                            const void* gate, int ldg, void* out, int ldo, int n_tokens, int q_heads, int kv_heads, int head_dim,
                            int v_dim, int page_tokens, int n_layers, int layer, float scale, float coef, int every, int window,
-                           int keep_first, int sink_one, hipStream_t stream);
+                           int keep_first, int sink_one, const float* sink, float softcap, hipStream_t stream);
 // biased_attention_fast.hip
 int celeg_biased_attention_fast_ok(int head_dim, int v_dim);
 int celeg_biased_attention_fast(int form, const void* q, int ldq, const void* k_pool, const void* v_pool, const int* table, int table_stride,
                                 const int* cu_seqlens, const int* seq_slot, const int* seq_start, int n_seqs, int max_tiles,
                                 const float* r1, const float* r2, const void* gate, int ldg, void* out, int ldo, int q_heads,
                                 int kv_heads, int head_dim, int v_dim, int page_tokens, int n_layers, int layer, float scale, float coef,
-                                int every, int window, int keep_first, int sink_one, hipStream_t stream);
+                                int every, int window, int keep_first, int sink_one, const float* sink, float softcap,
+                                hipStream_t stream);
+// matrix_memory.hip
+int celeg_matrix_memory(const void* proj, int ld, int dtype, int col_q, int col_k, int col_v, int col_g, int col_i, int col_f,
+                        const float* bias_i, const float* bias_f, const float* norm, float* S, size_t ldS, float* n, size_t ldn,
+                        float* m, size_t ldm, const int* cu_seqlens, const int* seq_slot, const int* token_slot, float* planes,
+                        float* chunk_s, float* chunk_n, void* out, int ldo, int n_rows, int n_seqs, int n_single, int max_chunks,
+                        int H, int D, int V, float cap, float eps, hipStream_t stream);
 // linear_scan.hip
 int celeg_lru_gates(const void* x, int ldx, int dtype, const float* conv_w, const float* conv_b, const float* ra_t, const float* ra_b,
                     const float* ri_t, const float* ri_b, const float* lam, const float* conv_state, size_t state_stride,

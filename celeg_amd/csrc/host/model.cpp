@@ -129,6 +129,7 @@ long long Model::weight_count() {
 
 CacheLayout Model::cache_layout() {
     CacheLayout layout;
+    for (const StateNeed& s : embedding_->state_needs()) layout.states.emplace_back(CacheLayout::EMBEDDING, s);
     for (size_t i = 0; i < spec.order.size(); ++i) {
         const RunStep& step = spec.order[i];
         Mixer& mixer = mixer_of(step.layer);
@@ -170,6 +171,7 @@ void Model::load(const WeightMap& tensors, Runtime& rt) {
 
 void Model::bind_cache(const CacheManager& cache) {
     caches_.clear();
+    embedding_cache_ = cache.layer_cache(CacheLayout::EMBEDDING);
     for (size_t i = 0; i < spec.order.size(); ++i) caches_.push_back(cache.layer_cache(static_cast<int>(i)));
     bound_ = true;
 }
@@ -183,7 +185,7 @@ Tensor Model::forward(const StepBatch& batch, Runtime& rt) {
     rt.stream_has_bf16 = false;
     rt.head_best = HeadBest{};
     if (!embedding_->takes_step_prologue()) rt.flush_prologue();
-    embedding_->forward(batch.token_ids, h, rt, &batch);
+    embedding_->forward(batch.token_ids, h, rt, &batch, embedding_cache_);
     rt.flush_prologue();      // (an embedding that said it would and did not)
     rt.mark("embedding");
     Tensor delta;

@@ -52,6 +52,7 @@ private:
     std::unique_ptr<Norm> final_norm_;
     std::unique_ptr<Head> head_;
     std::vector<LayerCache> caches_;
+    LayerCache embedding_cache_;
     bool bound_ = false, graph_safe_ = false;
 };
 

@@ -62,6 +62,9 @@ const char* path_name(Path p) {
         case Path::AttentionBiasedRows: return "attention_biased_rows";
         case Path::AttentionBiasedDecode: return "attention_biased_decode";
         case Path::ChannelScan: return "channel_scan";
+        case Path::MatrixMemory: return "matrix_memory";
+        case Path::MatrixMemoryRows: return "matrix_memory_rows";
+        case Path::MatrixMemoryStep: return "matrix_memory_step";
         case Path::LinearRecurrentUnit: return "linear_recurrent_unit";
         case Path::RoutedExperts: return "routed_experts";
         case Path::LinearF32: return "linear_f32";
@@ -98,6 +101,35 @@ void Ops::embed(const Tensor& table, const int* token_ids, const Tensor& out, fl
     need(table.ndim == 2 && out.ndim == 2 && table.shape[1] == out.shape[1] && table.contiguous(), "embed: shapes do not fit");
     kernel_check(celeg_embed(table.data, dt(table, "table"), token_ids, out.as<float>(), static_cast<int>(out.shape[0]),
                              static_cast<int>(out.shape[1]), static_cast<int>(table.shape[0]), scale, stream), "embed");
+}
+
+void Ops::embed_pairs(const Tensor& table, const Tensor& pairs, const PairRule& rule, const Tensor& last, const StepBatch& batch,
+                      const Tensor& out, const Tensor* xb, const Tensor* stats) {
+    dev(table, "table");
+    dev(pairs, "pairs", table.dtype);
+    dev(last, "last", DType::I32, false);
+    dev(out, "out", DType::F32);
+    const long long rows = out.shape[0], width = out.shape[1];
+    need(table.ndim == 2 && pairs.ndim == 2 && out.ndim == 2 && table.shape[1] == width && pairs.shape[1] == width && table.contiguous() &&
+             rows == batch.n_tokens, "embed_pairs: shapes do not fit");
+    need(rule.buckets > 0 && pairs.shape[0] == rule.buckets + 1, "embed_pairs: the table of pairs has a row per bucket and one more");
+    need(last.ndim == 2 && last.shape[1] == 1, "embed_pairs: last is [slots, 1]");
+    Operand o{};
+    if (xb) {
+        need(stats != nullptr, "embed_pairs: the stream's copy goes with its sums of squares");
+        dev(*xb, "xb", DType::BF16, false);
+        o = operand(*xb, "xb");
+        need(o.rows == rows && o.width == width, "embed_pairs: xb does not fit");
+    }
+    if (stats) {
+        dev(*stats, "stats", DType::F32);
+        need(stats->shape[0] >= rows, "embed_pairs: stats do not fit");
+    }
+    kernel_check(celeg_embed_pairs(table.data, pairs.data, dt(table, "table"), batch.token_ids, batch.positions, batch.token_seq,
+                                   batch.cu_seqlens, batch.token_slot, last.as<int>(), static_cast<size_t>(last.stride[0]), rule.buckets,
+                                   rule.mul_prev, rule.mul_cur, out.as<float>(), xb ? xb->data : nullptr, static_cast<int>(o.ld), o.k8,
+                                   stats ? stats->as<float>() : nullptr, stats ? static_cast<int>(stats->stride[0]) : 0,
+                                   static_cast<int>(rows), static_cast<int>(width), static_cast<int>(table.shape[0]), stream), "embed_pairs");
 }
 
 void Ops::scale(const Tensor& x, float factor) {
@@ -167,13 +199,13 @@ static void latent_cache_fits(const Ops::LatentShape& s, const KVView& kv, DType
 
 void Ops::latent_prepare(const Tensor& proj, int q_off, int dkv_off, const LatentShape& s, const Tensor& norm_weight,
                          float eps, const Tensor* inv_freq, int rotary_dim, int pairing, bool write, const StepBatch& batch,
-                         const KVView& kv) {
+                         const KVView& kv, int cq_off, const Tensor* cq_weight, const Tensor* cq) {
     dev(proj, "proj");
     dev(norm_weight, "norm_weight", DType::F32);
     const int ld = rows_of(proj, "proj");
     need(s.heads > 0 && s.dim > 0 && s.rot >= 0 && s.rank > 0, "latent_prepare: sizes must be positive");
     need(proj.shape[0] == batch.n_tokens, "latent_prepare: one row per token of the step");
-    need(q_off >= 0 && q_off + static_cast<long long>(s.heads) * (s.dim + s.rot) <= proj.shape[1] && dkv_off >= 0 &&
+    need((q_off < 0 || q_off + static_cast<long long>(s.heads) * (s.dim + s.rot) <= proj.shape[1]) && dkv_off >= 0 &&
              dkv_off + s.rank + s.rot <= proj.shape[1], "latent_prepare: the queries or the compressed part lie outside the rows");
     need(norm_weight.numel() == s.rank, "latent_prepare: the norm's weight must have `rank` entries");
     need(rotary_dim >= 0 && rotary_dim % 2 == 0 && rotary_dim <= s.rot, "latent_prepare: rotary_dim must be even and at most rot");
@@ -182,16 +214,26 @@ void Ops::latent_prepare(const Tensor& proj, int q_off, int dkv_off, const Laten
         dev(*inv_freq, "inv_freq", DType::F32);
         need(inv_freq->numel() == rotary_dim / 2, "latent_prepare: one frequency per rotated pair");
     }
+    int q_rank = 0;
+    if (cq) {
+        need(cq_weight != nullptr, "latent_prepare: the compressed queries need their norm's weight");
+        dev(*cq, "cq", proj.dtype);
+        dev(*cq_weight, "cq_weight", DType::F32);
+        q_rank = static_cast<int>(cq->shape[1]);
+        need(cq->ndim == 2 && cq->shape[0] == batch.n_tokens && q_rank > 0 && cq_weight->numel() == q_rank && cq_off >= 0 &&
+                 cq_off + q_rank <= proj.shape[1], "latent_prepare: the compressed queries do not fit");
+    }
     latent_cache_fits(s, kv, proj.dtype, "latent_prepare");
     kernel_check(celeg_latent_prepare(proj.data, ld, dt(proj, "proj"), q_off, dkv_off, s.heads, s.dim, s.rot, s.rank,
                                       norm_weight.as<float>(), eps, inv_freq && rotary_dim > 0 ? inv_freq->as<float>() : nullptr,
                                       rotary_dim, pairing, batch.positions, batch.token_slot, kv.table, kv.table_stride, kv.k,
-                                      kv.n_layers, kv.layer, kv.page_tokens, write ? 1 : 0, batch.n_tokens, stream),
+                                      kv.n_layers, kv.layer, kv.page_tokens, write ? 1 : 0, batch.n_tokens, cq_off, q_rank,
+                                      q_rank ? cq_weight->as<float>() : nullptr, q_rank ? cq->data : nullptr, stream),
                  "latent_prepare");
 }
 
 void Ops::headwise_linear(const Tensor& x, int x_head, const Tensor& w, const Tensor& out, int o_head, int tail,
-                          const Tensor* gate) {
+                          const Tensor* gate, const TailTurn* turn) {
     dev(x, "x");
     dev(w, "w", x.dtype);
     dev(out, "out", x.dtype, false);
@@ -207,16 +249,25 @@ void Ops::headwise_linear(const Tensor& x, int x_head, const Tensor& w, const Te
         ldg = rows_of(*gate, "gate");
         need(gate->shape[0] == x.shape[0] && gate->shape[1] == heads * N, "headwise_linear: gate must be [rows, heads * N]");
     }
+    const bool turns = turn && turn->inv_freq && turn->rotary_dim > 0;
+    if (turns) {
+        dev(*turn->inv_freq, "inv_freq", DType::F32);
+        need(turn->rotary_dim % 2 == 0 && turn->rotary_dim <= tail && turn->inv_freq->numel() == turn->rotary_dim / 2 && turn->positions,
+             "headwise_linear: the turned values must be pairs inside the tail, with a frequency each and the rows' positions");
+    }
     const bool cores = moe_matrix_cores_ok(x.dtype, N, K) && ldx % 8 == 0 && x_head % 8 == 0 && ldo % 4 == 0 && o_head % 4 == 0 &&
                        reinterpret_cast<uintptr_t>(x.data) % 16 == 0 && reinterpret_cast<uintptr_t>(out.data) % 8 == 0;
     kernel_check(celeg_headwise_linear(x.data, ldx, x_head, w.data, dt(x, "x"), static_cast<int>(heads), static_cast<int>(N),
                                        static_cast<int>(K), out.data, ldo, o_head, tail, gate ? gate->data : nullptr, ldg,
-                                       static_cast<int>(x.shape[0]), cores ? 1 : 0, stream), "headwise_linear");
+                                       static_cast<int>(x.shape[0]), cores ? 1 : 0, turns ? turn->inv_freq->as<float>() : nullptr,
+                                       turns ? turn->rotary_dim : 0, turns ? turn->pairing : 0, turns ? turn->positions : nullptr, stream),
+                 "headwise_linear");
 }
 
 void Ops::latent_attention(const Tensor& q_lat, const Tensor& out, const LatentShape& s, float scale, const Tensor* sink,
-                           const StepBatch& batch, const KVView& kv, Workspace& ws) {
+                           const StepBatch& batch, const KVView& kv, Workspace& ws, int window) {
     dev(q_lat, "q_lat");
+    need(window >= 0, "latent_attention: the window is not negative");
     dev(out, "out", q_lat.dtype);
     const int D = s.rank + s.rot;
     need(q_lat.ndim == 2 && q_lat.contiguous() && q_lat.shape[0] == batch.n_tokens && q_lat.shape[1] == static_cast<long long>(s.heads) * D,
@@ -236,7 +287,9 @@ void Ops::latent_attention(const Tensor& q_lat, const Tensor& out, const LatentS
         const float* sink_p = sink ? sink->as<float>() : nullptr;
         if (n_single > 0) {
             // single tokens: the keys of a row in shares, so that the chip is busy whatever the batch
-            const int blocks = (std::max(hint_of(batch, kv), 1) + 63) / 64;
+            // (a window lies over at most (window + 62) / 64 + 1 blocks)
+            int blocks = (std::max(hint_of(batch, kv), 1) + 63) / 64;
+            if (window > 0) blocks = std::min(blocks, (window + 62) / 64 + 1);
             const int groups = n_single * ((s.heads + 15) / 16);
             // (at most 64 shares, and a share is at least latent_decode_min_blocks blocks of 64 keys where there are that many)
             int n_splits = std::clamp(latent_decode_workgroups / std::max(groups, 1), 1, std::min(64, std::max(1, blocks / std::max(latent_decode_min_blocks, 1))));
@@ -250,7 +303,7 @@ void Ops::latent_attention(const Tensor& q_lat, const Tensor& out, const LatentS
                                                      batch.cu_seqlens, batch.seq_slot, batch.seq_start, batch.n_seqs, 0,
                                                      batch.token_slot, batch.positions, n_single, sink_p, out.data,
                                                      static_cast<int>(out.shape[1]), ws_o, ws_ml, n_splits, per_split, s.heads,
-                                                     s.rank, s.rot, kv.page_tokens, kv.n_layers, kv.layer, scale, stream),
+                                                     s.rank, s.rot, kv.page_tokens, kv.n_layers, kv.layer, scale, window, stream),
                          "latent_attention (single tokens)");
         }
         if (T > n_single) {
@@ -260,7 +313,7 @@ void Ops::latent_attention(const Tensor& q_lat, const Tensor& out, const LatentS
                                                      batch.cu_seqlens, batch.seq_slot, batch.seq_start, batch.n_seqs, max_tiles,
                                                      batch.token_slot, batch.positions, 0, sink_p, out.data,
                                                      static_cast<int>(out.shape[1]), nullptr, nullptr, 1, 0, s.heads, s.rank,
-                                                     s.rot, kv.page_tokens, kv.n_layers, kv.layer, scale, stream),
+                                                     s.rot, kv.page_tokens, kv.n_layers, kv.layer, scale, window, stream),
                          "latent_attention (rows)");
         }
         return;
@@ -268,7 +321,7 @@ void Ops::latent_attention(const Tensor& q_lat, const Tensor& out, const LatentS
     kernel_check(celeg_latent_attention(q_lat.data, static_cast<int>(q_lat.shape[1]), kv.k, dt(q_lat, "q_lat"), kv.table,
                                         kv.table_stride, batch.token_slot, batch.positions, sink ? sink->as<float>() : nullptr,
                                         out.data, static_cast<int>(out.shape[1]), batch.n_tokens, s.heads, s.rank, s.rot,
-                                        kv.page_tokens, kv.n_layers, kv.layer, scale, stream), "latent_attention");
+                                        kv.page_tokens, kv.n_layers, kv.layer, scale, window, stream), "latent_attention");
 }
 
 // ---------------------------------------------------------------------------- routed experts
@@ -944,6 +997,51 @@ void Ops::channel_scan(const Tensor& qk, const Tensor& v, const Tensor& decay, c
                                     batch.n_seqs, s.kv_heads, s.heads, s.dim, s.vdim, delta_general ? 1 : 0, stream), "channel_scan");
 }
 
+// ---------------------------------------------------------------------------- matrix memory
+void Ops::matrix_memory(const Tensor& proj, const MemoryColumns& at, const MemoryShape& s, const Tensor& bias_i, const Tensor& bias_f,
+                        const Tensor& norm, const Tensor& S, const Tensor& n, const Tensor& m, const Tensor& out, const StepBatch& batch,
+                        Workspace& ws) {
+    dev(proj, "proj");
+    dev(bias_i, "bias_i", DType::F32);
+    dev(bias_f, "bias_f", DType::F32);
+    dev(norm, "norm", DType::F32);
+    dev(out, "out", proj.dtype, false);
+    const long long T = batch.n_tokens, H = s.heads, D = s.dim, V = s.vdim;
+    need(H > 0 && D > 0 && V > 0 && D <= 256 && V <= 512, "matrix_memory: heads positive, dim up to 256, vdim up to 512");
+    need(s.gate_cap > 0.f && s.eps > 0.f, "matrix_memory: gate_cap and eps must be positive");
+    need(proj.ndim == 2 && proj.shape[0] == T && out.ndim == 2 && out.shape[0] == T && out.shape[1] == H * V, "matrix_memory: rows do not fit");
+    auto inside = [&](long long col, long long n_cols) { return col >= 0 && col + n_cols <= proj.shape[1]; };
+    need(inside(at.q, H * D) && inside(at.k, H * D) && inside(at.v, H * V) && inside(at.g, H * V) && inside(at.i, H) && inside(at.f, H),
+         "matrix_memory: a projection lies outside the rows");
+    need(bias_i.numel() == H && bias_f.numel() == H && norm.numel() == H * V, "matrix_memory: biases per head, a norm weight per value");
+    auto fits = [&](const Tensor& t, const char* name, long long per_slot) {
+        dev(t, name, DType::F32, false);
+        need(t.ndim >= 2 && t.numel() / t.shape[0] == per_slot && t.stride[t.ndim - 1] == 1, std::string("matrix_memory: state ") + name + " does not fit");
+    };
+    fits(S, "S", H * D * V);
+    fits(n, "n", H * D);
+    fits(m, "m", H);
+    const int n_single = std::min(batch.single_rows, batch.n_seqs), portions = batch.n_seqs - n_single;
+    float *planes = nullptr, *chunk_s = nullptr, *chunk_n = nullptr;
+    int max_chunks = 0;
+    took(Path::MatrixMemory);
+    if (n_single > 0) took(Path::MatrixMemoryStep);
+    if (portions > 0) {
+        took(Path::MatrixMemoryRows);
+        max_chunks = static_cast<int>(T - n_single) / 64 + portions;
+        planes = static_cast<float*>(ws.raw("memory_gates", static_cast<size_t>(6) * H * T * sizeof(float)));
+        chunk_s = static_cast<float*>(ws.raw("memory_chunks", static_cast<size_t>(max_chunks) * H * D * V * sizeof(float)));
+        chunk_n = static_cast<float*>(ws.raw("memory_chunk_norms", static_cast<size_t>(max_chunks) * H * D * sizeof(float)));
+    }
+    kernel_check(celeg_matrix_memory(proj.data, rows_of(proj, "proj"), dt(proj, "proj"), static_cast<int>(at.q), static_cast<int>(at.k),
+                                     static_cast<int>(at.v), static_cast<int>(at.g), static_cast<int>(at.i), static_cast<int>(at.f),
+                                     bias_i.as<float>(), bias_f.as<float>(), norm.as<float>(), S.as<float>(), static_cast<size_t>(S.stride[0]),
+                                     n.as<float>(), static_cast<size_t>(n.stride[0]), m.as<float>(), static_cast<size_t>(m.stride[0]),
+                                     batch.cu_seqlens, batch.seq_slot, batch.token_slot, planes, chunk_s, chunk_n, out.data, rows_of(out, "out"),
+                                     static_cast<int>(T), batch.n_seqs, n_single, max_chunks, s.heads, s.dim, s.vdim, s.gate_cap, s.eps, stream),
+                 "matrix_memory");
+}
+
 // ---------------------------------------------------------------------------- linear recurrent unit
 void Ops::lru_gates(const Tensor& x, const Tensor& conv_w, const Tensor* conv_b, const Tensor& ra_t, const Tensor& ra_b,
                     const Tensor& ri_t, const Tensor& ri_b, const Tensor& lam, const Tensor& conv_state, const Tensor& decay,
@@ -1009,7 +1107,7 @@ static void check_kv_wide(const KVView& kv, int kv_heads, int head_dim, int v_di
     need(kv.layer >= 0 && kv.layer < kv.n_layers, std::string(who) + ": layer index outside the cache");
 }
 
-void Ops::kv_store(const Tensor& k, const Tensor& v, const StepBatch& batch, const KVView& kv) {
+void Ops::kv_store(const Tensor& k, const Tensor& v, const StepBatch& batch, const KVView& kv, float v_eps) {
     dev(k, "k");
     dev(v, "v", k.dtype, false);
     check_kv_wide(kv, kv.kv_heads, kv.head_dim, kv.v_head_dim, k.dtype, "kv_store");
@@ -1020,11 +1118,11 @@ void Ops::kv_store(const Tensor& k, const Tensor& v, const StepBatch& batch, con
          "kv_store: k [rows, kv_heads * head_dim], v [rows, kv_heads * v_dim]");
     kernel_check(celeg_kv_store(k.data, rows_of(k, "k"), v.data, rows_of(v, "v"), dt(k, "k"), kv.k, kv.v, kv.table, kv.table_stride,
                                 batch.token_slot, batch.positions, static_cast<int>(T), kv.kv_heads, kv.head_dim, kv.v_head_dim,
-                                kv.page_tokens, kv.n_layers, kv.layer, stream), "kv_store");
+                                kv.page_tokens, kv.n_layers, kv.layer, v_eps, stream), "kv_store");
 }
 
 void Ops::biased_attention(const Tensor& q, const Tensor& out, const ScoreShape& s, const Tensor* r1, const Tensor* r2,
-                           const Tensor* gate, const StepBatch& batch, const KVView& kv, Workspace& ws) {
+                           const Tensor* gate, const StepBatch& batch, const KVView& kv, Workspace& ws, const Tensor* sink) {
     dev(q, "q");
     dev(out, "out", q.dtype, false);
     need(s.heads > 0 && s.kv_heads > 0 && s.heads % s.kv_heads == 0 && s.head_dim > 0 && s.v_dim > 0,
@@ -1043,6 +1141,12 @@ void Ops::biased_attention(const Tensor& q, const Tensor& out, const ScoreShape&
     }
     need(s.every >= 0 && s.window >= 0 && s.keep_first >= 0, "biased_attention: every, window and keep_first are not negative");
     const int keep_first = s.window > 0 ? s.keep_first : 0, sink_one = s.sink_one ? 1 : 0;
+    need(s.softcap >= 0.f, "biased_attention: the softcap is not negative");
+    if (sink) {
+        dev(*sink, "sink", DType::F32);
+        need(sink->numel() == s.heads && !s.sink_one, "biased_attention: one sink per head, and no other extra term");
+    }
+    const float* sink_at = sink ? sink->as<float>() : nullptr;
     if (gate) {
         dev(*gate, "gate", q.dtype, false);
         need(gate->ndim == 2 && gate->shape[0] == T && gate->shape[1] == out.shape[1], "biased_attention: gate [rows, heads * v_dim]");
@@ -1064,14 +1168,14 @@ void Ops::biased_attention(const Tensor& q, const Tensor& out, const ScoreShape&
                                                  batch.seq_start, batch.n_seqs, max_tiles, r1 ? r1->as<float>() : nullptr,
                                                  r2 ? r2->as<float>() : nullptr, gate ? gate->data : nullptr, ldg, out.data, ldo, s.heads,
                                                  s.kv_heads, s.head_dim, s.v_dim, kv.page_tokens, kv.n_layers, kv.layer, s.scale, s.coef,
-                                                 s.every, s.window, keep_first, sink_one, stream), "biased attention (bfloat16, matrix cores)");
+                                                 s.every, s.window, keep_first, sink_one, sink_at, s.softcap, stream), "biased attention (bfloat16, matrix cores)");
         return;
     }
     kernel_check(celeg_biased_attention(q.data, rows_of(q, "q"), dt(q, "q"), kv.k, kv.v, kv.table, kv.table_stride, batch.token_slot,
                                         batch.positions, r1 ? r1->as<float>() : nullptr, r2 ? r2->as<float>() : nullptr,
                                         gate ? gate->data : nullptr, gate ? rows_of(*gate, "gate") : 0, out.data, rows_of(out, "out"),
                                         static_cast<int>(T), s.heads, s.kv_heads, s.head_dim, s.v_dim, kv.page_tokens, kv.n_layers,
-                                        kv.layer, s.scale, s.coef, s.every, s.window, keep_first, sink_one, stream), "biased_attention");
+                                        kv.layer, s.scale, s.coef, s.every, s.window, keep_first, sink_one, sink_at, s.softcap, stream), "biased_attention");
 }
 
 void Ops::conv_rope_store(const Tensor& proj, const Tensor* conv_w, const Tensor* conv_state, int taps, const Tensor* inv_freq,
@@ -1137,17 +1241,17 @@ void Ops::softcap(const Tensor& x, float cap) {
 }
 
 // ---------------------------------------------------------------------------- layer glue
-void Ops::activation_bias(const Tensor& x, const Tensor* bias, const Tensor& out, int act) {
+void Ops::activation_bias(const Tensor& x, const Tensor* bias, const Tensor& out, int act, float p0, float p1) {
     dev(x, "x");
     dev(out, "out", x.dtype, false);
     need(x.ndim == 2 && out.ndim == 2 && x.shape[0] == out.shape[0] && x.shape[1] == out.shape[1], "activation_bias: x and out differ");
-    need(act >= 0 && act <= 2, "activation_bias: act is 0 (gelu), 1 (square of relu) or 2 (none)");
+    need(act >= 0 && act <= 3, "activation_bias: act is 0 (gelu), 1 (square of relu), 2 (none) or 3 (square and exponential)");
     if (bias) {
         dev(*bias, "bias", DType::F32);
         need(bias->numel() == x.shape[1], "activation_bias: one bias per column");
     }
     kernel_check(celeg_activation_bias(x.data, rows_of(x, "x"), bias ? bias->as<float>() : nullptr, out.data, rows_of(out, "out"),
-                                       dt(x, "x"), static_cast<int>(x.shape[0]), static_cast<int>(x.shape[1]), act, stream),
+                                       dt(x, "x"), static_cast<int>(x.shape[0]), static_cast<int>(x.shape[1]), act, p0, p1, stream),
                  "activation_bias");
 }
 

@@ -102,7 +102,7 @@ struct StepPrologue {
 // graph records; a replay counts nothing): what tests and tools ask to see that a size took the
 // path it was meant to take.
 enum class Path : int {
-    AttentionDecode = 0, AttentionDecodeFresh, AttentionRows, AttentionGeneral, AttentionSigmoid, AttentionSigmoidRows, AttentionSigmoidDecode, DeltaRule, AttentionLatent, AttentionLatentRows, AttentionLatentDecode, AttentionBiased, AttentionBiasedRows, AttentionBiasedDecode, ChannelScan, LinearRecurrentUnit, RoutedExperts, LinearF32, LinearLibrary, LinearStandIn,
+    AttentionDecode = 0, AttentionDecodeFresh, AttentionRows, AttentionGeneral, AttentionSigmoid, AttentionSigmoidRows, AttentionSigmoidDecode, DeltaRule, AttentionLatent, AttentionLatentRows, AttentionLatentDecode, AttentionBiased, AttentionBiasedRows, AttentionBiasedDecode, ChannelScan, MatrixMemory, MatrixMemoryRows, MatrixMemoryStep, LinearRecurrentUnit, RoutedExperts, LinearF32, LinearLibrary, LinearStandIn,
     FusedSliced, FusedRows, FusedStaged, Tiled, TiledQkv, ArgmaxMerged, Count
 };
 const char* path_name(Path p);
@@ -142,6 +142,12 @@ public:
 
     // row-wise
     void embed(const Tensor& table, const int* token_ids, const Tensor& out, float scale = 1.0f);
+    // out = table[id] + pairs[(previous id * mul_prev + id * mul_cur) mod buckets], a sequence's first token taking the
+    // last row of pairs [buckets + 1, width]; last [slots, 1] int32 keeps every request's last token.  xb and
+    // stats (or null) as for embed_stream.
+    struct PairRule { long long buckets = 0, mul_prev = 0, mul_cur = 0; };
+    void embed_pairs(const Tensor& table, const Tensor& pairs, const PairRule& rule, const Tensor& last, const StepBatch& batch,
+                     const Tensor& out, const Tensor* xb, const Tensor* stats);
     void scale(const Tensor& x, float factor);     // x *= factor, 32-bit x
     // several residual streams: xs [rows, streams * width] 32-bit
     void streams_spread(const Tensor& h, const Tensor& xs, int streams);
@@ -239,12 +245,14 @@ public:
     // f(i) = 1 + coef ln(floor((i + 1) / every) + 1) (every 0: f = 1); r1, r2 [heads] 32-bit or null.  Values of kv.v_head_dim.
     // gate: raw values [rows, heads * v_dim] (a view with dense rows) whose sigmoid multiplies the result, or null.
     // With a window, `keep_first` keys at the start of the sequence stay visible however far the window has moved;
-    // `sink_one`: the softmax's denominator holds a one more (a key of score 0 that has no value).
+    // The softmax's denominator may hold one more term, a key that has no value: of score 0 (`sink_one`), or of the
+    // head's own number in sink [heads] (neither scaled nor bent).  softcap c > 0 bends a scaled score s to c tanh(s / c).
     struct ScoreShape {
         int heads = 0, kv_heads = 0, head_dim = 0, v_dim = 0, window = 0, every = 0;
         float scale = 1.f, coef = 0.f;
         int keep_first = 0;
         bool sink_one = false;
+        float softcap = 0.f;
     };
     // What lies between an attention's q/k/v product and its scores where the projected channels pass a short causal
     // convolution: proj [rows, >= (heads + kv_heads) * head_dim + kv_heads * v_dim] holds q | k | v from column 0;
@@ -253,13 +261,23 @@ public:
     // the queries go to q_out [rows, heads * head_dim], keys and values to the rows' places in the pages.
     void conv_rope_store(const Tensor& proj, const Tensor* conv_w, const Tensor* conv_state, int taps, const Tensor* inv_freq,
                          int rotary_dim, int pairing, const Tensor& q_out, int heads, const StepBatch& batch, const KVView& kv);
-    // a step's keys [rows, kv_heads * head_dim] and values [rows, kv_heads * v_dim] to their places in the pages
-    void kv_store(const Tensor& k, const Tensor& v, const StepBatch& batch, const KVView& kv);
+    // a step's keys [rows, kv_heads * head_dim] and values [rows, kv_heads * v_dim] to their places in the pages;
+    // v_eps > 0: every head's value divided by sqrt(mean(v^2) + v_eps)
+    void kv_store(const Tensor& k, const Tensor& v, const StepBatch& batch, const KVView& kv, float v_eps = 0.f);
     void biased_attention(const Tensor& q, const Tensor& out, const ScoreShape& shape, const Tensor* r1, const Tensor* r2,
-                          const Tensor* gate, const StepBatch& batch, const KVView& kv, Workspace& ws);
+                          const Tensor* gate, const StepBatch& batch, const KVView& kv, Workspace& ws, const Tensor* sink = nullptr);
+    // The matrix memory (mLSTM) behind its one projection: proj [rows, ...] holds q, k (heads x dim), v, g (heads x
+    // vdim) and the gates' inputs i, f (heads) at the given columns; states S [slots, heads, dim, vdim], n [slots, heads,
+    // dim], m [slots, heads] 32-bit; out [rows, heads * vdim] is normed, weighted and gated.
+    struct MemoryShape { int heads = 0, dim = 0, vdim = 0; float gate_cap = 1.f, eps = 1e-6f; };
+    struct MemoryColumns { long long q = 0, k = 0, v = 0, g = 0, i = 0, f = 0; };
+    void matrix_memory(const Tensor& proj, const MemoryColumns& at, const MemoryShape& shape, const Tensor& bias_i, const Tensor& bias_f,
+                       const Tensor& norm, const Tensor& S, const Tensor& n, const Tensor& m, const Tensor& out, const StepBatch& batch,
+                       Workspace& ws);
     // layer glue (32-bit arithmetic; rows of the run's dtype)
-    // out = act(x + bias): act 0 gelu (tanh form), 1 square of relu, 2 none; x and out views with dense rows
-    void activation_bias(const Tensor& x, const Tensor* bias, const Tensor& out, int act);
+    // out = act(x + bias): act 0 gelu (tanh form), 1 square of relu, 2 none, 3 p0 z^2 + z / 2 for z > 0 and
+    // p1 (exp(z) - 1 - z) + z / 2 else; x and out views with dense rows
+    void activation_bias(const Tensor& x, const Tensor* bias, const Tensor& out, int act, float p0 = 0.f, float p1 = 0.f);
     // h += a (+ b), h the 32-bit stream; copy (or null) receives the new rows in the run's dtype
     void residual_sum(const Tensor& h, const Tensor& a, const Tensor* b, const Tensor* copy);
     // g[t, j] = gelu_tanh(z[t, j]) * table[token[t], offset + j]
@@ -276,18 +294,22 @@ public:
     struct LatentShape { int heads = 0, dim = 0, rot = 0, rank = 0; };
     // proj [rows, ...] holds the queries [heads, dim + rot] from column q_off and (dkv) [rank + rot] from
     // column dkv_off: the queries' rotated parts are turned in place; with `write` the normed
-    // compressed values and the turned key part go to the rows' places in the pages
+    // compressed values and the turned key part go to the rows' places in the pages.  q_off < 0: the rows hold no
+    // queries (they are turned by headwise_linear); cq: the values of proj from column cq_off on, RMS-normed
+    // with cq_weight, go to cq [rows, width].
     void latent_prepare(const Tensor& proj, int q_off, int dkv_off, const LatentShape& shape, const Tensor& norm_weight,
                         float eps, const Tensor* inv_freq, int rotary_dim, int pairing, bool write, const StepBatch& batch,
-                        const KVView& kv);
+                        const KVView& kv, int cq_off = 0, const Tensor* cq_weight = nullptr, const Tensor* cq = nullptr);
     // out[t, h, :N] = w[h] x[t, h, :K] (w [heads, N, K]); `tail` further values of x's head pass unchanged
     // behind them; with gate [rows, heads * N] (a view with dense rows) the result is multiplied by
-    // sigmoid(gate).  x_head / o_head: the distance between heads inside a row of x / out.
+    // sigmoid(gate).  x_head / o_head: the distance between heads inside a row of x / out.  With `turn` the tail's
+    // first rotary_dim values are turned by the rows' positions on the way.
+    struct TailTurn { const Tensor* inv_freq = nullptr; int rotary_dim = 0, pairing = 0; const int* positions = nullptr; };
     void headwise_linear(const Tensor& x, int x_head, const Tensor& w, const Tensor& out, int o_head, int tail,
-                         const Tensor* gate);
-    // q_lat [rows, heads * (rank + rot)] against the pages; out [rows, heads * rank]
+                         const Tensor* gate, const TailTurn* turn = nullptr);
+    // q_lat [rows, heads * (rank + rot)] against the pages; out [rows, heads * rank]; window 0: every earlier key
     void latent_attention(const Tensor& q_lat, const Tensor& out, const LatentShape& shape, float scale, const Tensor* sink,
-                          const StepBatch& batch, const KVView& kv, Workspace& ws);
+                          const StepBatch& batch, const KVView& kv, Workspace& ws, int window = 0);
     // routed experts
     struct RoutePlan {
         Tensor ids, weights;                       // [rows * top]: expert and score of every (row, choice)

@@ -118,6 +118,39 @@ std::shared_ptr<DeviceTensor> maybe(const PartTensors& t, const std::string& rol
 WeightSpec matrix(long long rows, long long cols) { return WeightSpec{{rows, cols}, "matrix", "normal", {}}; }
 WeightSpec vec(long long n, const char* init = "normal") { return WeightSpec{{n}, "vector", init, {}}; }
 
+// ---------------------------------------------------------------------------- projections side by side
+// The matrices of several projections of one input, one under the other, so that one product
+// makes them all.  A piece that a later product reads as its input starts at a multiple of 16
+// rows (zero rows in front of it); the whole is padded to a multiple of 16 rows.
+struct Stacked {
+    std::shared_ptr<DeviceTensor> weight;
+    std::vector<long long> at;        // the first row of every piece
+    long long rows = 0;
+};
+Stacked stack_projections(const std::vector<std::pair<std::shared_ptr<DeviceTensor>, bool>>& pieces, const char* who) {
+    Stacked out;
+    std::vector<std::shared_ptr<DeviceTensor>> parts;
+    const DType dtype = pieces.at(0).first->view.dtype;
+    const long long width = pieces.at(0).first->view.shape[1];
+    auto pad_to_16 = [&]() {
+        const long long pad = (16 - out.rows % 16) % 16;
+        if (pad) parts.push_back(from_host_floats(std::vector<float>(static_cast<size_t>(pad * width), 0.f), dtype, {pad, width}));
+        out.rows += pad;
+    };
+    for (const auto& piece : pieces) {
+        const Tensor& v = piece.first->view;
+        if (v.dtype != dtype || v.ndim != 2 || v.shape[1] != width)
+            throw SpecError(std::string(who) + ": the input projections differ in dtype or inner size");
+        if (piece.second) pad_to_16();
+        out.at.push_back(out.rows);
+        parts.push_back(piece.first);
+        out.rows += v.shape[0];
+    }
+    pad_to_16();
+    out.weight = concat_rows(parts);
+    return out;
+}
+
 // ---------------------------------------------------------------------------- norms
 // RMSNorm: y = x / sqrt(mean(x^2) + eps) * w, eps inside the root, w a plain scale
 // (src/backend/cpu/kernels/elementwise.cpp:56-76; CUDA kernels/norm.cuh:1-44).  The sum of
@@ -439,11 +472,12 @@ private:
 // ---------------------------------------------------------------------------- latent attention
 // Attention whose keys and values are expanded from one compressed row per token.
 //
-// From the mixer's input h: q = W_q h, head by head [dim plain | rot rotated]; W_dkv h gives
+// From the mixer's input h: q = W_q h, head by head [dim plain | rot rotated], or with "q_rank" r through a
+// compressed row of its own, q = W_uq c_q with c_q = W_dq h of r values, RMS-normed with a weight; W_dkv h gives
 // rank + rot values: the first rank, RMS-normed with a weight of their own, are the compressed
 // row c, the last rot are a key part that every head shares and that is rotated by the
 // position, as the queries' rot part is.  Head i's key is (W_uk[i] c | shared part), its value
-// W_uv[i] c; score = (q . k) * scale over positions 0..p; softmax, whose denominator may hold
+// W_uv[i] c; score = (q . k) * scale over positions 0..p (with "window" n the last n of them); softmax, whose denominator may hold
 // one more term exp(sink_i) (a learned number per head with no key and no value); the heads'
 // results, optionally times sigmoid(W_g h), go through W_o.
 //
@@ -464,6 +498,12 @@ public:
         eps_ = static_cast<float>(p.get_double("eps", 1e-6));
         sink_ = p.get_bool("sink", false);
         gate_ = p.get_bool("gate", false);
+        q_rank_ = p.get_int("q_rank", 0);
+        if (q_rank_ < 0) throw SpecError("latent_attention: q_rank is not negative");
+        if (!p["window"].is_null()) {
+            window_ = static_cast<int>(p["window"].as_int());
+            if (window_ <= 0) throw SpecError("latent_attention: window must be positive");
+        }
         if (width_ <= 0 || shape_.heads <= 0 || shape_.dim <= 0 || shape_.rot < 0 || shape_.rank <= 0 || vdim_ <= 0)
             throw SpecError("latent_attention: width, heads, dim, kv_rank and vdim must be positive");
         scale_ = p["scale"].is_null() ? static_cast<float>(1.0 / std::sqrt(static_cast<double>(shape_.dim + shape_.rot)))
@@ -480,24 +520,38 @@ public:
         need.kv_heads = 1;
         need.head_dim = shape_.rank + shape_.rot;
         need.keys_only = true;
+        if (window_ > 0) need.window = window_;
         return need;
     }
     WeightSpecs weight_specs() const override {
         const long long H = shape_.heads, qd = shape_.dim + shape_.rot;
-        WeightSpecs specs{{"q", matrix(H * qd, width_)},          {"dkv", matrix(shape_.rank + shape_.rot, width_)},
+        WeightSpecs specs{{"dkv", matrix(shape_.rank + shape_.rot, width_)},
                           {"dkv_norm", vec(shape_.rank, "around_one")}, {"uk", matrix(H * shape_.dim, shape_.rank)},
                           {"uv", matrix(H * vdim_, shape_.rank)},  {"o", matrix(width_, H * vdim_)}};
+        if (q_rank_ > 0) {
+            specs.push_back({"dq", matrix(q_rank_, width_)});
+            specs.push_back({"dq_norm", vec(q_rank_, "around_one")});
+            specs.push_back({"uq", matrix(H * qd, q_rank_)});
+        } else {
+            specs.push_back({"q", matrix(H * qd, width_)});
+        }
         if (sink_) specs.push_back({"sink", vec(H)});
         if (gate_) specs.push_back({"g", matrix(H * vdim_, width_)});
         return specs;
     }
     void load(const PartTensors& t, Runtime&) override {
-        // q, dkv and the gate read the same rows: one product
-        std::vector<std::shared_ptr<DeviceTensor>> in{get(t, "q"), get(t, "dkv")};
-        if (gate_) in.push_back(get(t, "g"));
-        for (const auto& w : in)
-            if (w->view.dtype != in[0]->view.dtype) throw SpecError("latent_attention: the input projections are stored in different dtypes");
-        w_in_ = concat_rows(in);
+        // q (or its compressed row), dkv and the gate read the same rows: one product
+        std::vector<std::pair<std::shared_ptr<DeviceTensor>, bool>> pieces{{get(t, q_rank_ > 0 ? "dq" : "q"), false}, {get(t, "dkv"), false}};
+        if (gate_) pieces.push_back({get(t, "g"), false});
+        const Stacked in = stack_projections(pieces, "latent_attention");
+        w_in_ = in.weight;
+        col_dkv_ = in.at[1];
+        col_g_ = gate_ ? in.at[2] : 0;
+        if (q_rank_ > 0) {
+            w_uq_ = get(t, "uq");
+            dq_norm_ = get(t, "dq_norm");
+            if (w_uq_->view.dtype != w_in_->view.dtype) throw SpecError("latent_attention: the query projections are stored in different dtypes");
+        }
         w_o_ = get(t, "o");
         dkv_norm_ = get(t, "dkv_norm");
         if (sink_) sink_w_ = get(t, "sink");
@@ -515,37 +569,66 @@ public:
         uv_view_ = Tensor::make(uv->view.data, uv->view.dtype, {H, vdim_, rank});
     }
     Tensor forward(const Tensor& x, const StepBatch& batch, const LayerCache& cache, Runtime& rt) override {
+        Tensor heads = project_and_attend(x, nullptr, batch, cache, rt);
+        Tensor out = rt.ws.buf("mixer_out", rt.dtype, {x.shape[0], width_});
+        rt.ops.linear(heads, w_o_->view, out, nullptr, rt.ws);
+        return out;
+    }
+    // h += mixer(norm(h)) with the norm folded into the one product in front and the sum into the one behind
+    bool forward_fused(const Tensor& h, const Norm::Foldable& norm, const StepBatch& batch, const LayerCache& cache,
+                       Runtime& rt) override {
+        if (!fused::fused_rows_ok(rt, batch, {width_, static_cast<long long>(shape_.heads) * vdim_}) || w_in_->view.dtype != rt.dtype ||
+            w_o_->view.dtype != rt.dtype)
+            return false;
+        Tensor heads = project_and_attend(h, &norm, batch, cache, rt);
+        fused::linear_into_stream(rt, heads, w_o_->view, h);
+        return true;
+    }
+
+private:
+    // norm null: x are normalised rows; else x is the stream and the norm is applied inside the product
+    Tensor project_and_attend(const Tensor& x, const Norm::Foldable* norm, const StepBatch& batch, const LayerCache& cache, Runtime& rt) {
         if (!cache.kv) throw SpecError("latent_attention: the cache has no rows for this layer");
         if (!cache.writes_kv) throw SpecError("latent_attention: reading another entry's cache is not supported");
         const long long T = x.shape[0], H = shape_.heads;
         const long long qd = shape_.dim + shape_.rot, D = shape_.rank + shape_.rot;
-        const long long q_cols = H * qd, dkv_cols = D, g_cols = gate_ ? H * vdim_ : 0;
-        Tensor proj = rt.ws.buf("latent_proj", rt.dtype, {T, q_cols + dkv_cols + g_cols});
-        rt.ops.linear(x, w_in_->view, proj, nullptr, rt.ws);
+        const long long q_cols = H * qd, g_cols = gate_ ? H * vdim_ : 0;
+        Tensor proj = rt.ws.buf("latent_proj", rt.dtype, {T, w_in_->view.shape[0]});
+        if (norm) fused::norm_linear(rt, x, *norm, w_in_->view, proj, Epilogue::Store);
+        else rt.ops.linear(x, w_in_->view, proj, nullptr, rt.ws);
         const PositionEncoding::Tables tables = position_->tables(rt);
         const Tensor* inv_freq = tables.inv_freq.defined() ? &tables.inv_freq : nullptr;
-        rt.ops.latent_prepare(proj, 0, static_cast<int>(q_cols), shape_, dkv_norm_->view, eps_, inv_freq,
-                              inv_freq ? tables.rotary_dim : 0, tables.pairing, true, batch, *cache.kv);
         Tensor q_lat = rt.ws.buf("latent_q", rt.dtype, {T, H * D});
-        rt.ops.headwise_linear(proj.cols(0, q_cols), static_cast<int>(qd), w_uk_t_->view, q_lat, static_cast<int>(D), shape_.rot, nullptr);
+        if (q_rank_ > 0) {
+            // the two norms and the cache write in one kernel; the queries' rotated parts turn as they pass by W_uk
+            Tensor cq = rt.ws.buf("latent_cq", rt.dtype, {T, q_rank_});
+            rt.ops.latent_prepare(proj, -1, static_cast<int>(col_dkv_), shape_, dkv_norm_->view, eps_, inv_freq,
+                                  inv_freq ? tables.rotary_dim : 0, tables.pairing, true, batch, *cache.kv, 0, &dq_norm_->view, &cq);
+            Tensor q = rt.ws.buf("latent_uq", rt.dtype, {T, q_cols});
+            rt.ops.linear(cq, w_uq_->view, q, nullptr, rt.ws);
+            Ops::TailTurn turn{inv_freq, tables.rotary_dim, tables.pairing, batch.positions};
+            rt.ops.headwise_linear(q, static_cast<int>(qd), w_uk_t_->view, q_lat, static_cast<int>(D), shape_.rot, nullptr, &turn);
+        } else {
+            rt.ops.latent_prepare(proj, 0, static_cast<int>(col_dkv_), shape_, dkv_norm_->view, eps_, inv_freq,
+                                  inv_freq ? tables.rotary_dim : 0, tables.pairing, true, batch, *cache.kv);
+            rt.ops.headwise_linear(proj.cols(0, q_cols), static_cast<int>(qd), w_uk_t_->view, q_lat, static_cast<int>(D), shape_.rot, nullptr);
+        }
         Tensor o_lat = rt.ws.buf("latent_o", rt.dtype, {T, H * shape_.rank});
-        rt.ops.latent_attention(q_lat, o_lat, shape_, scale_, sink_ ? &sink_w_->view : nullptr, batch, *cache.kv, rt.ws);
+        rt.ops.latent_attention(q_lat, o_lat, shape_, scale_, sink_ ? &sink_w_->view : nullptr, batch, *cache.kv, rt.ws, window_);
         Tensor heads = rt.ws.buf("latent_heads", rt.dtype, {T, H * vdim_});
-        Tensor gate = gate_ ? proj.cols(q_cols + dkv_cols, g_cols) : Tensor();
+        Tensor gate = gate_ ? proj.cols(col_g_, g_cols) : Tensor();
         rt.ops.headwise_linear(o_lat, shape_.rank, uv_view_, heads, vdim_, 0, gate_ ? &gate : nullptr);
-        Tensor out = rt.ws.buf("mixer_out", rt.dtype, {T, width_});
-        rt.ops.linear(heads, w_o_->view, out, nullptr, rt.ws);
-        return out;
+        return heads;
     }
 
-private:
-    long long width_ = 0;
+    long long width_ = 0, q_rank_ = 0, col_dkv_ = 0, col_g_ = 0;
+    int window_ = 0;
     Ops::LatentShape shape_;
     int vdim_ = 0;
     bool sink_ = false, gate_ = false;
     float eps_ = 1e-6f, scale_ = 1.f;
     std::unique_ptr<PositionEncoding> position_;
-    std::shared_ptr<DeviceTensor> w_in_, w_o_, dkv_norm_, sink_w_, w_uk_t_, w_uv_;
+    std::shared_ptr<DeviceTensor> w_in_, w_o_, dkv_norm_, sink_w_, w_uk_t_, w_uv_, w_uq_, dq_norm_;
     Tensor uv_view_;
 };
 
@@ -832,20 +915,59 @@ public:
 // Logits leave in 32-bit.  "scale" on the embedding multiplies the gathered rows (in 32-bit, as
 // they enter the residual stream); "scale" on a head multiplies the logits; "softcap" c > 0 bends them
 // afterwards to c * tanh(logit / c).
+// "pairs" {"buckets", "mul_prev", "mul_cur"}: a second table [buckets + 1, width] (role "pairs") adds row
+// (previous token * mul_prev + token * mul_cur) mod buckets to every row, the last row to a sequence's first
+// token.  The previous token is state of the request ("last", one int32 in its slot).
 class TokenEmbedding final : public Embedding {
 public:
     explicit TokenEmbedding(const PartSpec& s)
         : Embedding(s), vocab_(s.params.get_int("vocab", 0)), width_(s.params.get_int("width", 0)),
           scale_(static_cast<float>(s.params.get_double("scale", 1.0))) {
         if (vocab_ <= 0 || width_ <= 0) throw SpecError("embedding: vocab and width must be positive");
+        if (!s.params["pairs"].is_null()) {
+            const Json& p = s.params["pairs"];
+            rule_.buckets = p.get_int("buckets", 0);
+            rule_.mul_prev = p.get_int("mul_prev", 0);
+            rule_.mul_cur = p.get_int("mul_cur", 0);
+            if (rule_.buckets <= 0) throw SpecError("embedding: pairs.buckets must be positive");
+            if (scale_ != 1.0f) throw SpecError("embedding: a scale does not go with a table of pairs");
+        }
     }
     bool graph_safe() const override { return true; }
-    WeightSpecs weight_specs() const override { return {{"table", matrix(vocab_, width_)}}; }
-    void load(const PartTensors& t, Runtime&) override { table_ = get(t, "table"); }
+    WeightSpecs weight_specs() const override {
+        WeightSpecs specs{{"table", matrix(vocab_, width_)}};
+        if (rule_.buckets > 0) specs.push_back({"pairs", matrix(rule_.buckets + 1, width_)});
+        return specs;
+    }
+    std::vector<StateNeed> state_needs() const override {
+        if (rule_.buckets <= 0) return {};
+        return {StateNeed{"last", {1}, DType::I32}};
+    }
+    void load(const PartTensors& t, Runtime&) override {
+        table_ = get(t, "table");
+        pairs_ = maybe(t, "pairs");
+        if (pairs_ && pairs_->view.dtype != table_->view.dtype) throw SpecError("embedding: the two tables are stored in different dtypes");
+    }
     Tensor table() const override { return table_->view; }
     bool takes_step_prologue() const override { return true; }
-    void forward(const int* token_ids, const Tensor& out, Runtime& rt, const StepBatch* batch) override {
+    void forward(const int* token_ids, const Tensor& out, Runtime& rt, const StepBatch* batch, const LayerCache& cache) override {
         const int rows = static_cast<int>(out.shape[0]);
+        if (rule_.buckets > 0) {
+            if (!batch) throw SpecError("embedding: pairs of tokens need the step's batch");
+            rt.flush_prologue();
+            const Tensor& last = cache.states.at("last");
+            rt.stream_stat_blocks = 0;
+            rt.stream_has_bf16 = false;
+            if (fused::fused_rows_ok(rt, *batch, {width_}) && (fused::sliced(rt, rows, width_) || fused::tiled_step(rt, rows, width_))) {
+                const Tensor xb = fused::stream_bf16(rt, rows, width_), stats = fused::stream_stats(rt, width_, rows);
+                rt.ops.embed_pairs(table_->view, pairs_->view, rule_, last, *batch, out, &xb, &stats);
+                rt.stream_has_bf16 = true;
+                rt.stream_stat_blocks = 1;
+            } else {
+                rt.ops.embed_pairs(table_->view, pairs_->view, rule_, last, *batch, out, nullptr, nullptr);
+            }
+            return;
+        }
         if (scale_ != 1.0f) {
             rt.flush_prologue();
             rt.ops.embed(table_->view, token_ids, out, scale_);
@@ -879,7 +1001,8 @@ public:
 private:
     long long vocab_, width_;
     float scale_;
-    std::shared_ptr<DeviceTensor> table_;
+    Ops::PairRule rule_;
+    std::shared_ptr<DeviceTensor> table_, pairs_;
 };
 
 // final norm and output product in one kernel for few wanted rows, 32-bit logits
@@ -985,14 +1108,24 @@ private:
 // pre_norm: h += mixer(norm1(h)); h += ffn(norm2(h))
 // (src/backend/cpu/model_forward_token.cpp:93-172).  The residual stream h is 32-bit in every
 // mode and each sum into it is made in 32-bit; an addition is carried forward as delta and made
-// by the next norm's kernel, which reads h anyway.
+// by the next norm's kernel, which reads h anyway.  A feed-forward of kind "none" is left out with its norm.
 class PreNormBlock final : public Block {
 public:
     explicit PreNormBlock(const LayerSpec& layer)
         : mixer_norm_(build_as<Norm>("norm", layer.mixer_norm)), mixer_(build_as<Mixer>("mixer", layer.mixer)),
-          ffn_norm_(build_as<Norm>("norm", layer.ffn_norm)), ffn_(build_as<FeedForward>("ffn", layer.ffn)) {}
+          has_ffn_(layer.ffn.kind != "none") {
+        if (has_ffn_) {
+            ffn_norm_ = build_as<Norm>("norm", layer.ffn_norm);
+            ffn_ = build_as<FeedForward>("ffn", layer.ffn);
+        }
+    }
     std::vector<std::pair<std::string, Part*>> parts() override {
-        return {{"mixer_norm", mixer_norm_.get()}, {"mixer", mixer_.get()}, {"ffn_norm", ffn_norm_.get()}, {"ffn", ffn_.get()}};
+        std::vector<std::pair<std::string, Part*>> out{{"mixer_norm", mixer_norm_.get()}, {"mixer", mixer_.get()}};
+        if (has_ffn_) {
+            out.emplace_back("ffn_norm", ffn_norm_.get());
+            out.emplace_back("ffn", ffn_.get());
+        }
+        return out;
     }
     Mixer& mixer() override { return *mixer_; }
     Tensor forward(const Tensor& h, const Tensor& delta, const StepBatch& batch, const LayerCache& cache, Runtime& rt) override {
@@ -1001,8 +1134,8 @@ public:
         // Few rows: parts that can, take the norm in front of them and the addition behind them
         // into their own products and write the stream themselves.
         const Norm::Foldable* fold1 = mixer_norm_->foldable();
-        const Norm::Foldable* fold2 = ffn_norm_->foldable();
-        const bool fusable = fold1 && fold2;
+        const Norm::Foldable* fold2 = has_ffn_ ? ffn_norm_->foldable() : nullptr;
+        const bool fusable = fold1 && (fold2 || !has_ffn_);
         Tensor mixed;
         if (fusable && !delta.defined() && mixer_->forward_fused(h, *fold1, batch, cache, rt)) {
             // the stream holds the mixer's sum already
@@ -1012,6 +1145,7 @@ public:
             mixed = mixer_->forward(normed, batch, cache, rt);
         }
         rt.mark("mixer " + mixer_->spec.kind);
+        if (!has_ffn_) return mixed;          // (undefined where the mixer wrote the stream itself)
         if (fusable && !mixed.defined() && ffn_->forward_fused(h, *fold2, batch, rt)) {
             rt.mark("ffn " + ffn_->spec.kind);
             return Tensor();
@@ -1026,6 +1160,7 @@ public:
 private:
     std::unique_ptr<Norm> mixer_norm_;
     std::unique_ptr<Mixer> mixer_;
+    bool has_ffn_;
     std::unique_ptr<Norm> ffn_norm_;
     std::unique_ptr<FeedForward> ffn_;
 };
@@ -1328,39 +1463,6 @@ private:
     std::shared_ptr<DeviceTensor> w_in_, b_in_, w_o_, q_norm_, k_norm_, temp_, pb_;
 };
 
-// ---------------------------------------------------------------------------- projections side by side
-// The matrices of several projections of one input, one under the other, so that one product
-// makes them all.  A piece that a later product reads as its input starts at a multiple of 16
-// rows (zero rows in front of it); the whole is padded to a multiple of 16 rows.
-struct Stacked {
-    std::shared_ptr<DeviceTensor> weight;
-    std::vector<long long> at;        // the first row of every piece
-    long long rows = 0;
-};
-Stacked stack_projections(const std::vector<std::pair<std::shared_ptr<DeviceTensor>, bool>>& pieces, const char* who) {
-    Stacked out;
-    std::vector<std::shared_ptr<DeviceTensor>> parts;
-    const DType dtype = pieces.at(0).first->view.dtype;
-    const long long width = pieces.at(0).first->view.shape[1];
-    auto pad_to_16 = [&]() {
-        const long long pad = (16 - out.rows % 16) % 16;
-        if (pad) parts.push_back(from_host_floats(std::vector<float>(static_cast<size_t>(pad * width), 0.f), dtype, {pad, width}));
-        out.rows += pad;
-    };
-    for (const auto& piece : pieces) {
-        const Tensor& v = piece.first->view;
-        if (v.dtype != dtype || v.ndim != 2 || v.shape[1] != width)
-            throw SpecError(std::string(who) + ": the input projections differ in dtype or inner size");
-        if (piece.second) pad_to_16();
-        out.at.push_back(out.rows);
-        parts.push_back(piece.first);
-        out.rows += v.shape[0];
-    }
-    pad_to_16();
-    out.weight = concat_rows(parts);
-    return out;
-}
-
 // ---------------------------------------------------------------------------- gated delta rule
 // A recurrent mixer with a matrix of state per head.
 //
@@ -1621,7 +1723,10 @@ private:
 // with "distance_bias", a learned pair (r1, r2) per query head.  Keys j <= i (inside "window" where one is
 // given; with "keep_first" n the first n positions of the sequence stay visible behind the window, at their
 // true positions).  "gate": "sigmoid" multiplies the heads, side by side, element by element with sigmoid(W_g h).
-// "sink_one": the softmax's denominator holds a one more, p_j = exp(s_j) / (1 + sum exp(s_j)).
+// "sink_one": the softmax's denominator holds a one more, p_j = exp(s_j) / (1 + sum exp(s_j)); "sink": it holds
+// exp(sink[h]) more, a learned number per head (tensor "sink") that is neither scaled nor bent.  "softcap" c: the
+// scaled score s is bent to c tanh(s / c) before the distance bias.  "value_norm": every head's value is divided by
+// sqrt(mean(v^2) + eps) ("eps") before it is cached.
 // "taps" n > 0: every channel of q, k and v passes a causal convolution over time of n taps right behind its
 // projection (tensors q_conv, k_conv, v_conv [channels, taps], no bias; y_t = sum_j w[:, j] u_(t - n + 1 + j),
 // zeros before the sequence starts); the last n - 1 projected rows are the request's state.  "position": a
@@ -1656,11 +1761,22 @@ public:
             if (shape_.window <= 0) shape_.keep_first = 0;       // (without a window every key is visible anyway)
         }
         shape_.sink_one = p.get_bool("sink_one", false);
+        sink_ = p.get_bool("sink", false);
+        if (sink_ && shape_.sink_one) throw SpecError("biased_attention: sink and sink_one exclude each other");
+        if (!p["softcap"].is_null()) {
+            shape_.softcap = static_cast<float>(p["softcap"].as_double());
+            if (!(shape_.softcap > 0.f)) throw SpecError("biased_attention: softcap must be positive");
+        }
+        if (p.get_bool("value_norm", false)) {
+            v_eps_ = static_cast<float>(p.get_double("eps", 1e-6));
+            if (!(v_eps_ > 0.f)) throw SpecError("biased_attention: eps must be positive");
+        }
         taps_ = static_cast<int>(p.get_int("taps", 0));
         if (taps_ < 0) throw SpecError("biased_attention: taps is not negative");
         if (PartSpec::is_part(p["position"]))
             position_ = build_as<PositionEncoding>("position", PartSpec::from_json(p["position"], "biased_attention.position"));
         distance_bias_ = p.get_bool("distance_bias", false);
+        if (v_eps_ > 0.f && (taps_ > 0 || position_)) throw SpecError("biased_attention: value_norm does not go with taps or a position part");
         const std::string gate = p.get_string("gate", "none");
         if (gate != "none" && gate != "sigmoid") throw SpecError("biased_attention: gate is 'none' or 'sigmoid', not '" + gate + "'");
         gated_ = gate == "sigmoid";
@@ -1690,6 +1806,7 @@ public:
             specs.push_back({"r1", vec(shape_.heads, "around_one")});
             specs.push_back({"r2", vec(shape_.heads, "around_one")});
         }
+        if (sink_) specs.push_back({"sink", vec(shape_.heads)});
         if (gated_) specs.push_back({"g", matrix(o_width(), width_)});
         if (taps_ > 0) {
             auto taps = [&](long long n) { return WeightSpec{{n, taps_}, "vector", "normal", {}}; };
@@ -1711,13 +1828,32 @@ public:
         w_o_ = get(t, "o");
         r1_ = maybe(t, "r1");
         r2_ = maybe(t, "r2");
+        sink_w_ = maybe(t, "sink");
     }
     Tensor forward(const Tensor& x, const StepBatch& batch, const LayerCache& cache, Runtime& rt) override {
+        Tensor attended = project_and_attend(x, nullptr, batch, cache, rt);
+        Tensor out = rt.ws.buf("battn_mixer_out", rt.dtype, {x.shape[0], width_});
+        rt.ops.linear(attended, w_o_->view, out, nullptr, rt.ws);
+        return out;
+    }
+    // h += mixer(norm(h)) with the norm folded into the one product in front and the sum into the one behind
+    bool forward_fused(const Tensor& h, const Norm::Foldable& norm, const StepBatch& batch, const LayerCache& cache,
+                       Runtime& rt) override {
+        if (!fused::fused_rows_ok(rt, batch, {width_, o_width()}) || w_in_->view.dtype != rt.dtype || w_o_->view.dtype != rt.dtype) return false;
+        Tensor attended = project_and_attend(h, &norm, batch, cache, rt);
+        fused::linear_into_stream(rt, attended, w_o_->view, h);
+        return true;
+    }
+
+private:
+    // norm null: x are normalised rows; else x is the stream and the norm is applied inside the product
+    Tensor project_and_attend(const Tensor& x, const Norm::Foldable* norm, const StepBatch& batch, const LayerCache& cache, Runtime& rt) {
         if (!cache.kv) throw SpecError("biased_attention: the cache has no keys and values for this layer");
         if (!cache.writes_kv) throw SpecError("biased_attention: reading another entry's cache is not supported");
         const long long T = x.shape[0];
         Tensor proj = rt.ws.buf("battn_proj", rt.dtype, {T, w_in_->view.shape[0]});
-        rt.ops.linear(x, w_in_->view, proj, nullptr, rt.ws);
+        if (norm) fused::norm_linear(rt, x, *norm, w_in_->view, proj, Epilogue::Store);
+        else rt.ops.linear(x, w_in_->view, proj, nullptr, rt.ws);
         // every row's keys and values are in their pages before any row attends
         Tensor q = proj.cols(0, q_width());
         if (taps_ > 0 || position_) {
@@ -1730,24 +1866,22 @@ public:
             rt.ops.conv_rope_store(proj, taps_ > 0 ? &conv_w_->view : nullptr, state, taps_, inv_freq, tables.rotary_dim, tables.pairing,
                                    q, shape_.heads, batch, *cache.kv);
         } else {
-            rt.ops.kv_store(proj.cols(col_k_, k_width()), proj.cols(col_v_, v_width()), batch, *cache.kv);
+            rt.ops.kv_store(proj.cols(col_k_, k_width()), proj.cols(col_v_, v_width()), batch, *cache.kv, v_eps_);
         }
         Tensor attended = rt.ws.buf("battn_out", rt.dtype, {T, o_width()});
         Tensor gate = gated_ ? proj.cols(col_g_, o_width()) : Tensor();
         rt.ops.biased_attention(q, attended, shape_, r1_ ? &r1_->view : nullptr, r2_ ? &r2_->view : nullptr,
-                                gated_ ? &gate : nullptr, batch, *cache.kv, rt.ws);
-        Tensor out = rt.ws.buf("battn_mixer_out", rt.dtype, {T, width_});
-        rt.ops.linear(attended, w_o_->view, out, nullptr, rt.ws);
-        return out;
+                                gated_ ? &gate : nullptr, batch, *cache.kv, rt.ws, sink_w_ ? &sink_w_->view : nullptr);
+        return attended;
     }
 
-private:
     long long width_ = 0, col_k_ = 0, col_v_ = 0, col_g_ = 0;
     Ops::ScoreShape shape_;
-    bool distance_bias_ = false, gated_ = false;
+    bool distance_bias_ = false, gated_ = false, sink_ = false;
+    float v_eps_ = 0.f;
     int taps_ = 0;
     std::unique_ptr<PositionEncoding> position_;
-    std::shared_ptr<DeviceTensor> w_in_, w_o_, r1_, r2_, conv_w_;
+    std::shared_ptr<DeviceTensor> w_in_, w_o_, r1_, r2_, conv_w_, sink_w_;
 };
 
 // ---------------------------------------------------------------------------- real-gated linear recurrent unit
@@ -1984,16 +2118,105 @@ private:
     std::shared_ptr<DeviceTensor> w_in_, a2_, a2_b_, norm_, w_o_;
 };
 
+// ---------------------------------------------------------------------------- matrix memory
+// mLSTM: a matrix of memory per head, written through an exponential gate.
+//     q = W_q h * dim^-1/2, k = W_k h (heads x dim), v = W_v h (heads x vdim)
+//     i = c tanh((W_i h + b_i) / c),  f = log sigmoid(c tanh((W_f h + b_f) / c))      per head, c = "gate_cap"
+//     m' = max(f + m, i);  S <- e^(f + m - m') S + e^(i - m') k v^T;  n likewise with k alone
+//     o = S^T q / (max(|n.q|, e^-m') + 1e-6)
+// m, S and n from zero.  Each head's o is divided by sqrt(mean(o^2) + eps); the heads side by side, times a weight
+// of all their values, times sigmoid(W_g h), go through W_o.  State per request: S [heads, dim, vdim], n
+// [heads, dim], m [heads], 32-bit like everything behind the projections.
+class MatrixMemory final : public Mixer {
+public:
+    explicit MatrixMemory(const PartSpec& s) : Mixer(s) {
+        const Json& p = s.params;
+        width_ = p.get_int("width", 0);
+        shape_.heads = static_cast<int>(p.get_int("heads", 0));
+        shape_.dim = static_cast<int>(p.get_int("dim", 0));
+        shape_.vdim = static_cast<int>(p.get_int("vdim", shape_.dim));
+        shape_.gate_cap = static_cast<float>(p.get_double("gate_cap", 15.0));
+        shape_.eps = static_cast<float>(p.get_double("eps", 1e-6));
+        if (width_ <= 0 || shape_.heads <= 0 || shape_.dim <= 0 || shape_.vdim <= 0)
+            throw SpecError("matrix_memory: width, heads, dim and vdim must be positive");
+        if (shape_.dim > 256 || shape_.vdim > 512) throw SpecError("matrix_memory: dim may be at most 256 and vdim at most 512");
+        if (!(shape_.gate_cap > 0.f) || !(shape_.eps > 0.f)) throw SpecError("matrix_memory: gate_cap and eps must be positive");
+    }
+    bool graph_safe() const override { return true; }
+    long long qk_width() const { return static_cast<long long>(shape_.heads) * shape_.dim; }
+    long long v_width() const { return static_cast<long long>(shape_.heads) * shape_.vdim; }
+    std::vector<StateNeed> state_needs() const override {
+        return {StateNeed{"S", {shape_.heads, shape_.dim, shape_.vdim}, DType::F32}, StateNeed{"n", {shape_.heads, shape_.dim}, DType::F32},
+                StateNeed{"m", {shape_.heads}, DType::F32}};
+    }
+    WeightSpecs weight_specs() const override {
+        const long long H = shape_.heads;
+        return {{"q", matrix(qk_width(), width_)}, {"k", matrix(qk_width(), width_)}, {"v", matrix(v_width(), width_)},
+                {"g", matrix(v_width(), width_)},  {"i", matrix(H, width_)},          {"i_bias", vec(H)},
+                {"f", matrix(H, width_)},          {"f_bias", vec(H)},                {"norm", vec(v_width(), "around_one")},
+                {"o", matrix(width_, v_width())}};
+    }
+    void load(const PartTensors& t, Runtime&) override {
+        const Stacked in = stack_projections({{get(t, "q"), false}, {get(t, "k"), false}, {get(t, "v"), false}, {get(t, "g"), false},
+                                              {get(t, "i"), false}, {get(t, "f"), false}}, "matrix_memory");
+        w_in_ = in.weight;
+        at_.q = in.at[0];
+        at_.k = in.at[1];
+        at_.v = in.at[2];
+        at_.g = in.at[3];
+        at_.i = in.at[4];
+        at_.f = in.at[5];
+        b_i_ = get(t, "i_bias");
+        b_f_ = get(t, "f_bias");
+        norm_ = get(t, "norm");
+        w_o_ = get(t, "o");
+    }
+    Tensor forward(const Tensor& x, const StepBatch& batch, const LayerCache& cache, Runtime& rt) override {
+        Tensor read = project_and_read(x, nullptr, batch, cache, rt);
+        Tensor out = rt.ws.buf("memory_mixer_out", rt.dtype, {x.shape[0], width_});
+        rt.ops.linear(read, w_o_->view, out, nullptr, rt.ws);
+        return out;
+    }
+    // h += mixer(norm(h)) with the norm folded into the one product in front and the sum into the one behind
+    bool forward_fused(const Tensor& h, const Norm::Foldable& norm, const StepBatch& batch, const LayerCache& cache,
+                       Runtime& rt) override {
+        if (!fused::fused_rows_ok(rt, batch, {width_, v_width()}) || w_in_->view.dtype != rt.dtype || w_o_->view.dtype != rt.dtype) return false;
+        Tensor read = project_and_read(h, &norm, batch, cache, rt);
+        fused::linear_into_stream(rt, read, w_o_->view, h);
+        return true;
+    }
+
+private:
+    // norm null: x are normalised rows; else x is the stream and the norm is applied inside the product
+    Tensor project_and_read(const Tensor& x, const Norm::Foldable* norm, const StepBatch& batch, const LayerCache& cache, Runtime& rt) {
+        const long long T = x.shape[0];
+        Tensor proj = rt.ws.buf("memory_proj", rt.dtype, {T, w_in_->view.shape[0]});
+        if (norm) fused::norm_linear(rt, x, *norm, w_in_->view, proj, Epilogue::Store);
+        else rt.ops.linear(x, w_in_->view, proj, nullptr, rt.ws);
+        Tensor read = rt.ws.buf("memory_read", rt.dtype, {T, v_width()});
+        rt.ops.matrix_memory(proj, at_, shape_, b_i_->view, b_f_->view, norm_->view, cache.states.at("S"), cache.states.at("n"),
+                             cache.states.at("m"), read, batch, rt.ws);
+        return read;
+    }
+
+    long long width_ = 0;
+    Ops::MemoryShape shape_;
+    Ops::MemoryColumns at_;
+    std::shared_ptr<DeviceTensor> w_in_, b_i_, b_f_, norm_, w_o_;
+};
+
 // ---------------------------------------------------------------------------- dense feed-forward with biases
 // mlp: W_down act(W_up x + b_up) + b_down; "activation": "gelu_tanh" (0.5 z (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3))))
-// or "relu2" (the square of relu); "bias": false leaves both biases out.
+// or "relu2" (the square of relu) or "xielu" (for z > 0 softplus(p) z^2 + z / 2, else (1/2 + softplus(q)) (e^z - 1 - z) + z / 2
+// with two learned numbers, tensor "act" [2] = (p, q)); "bias": false leaves both biases out.
 class DenseMlp final : public FeedForward {
 public:
     explicit DenseMlp(const PartSpec& s) : FeedForward(s), width_(s.params.get_int("width", 0)), ff_(s.params.get_int("ff", 0)) {
         if (width_ <= 0 || ff_ <= 0) throw SpecError("mlp: width and ff must be positive");
         const std::string act = s.params.get_string("activation", "gelu_tanh");
-        if (act != "gelu_tanh" && act != "relu2") throw SpecError("mlp: activation is 'gelu_tanh' or 'relu2', not '" + act + "'");
-        act_ = act == "relu2" ? 1 : 0;
+        if (act != "gelu_tanh" && act != "relu2" && act != "xielu")
+            throw SpecError("mlp: activation is 'gelu_tanh', 'relu2' or 'xielu', not '" + act + "'");
+        act_ = act == "relu2" ? 1 : act == "xielu" ? 3 : 0;
         bias_ = s.params.get_bool("bias", true);
     }
     bool graph_safe() const override { return true; }
@@ -2003,9 +2226,16 @@ public:
             specs.push_back({"up_bias", vec(ff_)});
             specs.push_back({"down_bias", vec(width_)});
         }
+        if (act_ == 3) specs.push_back({"act", vec(2)});
         return specs;
     }
     void load(const PartTensors& t, Runtime&) override {
+        if (act_ == 3) {
+            const std::vector<float> a = to_host_floats(get(t, "act")->view);
+            auto softplus = [](double z) { return std::max(z, 0.0) + std::log1p(std::exp(-std::fabs(z))); };
+            p0_ = static_cast<float>(softplus(a.at(0)));
+            p1_ = static_cast<float>(0.5 + softplus(a.at(1)));
+        }
         w_up_ = get(t, "up");
         w_down_ = get(t, "down");
         b_up_ = maybe(t, "up_bias");
@@ -2015,15 +2245,25 @@ public:
         const long long T = x.shape[0];
         Tensor up = rt.ws.buf("mlp_up", rt.dtype, {T, ff_});
         rt.ops.linear(x, w_up_->view, up, nullptr, rt.ws);
-        rt.ops.activation_bias(up, b_up_ ? &b_up_->view : nullptr, up, act_);
+        rt.ops.activation_bias(up, b_up_ ? &b_up_->view : nullptr, up, act_, p0_, p1_);
         Tensor out = rt.ws.buf("ffn_out", rt.dtype, {T, width_});
         rt.ops.linear(up, w_down_->view, out, b_down_ ? &b_down_->view : nullptr, rt.ws);
         return out;
+    }
+    // h += ffn(norm(h)) with the norm folded into the first product and the sum into the second
+    bool forward_fused(const Tensor& h, const Norm::Foldable& norm, const StepBatch& batch, Runtime& rt) override {
+        if (!fused::fused_rows_ok(rt, batch, {width_, ff_}) || w_up_->view.dtype != rt.dtype || w_down_->view.dtype != rt.dtype) return false;
+        Tensor up = rt.ws.buf("mlp_up", rt.dtype, {h.shape[0], ff_});
+        fused::norm_linear(rt, h, norm, w_up_->view, up, Epilogue::Store);
+        rt.ops.activation_bias(up, b_up_ ? &b_up_->view : nullptr, up, act_, p0_, p1_);
+        fused::linear_into_stream(rt, up, w_down_->view, h, b_down_ ? &b_down_->view : nullptr);
+        return true;
     }
 
 private:
     long long width_, ff_;
     int act_ = 0;
+    float p0_ = 0.f, p1_ = 0.f;
     bool bias_ = true;
     std::shared_ptr<DeviceTensor> w_up_, w_down_, b_up_, b_down_;
 };
@@ -2163,6 +2403,7 @@ void register_builtin_parts() {
     r.parts["mixer"]["linear_recurrent_unit"] = factory_of<LinearRecurrentUnit>();
     r.parts["mixer"]["normed_pair"] = factory_of<NormedPair>();
     r.parts["mixer"]["gated_linear_attention"] = factory_of<GatedLinearAttention>();
+    r.parts["mixer"]["matrix_memory"] = factory_of<MatrixMemory>();
     r.parts["ffn"]["mlp"] = factory_of<DenseMlp>();
     r.parts["token_input"]["gated_table"] = factory_of<GatedTableInput>();
     r.parts["depth_mix"]["weighted_history"] = factory_of<WeightedHistory>();

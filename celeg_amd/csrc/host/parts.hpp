@@ -14,7 +14,8 @@
 //  * feed-forward: forward(x, batch, rt);
 //  * position encoding: tables(rt), what the mixer's kernels need to turn a row's position into
 //    its encoding;
-//  * embedding and head: forward.
+//  * embedding and head: forward; an embedding may keep state of fixed size per request too
+//    (state_needs()), for one that looks at more than a row's own token.
 // Optional, for the few-rows path: forward_fused, which takes the norm in front of the part and
 // the addition behind it into the part's own products and writes the stream itself.
 #pragma once
@@ -130,7 +131,9 @@ public:
 class Embedding : public Part {
 public:
     using Part::Part;
-    virtual void forward(const int* token_ids, const Tensor& out, Runtime& rt, const StepBatch* batch) = 0;
+    // state of fixed size per request (in the cache manager it belongs to entry CacheLayout::EMBEDDING)
+    virtual std::vector<StateNeed> state_needs() const { return {}; }
+    virtual void forward(const int* token_ids, const Tensor& out, Runtime& rt, const StepBatch* batch, const LayerCache& cache) = 0;
     virtual Tensor table() const { return Tensor(); }     // what a tied head multiplies with
     // true: forward looks at rt.prologue itself (its kernel takes the step's prologue along, or
     // it calls rt.flush_prologue() first); false: the model runs the prologue before forward

@@ -4,7 +4,7 @@
 // the query side takes W_uk in (q_lat = (W_uk^T q_plain, q_rotated), so that a score is one
 // dot product of q_lat with the cached row), the weighted sum runs over c, and W_uv is applied
 // to the result.  A learned number per head (the sink) may join the softmax's denominator; it
-// has no key and no value.
+// has no key and no value.  With a window, row i sees the keys at positions i - window + 1 .. i only.
 #include "mfma_rows.h"
 #include "small_gemm.h"
 
@@ -29,15 +29,17 @@ __device__ __forceinline__ void pair_of(int i, int rotary, int pairing, int& a, 
 // One workgroup per row.  proj[t] holds (q | dkv | ...): q is [heads, dim + rot] at column q_off,
 // dkv is [rank + rot] at column dkv_off.  The first `rank` values of dkv are RMS-normed with
 // `weight` and, with the rotated last `rot` values, written to the row's place in the pages; the
-// rotated part of every query head is turned in place.  The first `rotary` of the `rot` values
-// turn, the rest pass unchanged.
+// rotated part of every query head is turned in place (q_off < 0: no queries here).  The first `rotary`
+// of the `rot` values turn, the rest pass unchanged.  Where the queries come through a compressed row of
+// their own (q_rank > 0), the q_rank values at column cq_off are RMS-normed with q_weight into cq [rows, q_rank].
 template <typename T>
 __global__ void latent_prepare_kernel(T* __restrict__ proj, int ld, int q_off, int dkv_off, int heads, int dim, int rot,
                                       int rank, const float* __restrict__ weight, float eps,
                                       const float* __restrict__ inv_freq, int rotary, int pairing,
                                       const int* __restrict__ positions, const int* __restrict__ token_slot,
                                       const int* __restrict__ table, int table_stride, T* __restrict__ pool, int n_layers,
-                                      int layer, int page_tokens, int write) {
+                                      int layer, int page_tokens, int write, int cq_off, int q_rank,
+                                      const float* __restrict__ q_weight, T* __restrict__ cq) {
     __shared__ float scratch[16];
     const int t = blockIdx.x;
     const int pos = positions[t];
@@ -45,7 +47,7 @@ __global__ void latent_prepare_kernel(T* __restrict__ proj, int ld, int q_off, i
     T* row = proj + static_cast<size_t>(t) * ld;
     const int half = rotary / 2;
     // queries: pair i of head h
-    for (int j = threadIdx.x; j < heads * half; j += blockDim.x) {
+    for (int j = threadIdx.x; q_off >= 0 && j < heads * half; j += blockDim.x) {
         const int h = j / half, i = j - h * half;
         int a, b;
         pair_of(i, rotary, pairing, a, b);
@@ -54,6 +56,18 @@ __global__ void latent_prepare_kernel(T* __restrict__ proj, int ld, int q_off, i
         turn(u, v, fpos * inv_freq[i]);
         qr[a] = from_float<T>(u);
         qr[b] = from_float<T>(v);
+    }
+    if (q_rank > 0) {
+        const T* src = row + cq_off;
+        float sq = 0.f;
+        for (int i = threadIdx.x; i < q_rank; i += blockDim.x) {
+            const float x = to_float(src[i]);
+            sq += x * x;
+        }
+        sq = block_sum(sq, scratch);
+        const float inv = 1.0f / sqrtf(sq / static_cast<float>(q_rank) + eps);
+        for (int i = threadIdx.x; i < q_rank; i += blockDim.x)
+            cq[static_cast<size_t>(t) * q_rank + i] = from_float<T>(to_float(src[i]) * inv * q_weight[i]);
     }
     if (!write) return;
     const T* dkv = row + dkv_off;
@@ -81,12 +95,30 @@ __global__ void latent_prepare_kernel(T* __restrict__ proj, int ld, int q_off, i
 // ---------------------------------------------------------------- a matrix per head
 // out[t, h, n] = sum_k x[t, h, k] w[h, n, k] for n < N; then, if tail > 0, out[t, h, N + j] =
 // x[t, h, K + j] (values that pass by the matrix); with gate: out *= sigmoid(gate[t, h, n]).
+// With tail_freq the first `rotary` values of the tail are turned by the row's position on the way.
 // x: head h of row t starts at x + t * ldx + h * x_head; out likewise with ldo and o_head.
+struct TailTurn {
+    const float* freq;           // null: the tail passes as it is
+    const int* positions;
+    int rotary, pairing;
+};
+// value j of a head's tail (in: the tail's first value) as it goes out
+template <typename T>
+__device__ __forceinline__ T tail_value(const T* in, int j, int t, const TailTurn& turn_by) {
+    if (!turn_by.freq || j >= turn_by.rotary) return in[j];
+    const int i = turn_by.pairing ? j >> 1 : (j < turn_by.rotary / 2 ? j : j - turn_by.rotary / 2);
+    int a, b;
+    pair_of(i, turn_by.rotary, turn_by.pairing, a, b);
+    float u = static_cast<float>(to_float(in[a])), v = static_cast<float>(to_float(in[b]));
+    turn(u, v, static_cast<float>(turn_by.positions[t]) * turn_by.freq[i]);
+    return from_float<T>(j == a ? u : v);
+}
+
 template <typename T>
 __global__ __launch_bounds__(256) void headwise_linear_kernel(const T* __restrict__ x, int ldx, int x_head,
                                                               const T* __restrict__ w, int N, int K, T* __restrict__ out,
                                                               int ldo, int o_head, int tail, const T* __restrict__ gate,
-                                                              int ldg, int rows) {
+                                                              int ldg, int rows, const TailTurn turn_by) {
     __shared__ float as[SG_ROWS][SG_K + 1], ws[SG_COLS][SG_K + 1];
     const int h = blockIdx.z;
     const int row0 = blockIdx.x * SG_ROWS, col0 = blockIdx.y * SG_COLS;
@@ -115,7 +147,7 @@ __global__ __launch_bounds__(256) void headwise_linear_kernel(const T* __restric
         for (int i = threadIdx.x; i < rows_valid * tail; i += 256) {
             const int r = i / tail, j = i - r * tail;
             out[static_cast<size_t>(row0 + r) * ldo + static_cast<size_t>(h) * o_head + N + j] =
-                a[static_cast<size_t>(r) * ldx + K + j];
+                tail_value(a + static_cast<size_t>(r) * ldx + K, j, row0 + r, turn_by);
         }
 }
 
@@ -123,7 +155,8 @@ __global__ __launch_bounds__(256) void headwise_linear_kernel(const T* __restric
 __global__ __launch_bounds__(256) void headwise_linear_mfma_kernel(const __bf16* __restrict__ x, int ldx, int x_head,
                                                                    const __bf16* __restrict__ w, int N, int K,
                                                                    __bf16* __restrict__ out, int ldo, int o_head, int tail,
-                                                                   const __bf16* __restrict__ gate, int ldg, int rows) {
+                                                                   const __bf16* __restrict__ gate, int ldg, int rows,
+                                                                   const TailTurn turn_by) {
     const int h = blockIdx.z, row0 = blockIdx.x * MR_ROWS;
     const int rows_valid = min(MR_ROWS, rows - row0);
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, c = lane & 15, qd = lane >> 4;
@@ -132,7 +165,8 @@ __global__ __launch_bounds__(256) void headwise_linear_mfma_kernel(const __bf16*
     if (tail > 0 && blockIdx.y == 0)
         for (int i = threadIdx.x; i < rows_valid * tail; i += 256) {
             const int r = i / tail, j = i - r * tail;
-            out[static_cast<size_t>(row0 + r) * ldo + static_cast<size_t>(h) * o_head + N + j] = a[static_cast<size_t>(r) * ldx + K + j];
+            reinterpret_cast<bf16*>(out)[static_cast<size_t>(row0 + r) * ldo + static_cast<size_t>(h) * o_head + N + j] =
+                tail_value(reinterpret_cast<const bf16*>(a) + static_cast<size_t>(r) * ldx + K, j, row0 + r, turn_by);
         }
     if (col0 >= N) return;
     const __bf16* w_row[1][1] = {{col0 + c < N ? w + (static_cast<size_t>(h) * N + col0 + c) * K : nullptr}};
@@ -162,7 +196,7 @@ __global__ __launch_bounds__(256) void headwise_linear_mfma_kernel(const __bf16*
 
 // ---------------------------------------------------------------- attention, general form
 // One wavefront per (row, head).  The row's q_lat [rank + rot] against the cached rows of its
-// request at positions 0..pos, 64 keys at a time: a lane scores one key, the chunk joins a
+// request at positions 0..pos (the last `window` of them with a window), 64 keys at a time: a lane scores one key, the chunk joins a
 // running (max, sum, accumulator) in 32-bit, the accumulator running over the first `rank`
 // values of the cached rows.  The chunking depends on the row's own position only.
 #define LAT_MAX_CHUNKS 16     // rank <= 1024
@@ -172,7 +206,7 @@ __global__ void latent_attention_kernel(const T* __restrict__ q, int ldq, const 
                                         const int* __restrict__ table, int table_stride,
                                         const int* __restrict__ token_slot, const int* __restrict__ positions,
                                         const float* __restrict__ sink, T* __restrict__ out, int ldo, int heads, int rank,
-                                        int rot, int page_tokens, int n_layers, int layer, float scale) {
+                                        int rot, int page_tokens, int n_layers, int layer, float scale, int window) {
     extern __shared__ float lds[];      // rank + rot floats of q, then 64 weights
     const int D = rank + rot;
     float* qs = lds;
@@ -187,7 +221,7 @@ __global__ void latent_attention_kernel(const T* __restrict__ q, int ldq, const 
     float acc[LAT_MAX_CHUNKS];
 #pragma unroll
     for (int j = 0; j < LAT_MAX_CHUNKS; ++j) acc[j] = 0.f;
-    for (int base = 0; base <= pos; base += CELEG_WAVE) {
+    for (int base = window > 0 ? max(0, pos - window + 1) : 0; base <= pos; base += CELEG_WAVE) {
         const int key = base + lane;
         const bool valid = key <= pos;
         float s = -INFINITY;
@@ -241,50 +275,55 @@ __global__ void latent_attention_kernel(const T* __restrict__ q, int ldq, const 
 extern "C" int celeg_latent_prepare(void* proj, int ld, int dtype, int q_off, int dkv_off, int heads, int dim, int rot,
                                     int rank, const float* weight, float eps, const float* inv_freq, int rotary, int pairing,
                                     const int* positions, const int* token_slot, const int* table, int table_stride,
-                                    void* pool, int n_layers, int layer, int page_tokens, int write, int n_tokens,
-                                    hipStream_t stream) {
+                                    void* pool, int n_layers, int layer, int page_tokens, int write, int n_tokens, int cq_off,
+                                    int q_rank, const float* q_weight, void* cq, hipStream_t stream) {
     if (n_tokens <= 0) return 0;
     if (rotary < 0 || rotary % 2 || rotary > rot || (rotary > 0 && !inv_freq)) return static_cast<int>(hipErrorInvalidValue);
     if (dtype == CELEG_F32)
         hipLaunchKernelGGL(latent_prepare_kernel<float>, dim3(n_tokens), dim3(256), 0, stream, static_cast<float*>(proj), ld,
                            q_off, dkv_off, heads, dim, rot, rank, weight, eps, inv_freq, rotary, pairing, positions,
-                           token_slot, table, table_stride, static_cast<float*>(pool), n_layers, layer, page_tokens, write);
+                           token_slot, table, table_stride, static_cast<float*>(pool), n_layers, layer, page_tokens, write, cq_off,
+                           q_rank, q_weight, static_cast<float*>(cq));
     else
         hipLaunchKernelGGL(latent_prepare_kernel<bf16>, dim3(n_tokens), dim3(256), 0, stream, static_cast<bf16*>(proj), ld,
                            q_off, dkv_off, heads, dim, rot, rank, weight, eps, inv_freq, rotary, pairing, positions,
-                           token_slot, table, table_stride, static_cast<bf16*>(pool), n_layers, layer, page_tokens, write);
+                           token_slot, table, table_stride, static_cast<bf16*>(pool), n_layers, layer, page_tokens, write, cq_off,
+                           q_rank, q_weight, static_cast<bf16*>(cq));
     return CELEG_LAUNCH_RESULT();
 }
 
 extern "C" int celeg_headwise_linear(const void* x, int ldx, int x_head, const void* w, int dtype, int heads, int N, int K,
                                      void* out, int ldo, int o_head, int tail, const void* gate, int ldg, int rows,
-                                     int matrix_cores, hipStream_t stream) {
+                                     int matrix_cores, const float* tail_freq, int rotary, int pairing, const int* positions,
+                                     hipStream_t stream) {
     if (rows <= 0) return 0;
+    if (tail_freq && (rotary < 0 || rotary % 2 || rotary > tail || !positions)) return static_cast<int>(hipErrorInvalidValue);
+    const TailTurn turn_by{rotary > 0 ? tail_freq : nullptr, positions, rotary, pairing};
     if (matrix_cores) {
         if (dtype != CELEG_BF16 || K % 32 || N % 16 || ldx % 8 || x_head % 8 || ldo % 4 || o_head % 4)
             return static_cast<int>(hipErrorInvalidValue);
         dim3 mgrid((rows + MR_ROWS - 1) / MR_ROWS, (N + MR_COLS - 1) / MR_COLS, heads);
         hipLaunchKernelGGL(headwise_linear_mfma_kernel, mgrid, dim3(256), 0, stream, static_cast<const __bf16*>(x), ldx, x_head,
                            static_cast<const __bf16*>(w), N, K, static_cast<__bf16*>(out), ldo, o_head, tail,
-                           static_cast<const __bf16*>(gate), ldg, rows);
+                           static_cast<const __bf16*>(gate), ldg, rows, turn_by);
         return CELEG_LAUNCH_RESULT();
     }
     dim3 grid((rows + SG_ROWS - 1) / SG_ROWS, (N + SG_COLS - 1) / SG_COLS, heads);
     if (dtype == CELEG_F32)
         hipLaunchKernelGGL(headwise_linear_kernel<float>, grid, dim3(256), 0, stream, static_cast<const float*>(x), ldx,
                            x_head, static_cast<const float*>(w), N, K, static_cast<float*>(out), ldo, o_head, tail,
-                           static_cast<const float*>(gate), ldg, rows);
+                           static_cast<const float*>(gate), ldg, rows, turn_by);
     else
         hipLaunchKernelGGL(headwise_linear_kernel<bf16>, grid, dim3(256), 0, stream, static_cast<const bf16*>(x), ldx,
                            x_head, static_cast<const bf16*>(w), N, K, static_cast<bf16*>(out), ldo, o_head, tail,
-                           static_cast<const bf16*>(gate), ldg, rows);
+                           static_cast<const bf16*>(gate), ldg, rows, turn_by);
     return CELEG_LAUNCH_RESULT();
 }
 
 extern "C" int celeg_latent_attention(const void* q, int ldq, const void* pool, int dtype, const int* table,
                                       int table_stride, const int* token_slot, const int* positions, const float* sink,
                                       void* out, int ldo, int n_tokens, int heads, int rank, int rot, int page_tokens,
-                                      int n_layers, int layer, float scale, hipStream_t stream) {
+                                      int n_layers, int layer, float scale, int window, hipStream_t stream) {
     if (n_tokens <= 0) return 0;
     if (rank > LAT_MAX_CHUNKS * CELEG_WAVE) return static_cast<int>(hipErrorInvalidValue);
     dim3 grid(n_tokens, heads), block(CELEG_WAVE);
@@ -292,10 +331,10 @@ extern "C" int celeg_latent_attention(const void* q, int ldq, const void* pool, 
     if (dtype == CELEG_F32)
         hipLaunchKernelGGL(latent_attention_kernel<float>, grid, block, lds, stream, static_cast<const float*>(q), ldq,
                            static_cast<const float*>(pool), table, table_stride, token_slot, positions, sink,
-                           static_cast<float*>(out), ldo, heads, rank, rot, page_tokens, n_layers, layer, scale);
+                           static_cast<float*>(out), ldo, heads, rank, rot, page_tokens, n_layers, layer, scale, window);
     else
         hipLaunchKernelGGL(latent_attention_kernel<bf16>, grid, block, lds, stream, static_cast<const bf16*>(q), ldq,
                            static_cast<const bf16*>(pool), table, table_stride, token_slot, positions, sink,
-                           static_cast<bf16*>(out), ldo, heads, rank, rot, page_tokens, n_layers, layer, scale);
+                           static_cast<bf16*>(out), ldo, heads, rank, rot, page_tokens, n_layers, layer, scale, window);
     return CELEG_LAUNCH_RESULT();
 }

@@ -14,6 +14,9 @@
 // 16 of the rows), keys 0..position of its last row.  Form 1, single tokens: a workgroup owns one
 // row, 16 heads (the columns of one wavefront; all four load) and one share of the row's keys;
 // the shares' partial results meet in a second kernel, which also adds the sink.
+//
+// With a window the blocks begin at the first key that any column of the workgroup sees, and keys a column
+// no longer sees are masked; pages wholly before the window may be another request's by then and are not read.
 #include "common.h"
 
 typedef __bf16 lat_bf16x8 __attribute__((ext_vector_type(8)));
@@ -40,7 +43,8 @@ __global__ __launch_bounds__(256, (KSMAX <= 9 ? 2 : 1)) void latent_attention_mf
     const int* __restrict__ cu_seqlens, const int* __restrict__ seq_slot, const int* __restrict__ seq_start, int n_seqs,
     const int* __restrict__ token_slot, const int* __restrict__ positions, const float* __restrict__ sink,
     __bf16* __restrict__ out, int ldo, float* __restrict__ ws_o, float* __restrict__ ws_ml, int n_splits,
-    int blocks_per_split, int heads, int rank, int rot, int page_tokens, int n_layers, int layer, float scale_log2e) {
+    int blocks_per_split, int heads, int rank, int rot, int page_tokens, int n_layers, int layer, float scale_log2e,
+    int window) {
     extern __shared__ __attribute__((aligned(16))) unsigned char latf_lds[];
     const int D = rank + rot, KS = (D + 31) / 32, Dpad = KS * 32, KROW = Dpad + 8, DT = rank / 16;
     __bf16* sK = reinterpret_cast<__bf16*>(latf_lds);                 // [64][KROW]
@@ -50,7 +54,7 @@ __global__ __launch_bounds__(256, (KSMAX <= 9 ? 2 : 1)) void latent_attention_mf
 
     // ---- which columns this workgroup owns
     int slot, first_block, end_block;      // key blocks [first_block, end_block)
-    int wg_limit;                          // the last key any column of the workgroup sees
+    int wg_limit, wg_first;                // the last and the first key any column of the workgroup sees
     int col_row[RT], col_head, col_limit[RT];   // this lane's columns: row of q / out, head, last key seen (-1: none)
     bool wave_computes;
     if (FORM == 0) {
@@ -73,7 +77,8 @@ __global__ __launch_bounds__(256, (KSMAX <= 9 ? 2 : 1)) void latent_attention_mf
             col_limit[rt] = r < len ? start + r : -1;
         }
         const int last = min(len, tile * TILE + TILE) - 1;
-        first_block = 0;
+        wg_first = window > 0 ? max(0, start + tile * TILE - window + 1) : 0;
+        first_block = wg_first / LATF_KEYS;
         wg_limit = start + last;
         end_block = wg_limit / LATF_KEYS + 1;
         wave_computes = tile * TILE + wave * RT * 16 < len;
@@ -88,7 +93,8 @@ __global__ __launch_bounds__(256, (KSMAX <= 9 ? 2 : 1)) void latent_attention_mf
             col_limit[rt] = col_head < heads ? pos : -1;
         }
         wg_limit = pos;
-        first_block = blockIdx.z * blocks_per_split;
+        wg_first = window > 0 ? max(0, pos - window + 1) : 0;
+        first_block = wg_first / LATF_KEYS + blockIdx.z * blocks_per_split;
         end_block = min(pos / LATF_KEYS + 1, first_block + blocks_per_split);
         wave_computes = wave == 0;
     }
@@ -150,7 +156,7 @@ __global__ __launch_bounds__(256, (KSMAX <= 9 ? 2 : 1)) void latent_attention_mf
         __syncthreads();
         if (tid < LATF_KEYS) {
             const int pos = kb + tid;
-            s_page[tid] = pos <= wg_limit ? pages[pos >> page_shift] : -1;
+            s_page[tid] = pos <= wg_limit && pos >= wg_first ? pages[pos >> page_shift] : -1;
         }
         __syncthreads();
         {
@@ -194,7 +200,7 @@ __global__ __launch_bounds__(256, (KSMAX <= 9 ? 2 : 1)) void latent_attention_mf
         bool live[RT];
 #pragma unroll
         for (int rt = 0; rt < RT; ++rt) {
-            live[rt] = kb <= tile_limit[rt];
+            live[rt] = kb <= tile_limit[rt] && (window <= 0 || kb + LATF_KEYS - 1 > tile_min_limit[rt] - window);
 #pragma unroll
             for (int kt = 0; kt < 4; ++kt) sacc[rt][kt] = lat_f32x4{0.f, 0.f, 0.f, 0.f};
         }
@@ -215,12 +221,15 @@ __global__ __launch_bounds__(256, (KSMAX <= 9 ? 2 : 1)) void latent_attention_mf
         lat_bf16x8 pb[RT][2];
 #pragma unroll
         for (int rt = 0; rt < RT; ++rt) {
-            if (kb + LATF_KEYS - 1 > tile_min_limit[rt]) {
+            if (kb + LATF_KEYS - 1 > tile_min_limit[rt] || (window > 0 && kb <= tile_limit[rt] - window)) {
+                const int col_first = window > 0 ? col_limit[rt] - window + 1 : 0;
 #pragma unroll
                 for (int kt = 0; kt < 4; ++kt)
 #pragma unroll
-                    for (int r = 0; r < 4; ++r)
-                        if (kb + 32 * (kt >> 1) + 8 * qd + 4 * (kt & 1) + r > col_limit[rt]) sacc[rt][kt][r] = -INFINITY;
+                    for (int r = 0; r < 4; ++r) {
+                        const int key = kb + 32 * (kt >> 1) + 8 * qd + 4 * (kt & 1) + r;
+                        if (key > col_limit[rt] || key < col_first) sacc[rt][kt][r] = -INFINITY;
+                    }
             }
             float mx = -INFINITY;
 #pragma unroll
@@ -334,7 +343,7 @@ static int latent_mfma_launch(dim3 grid, size_t lds, hipStream_t stream, const v
                               const int* seq_start, int n_seqs, const int* token_slot, const int* positions,
                               const float* sink, void* out, int ldo, float* ws_o, float* ws_ml, int n_splits,
                               int blocks_per_split, int heads, int rank, int rot, int page_tokens, int n_layers, int layer,
-                              float scale_log2e) {
+                              float scale_log2e, int window) {
     auto kernel = latent_attention_mfma_kernel<FORM, KSMAX, DTMAX, RT>;
     if (lds > 64 * 1024) {
         const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(kernel), hipFuncAttributeMaxDynamicSharedMemorySize,
@@ -344,7 +353,7 @@ static int latent_mfma_launch(dim3 grid, size_t lds, hipStream_t stream, const v
     hipLaunchKernelGGL(kernel, grid, dim3(256), lds, stream, static_cast<const __bf16*>(q), ldq,
                        static_cast<const __bf16*>(pool), table, table_stride, cu_seqlens, seq_slot, seq_start, n_seqs,
                        token_slot, positions, sink, static_cast<__bf16*>(out), ldo, ws_o, ws_ml, n_splits, blocks_per_split,
-                       heads, rank, rot, page_tokens, n_layers, layer, scale_log2e);
+                       heads, rank, rot, page_tokens, n_layers, layer, scale_log2e, window);
     return CELEG_LAUNCH_RESULT();
 }
 
@@ -369,7 +378,7 @@ extern "C" int celeg_latent_attention_fast(int form, const void* q, int ldq, con
                                            const int* positions, int n_single, const float* sink, void* out, int ldo,
                                            float* ws_o, float* ws_ml, int n_splits, int blocks_per_split, int heads,
                                            int rank, int rot, int page_tokens, int n_layers, int layer, float scale,
-                                           hipStream_t stream) {
+                                           int window, hipStream_t stream) {
     if (!celeg_latent_attention_fast_ok(rank, rot) || (form == 1 && n_splits > LATF_MAX_SPLITS) || page_tokens <= 0 ||
         (page_tokens & (page_tokens - 1)))
         return static_cast<int>(hipErrorInvalidValue);
@@ -382,7 +391,7 @@ extern "C" int celeg_latent_attention_fast(int form, const void* q, int ldq, con
     return latent_mfma_launch<FORM, KSM, DTM, RT>(grid, lds, stream, q, ldq, pool, table, table_stride, cu_seqlens, seq_slot,  \
                                               seq_start, n_seqs, token_slot, positions, sink, out, ldo, ws_o, ws_ml,       \
                                               n_splits, blocks_per_split, heads, rank, rot, page_tokens, n_layers, layer,  \
-                                              scale_log2e)
+                                              scale_log2e, window)
     if (form == 0) {
         if (KS <= 5 && DT <= 8) LATF_GO(0, 5, 8, 1);
         if (KS <= 9 && DT <= 16) LATF_GO(0, 9, 16, 1);
@@ -392,15 +401,15 @@ extern "C" int celeg_latent_attention_fast(int form, const void* q, int ldq, con
     if (KS <= 5 && DT <= 8)
         rc = latent_mfma_launch<1, 5, 8, 1>(grid, lds, stream, q, ldq, pool, table, table_stride, cu_seqlens, seq_slot, seq_start,
                                          n_seqs, token_slot, positions, sink, out, ldo, ws_o, ws_ml, n_splits, blocks_per_split,
-                                         heads, rank, rot, page_tokens, n_layers, layer, scale_log2e);
+                                         heads, rank, rot, page_tokens, n_layers, layer, scale_log2e, window);
     else if (KS <= 9 && DT <= 16)
         rc = latent_mfma_launch<1, 9, 16, 1>(grid, lds, stream, q, ldq, pool, table, table_stride, cu_seqlens, seq_slot, seq_start,
                                           n_seqs, token_slot, positions, sink, out, ldo, ws_o, ws_ml, n_splits, blocks_per_split,
-                                          heads, rank, rot, page_tokens, n_layers, layer, scale_log2e);
+                                          heads, rank, rot, page_tokens, n_layers, layer, scale_log2e, window);
     else
         rc = latent_mfma_launch<1, 18, 32, 1>(grid, lds, stream, q, ldq, pool, table, table_stride, cu_seqlens, seq_slot,
                                            seq_start, n_seqs, token_slot, positions, sink, out, ldo, ws_o, ws_ml, n_splits,
-                                           blocks_per_split, heads, rank, rot, page_tokens, n_layers, layer, scale_log2e);
+                                           blocks_per_split, heads, rank, rot, page_tokens, n_layers, layer, scale_log2e, window);
     if (rc) return rc;
     hipLaunchKernelGGL(latent_attention_join_kernel, dim3(n_single, heads), dim3(128), 0, stream, ws_o, ws_ml, n_splits, sink,
                        static_cast<__bf16*>(out), ldo, heads, rank);

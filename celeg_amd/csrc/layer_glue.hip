@@ -17,16 +17,21 @@ __device__ __forceinline__ float lg_relu2(float z) {
     return r * r;
 }
 
-// out = act(x + bias); act 0: gelu (tanh form), 1: square of relu, 2: none
+// z > 0: right z^2 + z / 2;  z <= 0: left (exp(z) - 1 - z) + z / 2 (both pieces and their slopes meet at 0)
+__device__ __forceinline__ float lg_bent(float z, float right, float left) {
+    return (z > 0.f ? right * z * z : left * (expm1f(z) - z)) + 0.5f * z;
+}
+
+// out = act(x + bias); act 0: gelu (tanh form), 1: square of relu, 2: none, 3: lg_bent with (p0, p1)
 template <typename T>
 __global__ void activation_bias_kernel(const T* __restrict__ x, int ldx, const float* __restrict__ bias, T* __restrict__ out,
-                                       int ldo, int cols, int act) {
+                                       int ldo, int cols, int act, float p0, float p1) {
     const int t = blockIdx.y;
     const int c = blockIdx.x * blockDim.x + threadIdx.x;
     if (c >= cols) return;
     float z = to_float(x[static_cast<size_t>(t) * ldx + c]);
     if (bias) z += bias[c];
-    const float y = act == 0 ? lg_gelu_tanh(z) : act == 1 ? lg_relu2(z) : z;
+    const float y = act == 0 ? lg_gelu_tanh(z) : act == 1 ? lg_relu2(z) : act == 3 ? lg_bent(z, p0, p1) : z;
     out[static_cast<size_t>(t) * ldo + c] = from_float<T>(y);
 }
 
@@ -122,10 +127,10 @@ __global__ void softcap_kernel(float* __restrict__ x, size_t n, float cap) {
     }
 
 extern "C" int celeg_activation_bias(const void* x, int ldx, const float* bias, void* out, int ldo, int dtype, int rows, int cols,
-                                     int act, hipStream_t stream) {
+                                     int act, float p0, float p1, hipStream_t stream) {
     if (rows <= 0 || cols <= 0) return 0;
     dim3 grid((cols + 255) / 256, rows), block(256);
-    LG_BY_DTYPE(activation_bias_kernel, grid, block, static_cast<const T*>(x), ldx, bias, static_cast<T*>(out), ldo, cols, act);
+    LG_BY_DTYPE(activation_bias_kernel, grid, block, static_cast<const T*>(x), ldx, bias, static_cast<T*>(out), ldo, cols, act, p0, p1);
     return CELEG_LAUNCH_RESULT();
 }
 
