@@ -223,6 +223,39 @@ VABUZEN_SHAPES = {
            regipel_shape(2048, 8, 16, 128, 64, 128, 512, 32, 6, 1024, streams=None)),
 }
 
+# Minilorn beside Kifetar, the closest existing design with both attention and a matrix state per head: attention (inside
+# the same window where Minilorn's compressed rows have one) where Minilorn has attention of either kind, the delta rule
+# where Minilorn has its matrix memory, with as many state numbers; feed-forwards of as many weights.
+MINILORN_PATTERN = "lmallmal"
+
+
+def minilorn_shape(width, heads, kv_heads, dim, window, l_dim, l_rot, rank, q_rank, m_heads, m_dim, m_vdim, ff, vocab=65536):
+    kinds = {"a": ("attention", {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "scale": dim ** -0.5,
+                                 "q_temp": {"coef": 0.1, "every": 512}, "softcap": 30.0}),
+             "l": ("latent_attention", {"heads": heads, "dim": l_dim, "rot_dim": l_rot, "vdim": l_dim, "q_rank": q_rank, "kv_rank": rank,
+                                        "scale": (l_dim + l_rot) ** -0.5, "rot": {"base": 500000.0, "dims": l_rot}, "mask": {"size": window}}),
+             "m": ("mlstm", {"heads": m_heads, "dim": m_dim, "vdim": m_vdim, "gate_cap": 15.0})}
+    return {"architecture": "Minilorn", "vocab": vocab, "width": width, "norm": {"eps": 1e-5}, "max_context": 8192,
+            "embedding": {"bigram": {"buckets": 16381, "mul_prev": 7919, "mul_cur": 104729}},
+            "layers": [{"type": kinds[c][0], "mixer": kinds[c][1], "mlp": {"kind": "dense", "ff": ff}} for c in MINILORN_PATTERN]}
+
+
+def minilorn_beside(width, heads, kv_heads, dim, window, d_heads, d_kv_heads, d_dim, d_vdim, ff):
+    cfg = kifetar_shape(width, "".join("d" if c == "m" else "a" for c in MINILORN_PATTERN), heads, kv_heads, dim, window,
+                        d_heads, d_kv_heads, d_dim, d_vdim, ff)
+    for c, layer in zip(MINILORN_PATTERN, cfg["layers"]):
+        if c == "a":
+            layer["mixer"] = {k: v for k, v in layer["mixer"].items() if k != "mask"}
+    return cfg
+
+
+MINILORN_SHAPES = {
+    "1k": (minilorn_shape(1024, 16, 8, 64, 1024, 64, 32, 256, 512, 8, 64, 128, 3072),
+           minilorn_beside(1024, 16, 8, 64, 1024, 16, 8, 64, 64, 2048)),
+    "2k": (minilorn_shape(2048, 16, 8, 128, 1024, 128, 64, 512, 1024, 8, 128, 256, 6144),
+           minilorn_beside(2048, 16, 8, 128, 1024, 16, 8, 128, 128, 4096)),
+}
+
 DESIGN_SHAPES = {
     "1k": (regipel_shape(1024, 8, 16, 64, 32, 64, 256, 16, 2, 1024), lfm2_shape(1024, 16, 8, 2048, set(range(8)), 8, 8192)),
     "2k": (regipel_shape(2048, 8, 16, 128, 64, 128, 512, 32, 4, 1024), lfm2_shape(2048, 32, 8, 4096, set(range(8)), 8, 8192)),
@@ -239,7 +272,8 @@ def design(shapes, steps: int, warmup: int, batch: int, layers: int = 0, profile
     out = {}
     for shape in shapes:
         table, beside = {"kifetar": (KIFETAR_SHAPES, "lfm2_hybrid"), "kivorax": (KIVORAX_SHAPES, "kifetar_beside"),
-                         "regipel": (DESIGN_SHAPES, "lfm2_attention"), "vabuzen": (VABUZEN_SHAPES, "regipel_beside")}[which]
+                         "regipel": (DESIGN_SHAPES, "lfm2_attention"), "vabuzen": (VABUZEN_SHAPES, "regipel_beside"),
+                         "minilorn": (MINILORN_SHAPES, "kifetar_beside")}[which]
         for label, cfg in zip((which, beside), table[shape]):
             if profile_only and label != profile_only:
                 continue
@@ -271,7 +305,8 @@ def design(shapes, steps: int, warmup: int, batch: int, layers: int = 0, profile
             engine.close()
     title = {"kifetar": "Kifetar beside LFM2 convolution and attention layers", "regipel": "Regipel beside LFM2 attention layers",
              "kivorax": "Kivorax beside Kifetar attention and delta-rule layers",
-             "vabuzen": "Vabuzen beside Regipel layers of one residual stream"}[which]
+             "vabuzen": "Vabuzen beside Regipel layers of one residual stream",
+             "minilorn": "Minilorn beside Kifetar attention and delta-rule layers"}[which]
     print(json.dumps({"metric": title + " at equal size: prefill tok/s @ 2048 tokens, "
                                 f"decode tok/s @ batch {batch}, context 2048 (bf16, random weights)",
                       "phase": "design", "design": which, "batch": batch, "steps": steps, "warmup": warmup, "dtype": "bf16",
@@ -301,9 +336,9 @@ def main() -> int:
                          "(default 2048, the headline's); with --phase prefill: tokens of the same "
                          "prompt that the cache holds before the measured portion of 2,048 (default 0)")
     ap.add_argument("--design-shape", default="1k,2k", help="with --phase design: which sizes (1k, 2k)")
-    ap.add_argument("--design", default="regipel", choices=["regipel", "kifetar", "kivorax", "vabuzen"],
+    ap.add_argument("--design", default="regipel", choices=["regipel", "kifetar", "kivorax", "vabuzen", "minilorn"],
                     help="with --phase design: which design is measured beside its closest LFM2 shape")
-    ap.add_argument("--design-model", default="", choices=["", "regipel", "lfm2_attention", "kifetar", "lfm2_hybrid", "kivorax", "kifetar_beside", "vabuzen", "regipel_beside"],
+    ap.add_argument("--design-model", default="", choices=["", "regipel", "lfm2_attention", "kifetar", "lfm2_hybrid", "kivorax", "kifetar_beside", "vabuzen", "regipel_beside", "minilorn"],
                     help="with --phase design: only this model (for profiling)")
     ap.add_argument("--phase", choices=["all", "prefill", "decode", "serve", "design"], default="all",
                     help="for profiling: run only the prefill measurement, or only the batch-8 "

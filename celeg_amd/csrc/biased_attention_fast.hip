@@ -5,8 +5,8 @@
 // denominator may hold one more term, a key without a value that the row meets before all others: of score 0
 // (`sink_one`) or of a learned score per head (`sink`).  With `softcap` c a scaled score s is bent to
 // c * tanh(s / c) = c - 2 c / (exp(2 s / c) + 1) before the bias.
-// Keys of up to `D` numbers, values of up to `V` numbers a head (D, V multiples of 32 up to 128; smaller heads,
-// keys in multiples of 8 and values in multiples of 4, are staged with zeros behind them).
+// Keys of `D` numbers, values of `V` numbers a head (multiples of 32 up to 128: FULL), or of fewer, keys in
+// multiples of 8 and values in multiples of 4, which are staged with zeros behind them (not FULL).
 // Cache layout: K [pages, layers, kv_heads, page_tokens, D], V [pages, layers, kv_heads, V, page_tokens].
 //
 // Scores are computed transposed (keys as the first operand of a 16x16x32 instruction): a lane
@@ -53,29 +53,31 @@ struct BfRow {
 
 // the pieces of a key block that a thread brings from the pages: keys kb .. kb + 63 (those past
 // pos_last: the last one again), values with zeros past pos_last
-template <int D, int V, int THREADS>
+template <int D, int V, int THREADS, bool FULL>
 struct BfFetch {
     static constexpr int KCH = BF_KEYS * (D / 8) / THREADS, VCH = V * (BF_KEYS / 8) / THREADS;
     bf_u32x4 k[KCH], v[VCH];
     __device__ __forceinline__ void load(int tid, int kb, int pos_last, const bf16* __restrict__ k_pool, const bf16* __restrict__ v_pool,
                                          const int* __restrict__ pages, int page_shift, int page_mask, int page_tokens,
-                                         size_t head_index_stride, int kvh, size_t layer_index, int kd, int vd) {
+                                         size_t head_index_stride, int kvh, size_t layer_index, int kd_, int vd_) {
+        const int kd = FULL ? D : kd_, vd = FULL ? V : vd_;
 #pragma unroll
         for (int i = 0; i < KCH; ++i) {
             const int c = tid + THREADS * i, key_in = c / (D / 8), part = c % (D / 8);
             const int key = min(kb + key_in, pos_last);
             const size_t head = (static_cast<size_t>(pages[key >> page_shift]) * head_index_stride + layer_index) + kvh;
-            k[i] = bf_u32x4{0u, 0u, 0u, 0u};
-            if (8 * part < kd) k[i] = *reinterpret_cast<const bf_u32x4*>(k_pool + (head * page_tokens + (key & page_mask)) * kd + 8 * part);
+            // (pieces behind the head's last number bring that one's piece again and are zeroed: no load waits for a branch)
+            k[i] = *reinterpret_cast<const bf_u32x4*>(k_pool + (head * page_tokens + (key & page_mask)) * kd + (FULL ? 8 * part : min(8 * part, kd - 8)));
+            if (!FULL && 8 * part >= kd) k[i] = bf_u32x4{0u, 0u, 0u, 0u};
         }
 #pragma unroll
         for (int i = 0; i < VCH; ++i) {
             const int c = tid + THREADS * i, d = c / (BF_KEYS / 8), part = c % (BF_KEYS / 8);
             const int key = kb + 8 * part;         // eight keys that lie side by side in one page
             bf_u32x4 val = {0u, 0u, 0u, 0u};
-            if (key <= pos_last && d < vd) {
+            if (key <= pos_last) {
                 const size_t head = (static_cast<size_t>(pages[key >> page_shift]) * head_index_stride + layer_index) + kvh;
-                val = *reinterpret_cast<const bf_u32x4*>(v_pool + (head * vd + d) * page_tokens + (key & page_mask));
+                val = *reinterpret_cast<const bf_u32x4*>(v_pool + (head * vd + (FULL ? d : min(d, vd - 1))) * page_tokens + (key & page_mask));
                 const int live = pos_last - key + 1;       // keys of this piece that exist
                 if (live < 8) {
                     if (live <= 6) val[3] = 0u; else val[3] &= 0x0000ffffu;
@@ -84,6 +86,7 @@ struct BfFetch {
                     if (live == 1) val[0] &= 0x0000ffffu;
                 }
             }
+            if (!FULL && d >= vd) val = bf_u32x4{0u, 0u, 0u, 0u};
             v[i] = val;
         }
     }
@@ -181,13 +184,13 @@ __device__ __forceinline__ void bf_block(const __bf16* ks, const __bf16* vs, con
 }
 
 // a finished row: divided by its normaliser, times sigmoid(gate), stored
-template <int V>
+template <int V, bool FULL>
 __device__ __forceinline__ void bf_store(const BfRow<V / 16>& row, float total, const bf16* __restrict__ gate_row, bf16* __restrict__ out_row,
                                          int quad, int vd) {
     const float inv = 1.0f / total;
 #pragma unroll
     for (int dt = 0; dt < V / 16; ++dt) {
-        if (16 * dt + 4 * quad >= vd) continue;
+        if (!FULL && 16 * dt + 4 * quad >= vd) continue;
         float g[4] = {1.f, 1.f, 1.f, 1.f};
         if (gate_row) {
             const bf_bf16x4 g4 = __builtin_bit_cast(bf_bf16x4, *reinterpret_cast<const bf_u32x2*>(gate_row + 16 * dt + 4 * quad));
@@ -256,9 +259,10 @@ __device__ __forceinline__ bool bf_find_tile(const BfArgs& a, int rows, int& til
     return false;
 }
 
-template <int D, int V>
+template <int D, int V, bool FULL>
 __global__ __launch_bounds__(BF_WAVES * CELEG_WAVE) void biased_attention_rows_kernel(const BfArgs a) {
     constexpr int KROW = D + 8, VROW = BF_KEYS + 8, KS = D / 32, DT = V / 16, BUF = BF_KEYS * KROW + V * VROW;
+    const int kd = FULL ? D : a.kd, vd = FULL ? V : a.vd;
     constexpr int THREADS = BF_WAVES * CELEG_WAVE;
     extern __shared__ __attribute__((aligned(16))) unsigned char bf_lds[];
     __bf16* lds = reinterpret_cast<__bf16*>(bf_lds);
@@ -280,11 +284,11 @@ __global__ __launch_bounds__(BF_WAVES * CELEG_WAVE) void biased_attention_rows_k
     const bool biased = a.r1 != nullptr;
     const float b1 = biased ? a.r1[h] : 0.f, b2 = biased ? a.r2[h] : 0.f;
     bf_bf16x8 qreg[KS];
-    const bf16* qrow = a.q + static_cast<size_t>(row0 + safe_row) * a.ldq + static_cast<size_t>(h) * a.kd;
+    const bf16* qrow = a.q + static_cast<size_t>(row0 + safe_row) * a.ldq + static_cast<size_t>(h) * kd;
 #pragma unroll
     for (int st = 0; st < KS; ++st) {
         bf_u32x4 piece = {0u, 0u, 0u, 0u};
-        if (32 * st + 8 * quad < a.kd) piece = *reinterpret_cast<const bf_u32x4*>(qrow + 32 * st + 8 * quad);
+        if (FULL || 32 * st + 8 * quad < kd) piece = *reinterpret_cast<const bf_u32x4*>(qrow + 32 * st + 8 * quad);
         qreg[st] = __builtin_bit_cast(bf_bf16x8, piece);
     }
     BfRow<DT> row;
@@ -296,11 +300,11 @@ __global__ __launch_bounds__(BF_WAVES * CELEG_WAVE) void biased_attention_rows_k
     }
     const int page_shift = 31 - __builtin_clz(a.page_tokens), page_mask = a.page_tokens - 1;
     const size_t head_index_stride = static_cast<size_t>(a.n_layers) * a.kv_heads, layer_index = static_cast<size_t>(a.layer) * a.kv_heads;
-    BfFetch<D, V, THREADS> pre;
+    BfFetch<D, V, THREADS, FULL> pre;
     const BfBlocks blocks(tile_pos0, a.window, a.keep_first);
     const int n_blocks = blocks.count(pos_last);
     pre.load(tid, blocks.start(0), blocks.last(0, pos_last, a.keep_first), a.k_pool, a.v_pool, pages, page_shift, page_mask, a.page_tokens,
-             head_index_stride, kvh, layer_index, a.kd, a.vd);
+             head_index_stride, kvh, layer_index, kd, vd);
     int turn = 0;
     for (int i = 0; i < n_blocks; ++i, turn ^= 1) {
         const int kb = blocks.start(i);
@@ -310,7 +314,7 @@ __global__ __launch_bounds__(BF_WAVES * CELEG_WAVE) void biased_attention_rows_k
         __syncthreads();
         if (i + 1 < n_blocks)
             pre.load(tid, blocks.start(i + 1), blocks.last(i + 1, pos_last, a.keep_first), a.k_pool, a.v_pool, pages, page_shift, page_mask,
-                     a.page_tokens, head_index_stride, kvh, layer_index, a.kd, a.vd);
+                     a.page_tokens, head_index_stride, kvh, layer_index, kd, vd);
         // blocks none of this wavefront's rows can see
         if (rows_here <= 0) continue;
         if (!blocks.kept(i) && (kb > wave_last || (a.window > 0 && kb >= a.keep_first && kb + BF_KEYS - 1 < wave_pos0 - a.window + 1))) continue;
@@ -321,13 +325,14 @@ __global__ __launch_bounds__(BF_WAVES * CELEG_WAVE) void biased_attention_rows_k
     total += __shfl_xor(total, 32, CELEG_WAVE);
     if (r >= rows_here) return;
     const size_t at = static_cast<size_t>(row0 + my_row);
-    bf_store<V>(row, total, a.gate ? a.gate + at * a.ldg + static_cast<size_t>(h) * a.vd : nullptr, a.out + at * a.ldo + static_cast<size_t>(h) * a.vd,
-                quad, a.vd);
+    bf_store<V, FULL>(row, total, a.gate ? a.gate + at * a.ldg + static_cast<size_t>(h) * vd : nullptr, a.out + at * a.ldo + static_cast<size_t>(h) * vd,
+                quad, vd);
 }
 
-template <int D, int V, int WAVES>
+template <int D, int V, int WAVES, bool FULL>
 __global__ __launch_bounds__(WAVES * CELEG_WAVE) void biased_attention_tile_kernel(const BfArgs a) {
     constexpr int KROW = D + 8, VROW = BF_KEYS + 8, KS = D / 32, DT = V / 16, BUF = BF_KEYS * KROW + V * VROW;
+    const int kd = FULL ? D : a.kd, vd = FULL ? V : a.vd;
     extern __shared__ __attribute__((aligned(16))) unsigned char bf_lds[];
     const int wave = threadIdx.x / CELEG_WAVE, lane = threadIdx.x % CELEG_WAVE;
     __bf16* ks = reinterpret_cast<__bf16*>(bf_lds) + static_cast<size_t>(wave) * BUF;
@@ -346,11 +351,11 @@ __global__ __launch_bounds__(WAVES * CELEG_WAVE) void biased_attention_tile_kern
     const bool biased = a.r1 != nullptr;
     const float b1 = biased ? a.r1[h] : 0.f, b2 = biased ? a.r2[h] : 0.f;
     bf_bf16x8 qreg[KS];
-    const bf16* qrow = a.q + static_cast<size_t>(row0 + my_row) * a.ldq + static_cast<size_t>(h) * a.kd;
+    const bf16* qrow = a.q + static_cast<size_t>(row0 + my_row) * a.ldq + static_cast<size_t>(h) * kd;
 #pragma unroll
     for (int st = 0; st < KS; ++st) {
         bf_u32x4 piece = {0u, 0u, 0u, 0u};
-        if (32 * st + 8 * quad < a.kd) piece = *reinterpret_cast<const bf_u32x4*>(qrow + 32 * st + 8 * quad);
+        if (FULL || 32 * st + 8 * quad < kd) piece = *reinterpret_cast<const bf_u32x4*>(qrow + 32 * st + 8 * quad);
         qreg[st] = __builtin_bit_cast(bf_bf16x8, piece);
     }
     BfRow<DT> row;
@@ -362,12 +367,12 @@ __global__ __launch_bounds__(WAVES * CELEG_WAVE) void biased_attention_tile_kern
     }
     const int page_shift = 31 - __builtin_clz(a.page_tokens), page_mask = a.page_tokens - 1;
     const size_t head_index_stride = static_cast<size_t>(a.n_layers) * a.kv_heads, layer_index = static_cast<size_t>(a.layer) * a.kv_heads;
-    BfFetch<D, V, CELEG_WAVE> pre;
+    BfFetch<D, V, CELEG_WAVE, FULL> pre;
     const BfBlocks blocks(pos0, a.window, a.keep_first);
     const int n_blocks = blocks.count(pos_last);
     if (wave < n_blocks)
         pre.load(lane, blocks.start(wave), blocks.last(wave, pos_last, a.keep_first), a.k_pool, a.v_pool, pages, page_shift, page_mask,
-                 a.page_tokens, head_index_stride, kvh, layer_index, a.kd, a.vd);
+                 a.page_tokens, head_index_stride, kvh, layer_index, kd, vd);
     for (int i = wave; i < n_blocks; i += WAVES) {
         __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
         __builtin_amdgcn_wave_barrier();
@@ -377,7 +382,7 @@ __global__ __launch_bounds__(WAVES * CELEG_WAVE) void biased_attention_tile_kern
         __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
         if (i + WAVES < n_blocks)
             pre.load(lane, blocks.start(i + WAVES), blocks.last(i + WAVES, pos_last, a.keep_first), a.k_pool, a.v_pool, pages, page_shift,
-                     page_mask, a.page_tokens, head_index_stride, kvh, layer_index, a.kd, a.vd);
+                     page_mask, a.page_tokens, head_index_stride, kvh, layer_index, kd, vd);
         bf_block<D, V>(ks, vs, qreg, row, blocks.start(i), my_pos, a.window, a.keep_first, blocks.kept(i), r, quad, s2, b1, b2, biased, cap2);
     }
     // the wavefronts' maxima, normalisers and sums meet in LDS (every wavefront's staging area is
@@ -420,25 +425,29 @@ __global__ __launch_bounds__(WAVES * CELEG_WAVE) void biased_attention_tile_kern
     total += __shfl_xor(total, 32, CELEG_WAVE);
     if (r >= rows_here) return;
     const size_t at = static_cast<size_t>(row0 + my_row);
-    bf_store<V>(row, total, a.gate ? a.gate + at * a.ldg + static_cast<size_t>(h) * a.vd : nullptr, a.out + at * a.ldo + static_cast<size_t>(h) * a.vd,
-                quad, a.vd);
+    bf_store<V, FULL>(row, total, a.gate ? a.gate + at * a.ldg + static_cast<size_t>(h) * vd : nullptr, a.out + at * a.ldo + static_cast<size_t>(h) * vd,
+                quad, vd);
 }
 
 constexpr int bf_block_bytes(int d, int v) { return (BF_KEYS * (d + 8) + v * (BF_KEYS + 8)) * 2; }
 // single tiles: eight wavefronts share out the key blocks where their staging areas fit LDS
 constexpr int bf_tile_waves(int d, int v) { return 8 * bf_block_bytes(d, v) <= 160 * 1024 ? 8 : BF_WAVES; }
 
-template <int D, int V>
-int bf_launch(int form, int max_tiles, const BfArgs& a, hipStream_t stream) {
+template <int D, int V, bool FULL>
+int bf_launch_full(int form, int max_tiles, const BfArgs& a, hipStream_t stream) {
     if (form == 1) {
         dim3 grid(max_tiles, a.q_heads), block(BF_WAVES * CELEG_WAVE);
-        hipLaunchKernelGGL((biased_attention_rows_kernel<D, V>), grid, block, 2 * bf_block_bytes(D, V), stream, a);
+        hipLaunchKernelGGL((biased_attention_rows_kernel<D, V, FULL>), grid, block, 2 * bf_block_bytes(D, V), stream, a);
     } else {
         constexpr int WAVES = bf_tile_waves(D, V);
         dim3 grid(max_tiles, a.q_heads), block(WAVES * CELEG_WAVE);
-        hipLaunchKernelGGL((biased_attention_tile_kernel<D, V, WAVES>), grid, block, WAVES * bf_block_bytes(D, V), stream, a);
+        hipLaunchKernelGGL((biased_attention_tile_kernel<D, V, WAVES, FULL>), grid, block, WAVES * bf_block_bytes(D, V), stream, a);
     }
     return CELEG_LAUNCH_RESULT();
+}
+template <int D, int V>
+int bf_launch(int form, int max_tiles, const BfArgs& a, hipStream_t stream) {
+    return a.kd == D && a.vd == V ? bf_launch_full<D, V, true>(form, max_tiles, a, stream) : bf_launch_full<D, V, false>(form, max_tiles, a, stream);
 }
 
 template <int D>

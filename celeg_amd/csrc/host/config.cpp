@@ -1459,7 +1459,8 @@ ModelSpec minilorn_build_spec(const Json& c) {
         } else if (type == "latent_attention") {
             layer.mixer.kind = "latent_attention";
             layer.mixer.params.set("dim", m["dim"]).set("rot_dim", m["rot_dim"]).set("vdim", m["vdim"]).set("q_rank", m["q_rank"])
-                .set("kv_rank", m["kv_rank"]).set("scale", m["scale"]).set("eps", eps).set("sink", false).set("gate", false);
+                .set("kv_rank", m["kv_rank"]).set("scale", m["scale"]).set("eps", eps).set("sink", false).set("gate", false)
+                .set("exact_weights", true);
             if (!m["mask"].is_null()) layer.mixer.params.set("window", m["mask"]["size"]);
             if (!m["rot"].is_null()) {
                 PartSpec rope;

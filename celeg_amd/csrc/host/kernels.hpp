@@ -58,7 +58,8 @@ int celeg_latent_attention_fast(int form, const void* q, int ldq, const void* po
                                 const int* cu_seqlens, const int* seq_slot, const int* seq_start, int n_seqs, int max_tiles,
                                 const int* token_slot, const int* positions, int n_single, const float* sink, void* out,
                                 int ldo, float* ws_o, float* ws_ml, int n_splits, int blocks_per_split, int heads, int rank,
-                                int rot, int page_tokens, int n_layers, int layer, float scale, int window, hipStream_t stream);
+                                int rot, int page_tokens, int n_layers, int layer, float scale, int window, int exact,
+                                hipStream_t stream);
 // moe.hip
 int celeg_moe_route(const float* logits, int rows, int experts, int top, int score, int renorm, int groups, int keep,
                     float renorm_eps, float scale, int* ids, float* weights, hipStream_t stream);

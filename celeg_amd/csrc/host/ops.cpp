@@ -303,7 +303,7 @@ void Ops::latent_attention(const Tensor& q_lat, const Tensor& out, const LatentS
                                                      batch.cu_seqlens, batch.seq_slot, batch.seq_start, batch.n_seqs, 0,
                                                      batch.token_slot, batch.positions, n_single, sink_p, out.data,
                                                      static_cast<int>(out.shape[1]), ws_o, ws_ml, n_splits, per_split, s.heads,
-                                                     s.rank, s.rot, kv.page_tokens, kv.n_layers, kv.layer, scale, window, stream),
+                                                     s.rank, s.rot, kv.page_tokens, kv.n_layers, kv.layer, scale, window, s.exact_weights ? 1 : 0, stream),
                          "latent_attention (single tokens)");
         }
         if (T > n_single) {
@@ -313,7 +313,7 @@ void Ops::latent_attention(const Tensor& q_lat, const Tensor& out, const LatentS
                                                      batch.cu_seqlens, batch.seq_slot, batch.seq_start, batch.n_seqs, max_tiles,
                                                      batch.token_slot, batch.positions, 0, sink_p, out.data,
                                                      static_cast<int>(out.shape[1]), nullptr, nullptr, 1, 0, s.heads, s.rank,
-                                                     s.rot, kv.page_tokens, kv.n_layers, kv.layer, scale, window, stream),
+                                                     s.rot, kv.page_tokens, kv.n_layers, kv.layer, scale, window, s.exact_weights ? 1 : 0, stream),
                          "latent_attention (rows)");
         }
         return;

@@ -291,7 +291,8 @@ public:
                             const KVView& kv, DType dtype) const;
     // attention over a latent cache (one cached row per token: `rank` compressed values, then `rot`
     // rotated key values shared by the heads)
-    struct LatentShape { int heads = 0, dim = 0, rot = 0, rank = 0; };
+    // (exact_weights: in bfloat16 a softmax weight enters the product with the values as two bfloat16 numbers, not one)
+    struct LatentShape { int heads = 0, dim = 0, rot = 0, rank = 0; bool exact_weights = false; };
     // proj [rows, ...] holds the queries [heads, dim + rot] from column q_off and (dkv) [rank + rot] from
     // column dkv_off: the queries' rotated parts are turned in place; with `write` the normed
     // compressed values and the turned key part go to the rows' places in the pages.  q_off < 0: the rows hold no

@@ -477,7 +477,7 @@ private:
 // rank + rot values: the first rank, RMS-normed with a weight of their own, are the compressed
 // row c, the last rot are a key part that every head shares and that is rotated by the
 // position, as the queries' rot part is.  Head i's key is (W_uk[i] c | shared part), its value
-// W_uv[i] c; score = (q . k) * scale over positions 0..p (with "window" n the last n of them); softmax, whose denominator may hold
+// W_uv[i] c ("exact_weights": its softmax weights keep sixteen bits in bfloat16); score = (q . k) * scale over positions 0..p (with "window" n the last n of them); softmax, whose denominator may hold
 // one more term exp(sink_i) (a learned number per head with no key and no value); the heads'
 // results, optionally times sigmoid(W_g h), go through W_o.
 //
@@ -498,6 +498,7 @@ public:
         eps_ = static_cast<float>(p.get_double("eps", 1e-6));
         sink_ = p.get_bool("sink", false);
         gate_ = p.get_bool("gate", false);
+        shape_.exact_weights = p.get_bool("exact_weights", false);
         q_rank_ = p.get_int("q_rank", 0);
         if (q_rank_ < 0) throw SpecError("latent_attention: q_rank is not negative");
         if (!p["window"].is_null()) {

@@ -8,7 +8,8 @@
 // transposed (S^T = K Q^T) with the keys of a block dealt to the accumulator registers so that a
 // lane's eight registers of two score tiles are eight neighbouring keys of one query: they are
 // the operand of O^T = V^T P^T as they stand, no exchange between lanes.  Softmax state (running
-// maximum in the base-2 domain, sum) and the output accumulators are 32-bit.
+// maximum in the base-2 domain, sum) and the output accumulators are 32-bit.  With EXACT a 32-bit weight
+// enters the product with the values as two bfloat16 numbers (its rounding, and what that left), else as one.
 //
 // Form 0, portions of prompts: a workgroup owns 64 rows of one sequence and one head (a wavefront
 // 16 of the rows), keys 0..position of its last row.  Form 1, single tokens: a workgroup owns one
@@ -37,7 +38,7 @@ __device__ __forceinline__ float quad_sum(float v) {
     return v + __shfl_xor(v, 32, 64);
 }
 
-template <int FORM, int KSMAX, int DTMAX, int RT>
+template <int FORM, int KSMAX, int DTMAX, int RT, bool EXACT>
 __global__ __launch_bounds__(256, (KSMAX <= 9 ? 2 : 1)) void latent_attention_mfma_kernel(
     const __bf16* __restrict__ q, int ldq, const __bf16* __restrict__ pool, const int* __restrict__ table, int table_stride,
     const int* __restrict__ cu_seqlens, const int* __restrict__ seq_slot, const int* __restrict__ seq_start, int n_seqs,
@@ -218,7 +219,7 @@ __global__ __launch_bounds__(256, (KSMAX <= 9 ? 2 : 1)) void latent_attention_mf
                         if (live[rt]) sacc[rt][kt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qreg[rt][st], sacc[rt][kt], 0, 0, 0);
                 }
         }
-        lat_bf16x8 pb[RT][2];
+        lat_bf16x8 pb[RT][2], rest[RT][2];
 #pragma unroll
         for (int rt = 0; rt < RT; ++rt) {
             if (kb + LATF_KEYS - 1 > tile_min_limit[rt] || (window > 0 && kb <= tile_limit[rt] - window)) {
@@ -257,10 +258,12 @@ __global__ __launch_bounds__(256, (KSMAX <= 9 ? 2 : 1)) void latent_attention_mf
             l[rt] += psum;
 #pragma unroll
             for (int kp = 0; kp < 2; ++kp)
-                pb[rt][kp] = lat_bf16x8{static_cast<__bf16>(sacc[rt][2 * kp][0]),     static_cast<__bf16>(sacc[rt][2 * kp][1]),
-                                        static_cast<__bf16>(sacc[rt][2 * kp][2]),     static_cast<__bf16>(sacc[rt][2 * kp][3]),
-                                        static_cast<__bf16>(sacc[rt][2 * kp + 1][0]), static_cast<__bf16>(sacc[rt][2 * kp + 1][1]),
-                                        static_cast<__bf16>(sacc[rt][2 * kp + 1][2]), static_cast<__bf16>(sacc[rt][2 * kp + 1][3])};
+#pragma unroll
+                for (int e = 0; e < 8; ++e) {
+                    const float p = sacc[rt][2 * kp + e / 4][e % 4];
+                    pb[rt][kp][e] = static_cast<__bf16>(p);
+                    if (EXACT) rest[rt][kp][e] = static_cast<__bf16>(p - static_cast<float>(pb[rt][kp][e]));
+                }
         }
         // ---- O^T += V^T P^T
 #pragma unroll
@@ -271,7 +274,10 @@ __global__ __launch_bounds__(256, (KSMAX <= 9 ? 2 : 1)) void latent_attention_mf
                     const lat_bf16x8 vf = *reinterpret_cast<const lat_bf16x8*>(sVt + (dt * 16 + c) * LATF_VROW + 32 * kp + 8 * qd);
 #pragma unroll
                     for (int rt = 0; rt < RT; ++rt)
-                        if (live[rt]) oacc[rt][dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pb[rt][kp], oacc[rt][dt], 0, 0, 0);
+                        if (live[rt]) {
+                            oacc[rt][dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pb[rt][kp], oacc[rt][dt], 0, 0, 0);
+                            if (EXACT) oacc[rt][dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, rest[rt][kp], oacc[rt][dt], 0, 0, 0);
+                        }
                 }
             }
     }
@@ -337,14 +343,14 @@ __global__ void latent_attention_join_kernel(const float* __restrict__ ws_o, con
     }
 }
 
-template <int FORM, int KSMAX, int DTMAX, int RT>
+template <int FORM, int KSMAX, int DTMAX, int RT, bool EXACT>
 static int latent_mfma_launch(dim3 grid, size_t lds, hipStream_t stream, const void* q, int ldq, const void* pool,
                               const int* table, int table_stride, const int* cu_seqlens, const int* seq_slot,
                               const int* seq_start, int n_seqs, const int* token_slot, const int* positions,
                               const float* sink, void* out, int ldo, float* ws_o, float* ws_ml, int n_splits,
                               int blocks_per_split, int heads, int rank, int rot, int page_tokens, int n_layers, int layer,
                               float scale_log2e, int window) {
-    auto kernel = latent_attention_mfma_kernel<FORM, KSMAX, DTMAX, RT>;
+    auto kernel = latent_attention_mfma_kernel<FORM, KSMAX, DTMAX, RT, EXACT>;
     if (lds > 64 * 1024) {
         const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(kernel), hipFuncAttributeMaxDynamicSharedMemorySize,
                                                  static_cast<int>(lds));
@@ -371,14 +377,14 @@ extern "C" int celeg_latent_attention_fast_ok(int rank, int rot) {
 
 // form 0: rows of the sequences of more than one token (max_tiles: a bound on their tiles of 64 rows);
 // form 1: rows [0, n_single), each one token of its request, keys in n_splits shares of blocks_per_split
-// blocks of 64; ws_o [n_single, heads, n_splits, rank] and ws_ml [n_single, heads, n_splits, 2] 32-bit.
+// blocks of 64 (of the keys in the row's window); exact: weights as two bfloat16 numbers; ws_o [n_single, heads, n_splits, rank] and ws_ml [n_single, heads, n_splits, 2] 32-bit.
 extern "C" int celeg_latent_attention_fast(int form, const void* q, int ldq, const void* pool, const int* table,
                                            int table_stride, const int* cu_seqlens, const int* seq_slot,
                                            const int* seq_start, int n_seqs, int max_tiles, const int* token_slot,
                                            const int* positions, int n_single, const float* sink, void* out, int ldo,
                                            float* ws_o, float* ws_ml, int n_splits, int blocks_per_split, int heads,
                                            int rank, int rot, int page_tokens, int n_layers, int layer, float scale,
-                                           int window, hipStream_t stream) {
+                                           int window, int exact, hipStream_t stream) {
     if (!celeg_latent_attention_fast_ok(rank, rot) || (form == 1 && n_splits > LATF_MAX_SPLITS) || page_tokens <= 0 ||
         (page_tokens & (page_tokens - 1)))
         return static_cast<int>(hipErrorInvalidValue);
@@ -387,32 +393,21 @@ extern "C" int celeg_latent_attention_fast(int form, const void* q, int ldq, con
     const float scale_log2e = scale * LOG2E;
     if (form == 0 ? max_tiles <= 0 : n_single <= 0) return 0;
     const dim3 grid = form == 0 ? dim3(max_tiles, heads) : dim3(n_single, (heads + 15) / 16, n_splits);
-#define LATF_GO(FORM, KSM, DTM, RT)                                                                                            \
-    return latent_mfma_launch<FORM, KSM, DTM, RT>(grid, lds, stream, q, ldq, pool, table, table_stride, cu_seqlens, seq_slot,  \
-                                              seq_start, n_seqs, token_slot, positions, sink, out, ldo, ws_o, ws_ml,       \
-                                              n_splits, blocks_per_split, heads, rank, rot, page_tokens, n_layers, layer,  \
-                                              scale_log2e, window)
-    if (form == 0) {
-        if (KS <= 5 && DT <= 8) LATF_GO(0, 5, 8, 1);
-        if (KS <= 9 && DT <= 16) LATF_GO(0, 9, 16, 1);
-        LATF_GO(0, 18, 32, 1);
-    }
-    int rc;
-    if (KS <= 5 && DT <= 8)
-        rc = latent_mfma_launch<1, 5, 8, 1>(grid, lds, stream, q, ldq, pool, table, table_stride, cu_seqlens, seq_slot, seq_start,
-                                         n_seqs, token_slot, positions, sink, out, ldo, ws_o, ws_ml, n_splits, blocks_per_split,
-                                         heads, rank, rot, page_tokens, n_layers, layer, scale_log2e, window);
-    else if (KS <= 9 && DT <= 16)
-        rc = latent_mfma_launch<1, 9, 16, 1>(grid, lds, stream, q, ldq, pool, table, table_stride, cu_seqlens, seq_slot, seq_start,
-                                          n_seqs, token_slot, positions, sink, out, ldo, ws_o, ws_ml, n_splits, blocks_per_split,
-                                          heads, rank, rot, page_tokens, n_layers, layer, scale_log2e, window);
-    else
-        rc = latent_mfma_launch<1, 18, 32, 1>(grid, lds, stream, q, ldq, pool, table, table_stride, cu_seqlens, seq_slot,
-                                           seq_start, n_seqs, token_slot, positions, sink, out, ldo, ws_o, ws_ml, n_splits,
-                                           blocks_per_split, heads, rank, rot, page_tokens, n_layers, layer, scale_log2e, window);
+#define LATF_GO(FORM, KSM, DTM, EXACT)                                                                                      \
+    latent_mfma_launch<FORM, KSM, DTM, 1, EXACT>(grid, lds, stream, q, ldq, pool, table, table_stride, cu_seqlens, seq_slot, \
+                                                 seq_start, n_seqs, token_slot, positions, sink, out, ldo, ws_o, ws_ml,      \
+                                                 n_splits, blocks_per_split, heads, rank, rot, page_tokens, n_layers, layer, \
+                                                 scale_log2e, window)
+#define LATF_SIZES(FORM)                                                                        \
+    (KS <= 5 && DT <= 8    ? (exact ? LATF_GO(FORM, 5, 8, true) : LATF_GO(FORM, 5, 8, false))   \
+     : KS <= 9 && DT <= 16 ? (exact ? LATF_GO(FORM, 9, 16, true) : LATF_GO(FORM, 9, 16, false)) \
+                           : (exact ? LATF_GO(FORM, 18, 32, true) : LATF_GO(FORM, 18, 32, false)))
+    if (form == 0) return LATF_SIZES(0);
+    const int rc = LATF_SIZES(1);
     if (rc) return rc;
     hipLaunchKernelGGL(latent_attention_join_kernel, dim3(n_single, heads), dim3(128), 0, stream, ws_o, ws_ml, n_splits, sink,
                        static_cast<__bf16*>(out), ldo, heads, rank);
     return CELEG_LAUNCH_RESULT();
+#undef LATF_SIZES
 #undef LATF_GO
 }

@@ -35,6 +35,22 @@ __global__ void activation_bias_kernel(const T* __restrict__ x, int ldx, const f
     out[static_cast<size_t>(t) * ldo + c] = from_float<T>(y);
 }
 
+// The same without a bias on dense rows of the run's dtype that lie one after the other: eight values a thread.
+template <typename T>
+__global__ __launch_bounds__(256) void activation_dense_kernel(const T* __restrict__ x, T* __restrict__ out, size_t groups, int act, float p0,
+                                                               float p1) {
+    struct alignas(8 * sizeof(T)) Eight { T v[8]; };
+    const size_t i = static_cast<size_t>(blockIdx.x) * 256 + threadIdx.x;
+    if (i >= groups) return;
+    Eight in = reinterpret_cast<const Eight*>(x)[i];
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+        const float z = to_float(in.v[e]);
+        in.v[e] = from_float<T>(act == 0 ? lg_gelu_tanh(z) : act == 1 ? lg_relu2(z) : act == 3 ? lg_bent(z, p0, p1) : z);
+    }
+    reinterpret_cast<Eight*>(out)[i] = in;
+}
+
 // h += a (+ b); copy (optional) receives the new rows in the run's dtype
 template <typename T>
 __global__ void residual_sum_kernel(float* __restrict__ h, const T* __restrict__ a, int lda, const T* __restrict__ b, int ldb,
@@ -129,6 +145,13 @@ __global__ void softcap_kernel(float* __restrict__ x, size_t n, float cap) {
 extern "C" int celeg_activation_bias(const void* x, int ldx, const float* bias, void* out, int ldo, int dtype, int rows, int cols,
                                      int act, float p0, float p1, hipStream_t stream) {
     if (rows <= 0 || cols <= 0) return 0;
+    const size_t piece = 8 * (dtype == CELEG_F32 ? 4 : 2), count = static_cast<size_t>(rows) * cols;
+    if (!bias && count % 8 == 0 && (rows == 1 || (ldx == cols && ldo == cols)) &&
+        ((reinterpret_cast<uintptr_t>(x) | reinterpret_cast<uintptr_t>(out)) & (piece - 1)) == 0) {
+        dim3 grid(static_cast<unsigned>((count / 8 + 255) / 256)), block(256);
+        LG_BY_DTYPE(activation_dense_kernel, grid, block, static_cast<const T*>(x), static_cast<T*>(out), count / 8, act, p0, p1);
+        return CELEG_LAUNCH_RESULT();
+    }
     dim3 grid((cols + 255) / 256, rows), block(256);
     LG_BY_DTYPE(activation_bias_kernel, grid, block, static_cast<const T*>(x), ldx, bias, static_cast<T*>(out), ldo, cols, act, p0, p1);
     return CELEG_LAUNCH_RESULT();
