@@ -100,6 +100,11 @@ def write_model(folder, cfg, seed, storage=torch.float32, std=STD, change=None):
             tensors[name] = 1.2 * unit
         elif name in ("embed", "bigram"):
             tensors[name] = 3.0 * tensors[name]
+    # a memory read with a query at right angles to its keys is a small number that the norm behind it makes large,
+    # sign and all: keys that lean towards the queries keep rounding from deciding such rows
+    for name in [n for n in tensors if n.endswith(".mix.i")]:
+        p = name[:-1]
+        tensors[p + "k"] = 0.5 * tensors[p + "k"] + 0.9 * tensors[p + "q"]
     for name, fn in (change or {}).items():
         tensors[name] = fn(tensors[name])
     tensors = {k: v.to(storage).contiguous() for k, v in tensors.items()}
