@@ -1,6 +1,6 @@
 // The registries of parts and block arrangements, and the parts this library brings:
 // RMS norm, rotary and no position encoding, grouped-query attention over the paged cache,
-// attention over a latent cache, the double-gated short convolution, the SwiGLU feed-forward,
+// attention over a latent cache, recurrent mixers, the double-gated short convolution, the SwiGLU feed-forward,
 // routed experts, token embedding, tied and own output head, the pre-norm block and the block
 // on several residual streams; beside them the neutral parts ("none" mixer and
 // feed-forward, "identity" norm, "hidden" head) with which a test runs a single part alone

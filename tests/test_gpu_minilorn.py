@@ -299,6 +299,35 @@ def test_long_decoding_while_the_window_passes(folders, dtype):
     assert lm.runner.counters()["graph_replays"] > 100
 
 
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_portions_replayed_from_a_recorded_graph(folders, dtype):
+    """Portions of 70 tokens of three requests, one after the other and with single tokens of another request
+    between them: from the second on they are replayed from a recorded graph (a chunk of the memory and six rows
+    of a second one), and every portion's last logits are the plain ones."""
+    from celeg_amd.engine import StepEntry, load_model
+    folder = folders("M1", dtype)
+    c, W = plain.load_model_folder(folder)
+    lm = load_model(folder, dtype=dtype, device=DEV, page_tokens=16, n_pages=64, max_requests=3, max_context=256, max_batched_tokens=128)
+    other = random_tokens(M1["vocab"], 9, seed=90)
+    other_slot, at = lm.cache.open(), 0
+    other_ref = plain.model_logits(c, W, other)
+    for r in range(3):
+        toks = random_tokens(M1["vocab"], 210, seed=91 + r)
+        ref = plain.model_logits(c, W, toks)
+        slot = lm.cache.open()
+        for start in (0, 70, 140):
+            assert lm.cache.prepare(slot, start, 70)
+            got = lm.runner.step([StepEntry(slot, start, toks[start:start + 70], [69])]).detach().cpu()
+            assert_close(got[0], ref[start + 69], dtype, f"request {r}, portion from {start}")
+            assert lm.cache.prepare(other_slot, at, 1)
+            single = lm.runner.step([StepEntry(other_slot, at, other[at:at + 1], [0])]).detach().cpu()
+            assert_close(single[0], other_ref[at], dtype, f"single token {at}")
+            at += 1
+        lm.cache.close(slot)
+    assert lm.runner.counters()["graph_replays"] >= 16
+    lm.close()
+
+
 def test_pages_of_the_passed_window_return(folders):
     """While a request grows, the group of the windowed compressed rows holds the pages of the window only;
     the other groups hold all."""
