@@ -313,22 +313,32 @@ extern "C" int celeg_rmsnorm(void* x, int x_dtype, const void* delta, int delta_
 // ---------------------------------------------------------------- SwiGLU
 // out[t, i] = silu(gu[t, i]) * gu[t, ff + i], silu(g) = g / (1 + exp(-g)); computed in
 // 32-bit and rounded once.  Reference: src/backend/cpu/kernels/elementwise.cpp:101-119.
+// limit > 0: the clamped form g sigmoid(alpha g) (u + 1), g = min(gate, limit), u = clamp(up, -limit, limit).
+__device__ __forceinline__ float swiglu_of(float g, float u, float limit, float alpha) {
+    if (limit > 0.f) {
+        g = fminf(g, limit);
+        u = fminf(fmaxf(u, -limit), limit) + 1.0f;
+        return (g / (1.0f + expf(-alpha * g))) * u;
+    }
+    return (g / (1.0f + expf(-g))) * u;
+}
+
 template <typename T>
 __global__ void swiglu_kernel(const T* __restrict__ gu, T* __restrict__ out, int ff,
-                              size_t total) {
+                              size_t total, float limit, float alpha) {
     const size_t i = static_cast<size_t>(blockIdx.x) * blockDim.x + threadIdx.x;
     if (i >= total) return;
     const size_t t = i / ff;
     const int c = static_cast<int>(i - t * ff);
     const float g = to_float(gu[t * 2 * ff + c]);
     const float u = to_float(gu[t * 2 * ff + ff + c]);
-    out[i] = from_float<T>((g / (1.0f + expf(-g))) * u);
+    out[i] = from_float<T>(swiglu_of(g, u, limit, alpha));
 }
 
 // groups of 8 values a thread (ff % 8 == 0)
 template <typename T>
 __global__ __launch_bounds__(256) void swiglu_vec_kernel(const T* __restrict__ gu, T* __restrict__ out,
-                                                         int ff, size_t groups) {
+                                                         int ff, size_t groups, float limit, float alpha) {
     const size_t i = static_cast<size_t>(blockIdx.x) * blockDim.x + threadIdx.x;
     if (i >= groups) return;
     const int per_row = ff >> 3;
@@ -343,12 +353,12 @@ __global__ __launch_bounds__(256) void swiglu_vec_kernel(const T* __restrict__ g
 #pragma unroll
     for (int h = 0; h < 2; ++h) {
 #pragma unroll
-        for (int e = 0; e < 4; ++e) o[h][e] = (g[h][e] / (1.0f + expf(-g[h][e]))) * u[h][e];
+        for (int e = 0; e < 4; ++e) o[h][e] = swiglu_of(g[h][e], u[h][e], limit, alpha);
         Vec4<T>::store(out + t * ff + c + 4 * h, o[h]);
     }
 }
 
-extern "C" int celeg_swiglu(const void* gu, void* out, int dtype, int rows, int ff,
+extern "C" int celeg_swiglu(const void* gu, void* out, int dtype, int rows, int ff, float limit, float alpha,
                             hipStream_t stream) {
     const size_t total = static_cast<size_t>(rows) * ff;
     if (total == 0) return 0;
@@ -357,19 +367,19 @@ extern "C" int celeg_swiglu(const void* gu, void* out, int dtype, int rows, int 
         dim3 vblock(256), vgrid(static_cast<unsigned>((groups + 255) / 256));
         if (dtype == CELEG_F32)
             hipLaunchKernelGGL(swiglu_vec_kernel<float>, vgrid, vblock, 0, stream,
-                               static_cast<const float*>(gu), static_cast<float*>(out), ff, groups);
+                               static_cast<const float*>(gu), static_cast<float*>(out), ff, groups, limit, alpha);
         else
             hipLaunchKernelGGL(swiglu_vec_kernel<bf16>, vgrid, vblock, 0, stream,
-                               static_cast<const bf16*>(gu), static_cast<bf16*>(out), ff, groups);
+                               static_cast<const bf16*>(gu), static_cast<bf16*>(out), ff, groups, limit, alpha);
         return CELEG_LAUNCH_RESULT();
     }
     dim3 block(256), grid(static_cast<unsigned>((total + 255) / 256));
     if (dtype == CELEG_F32)
         hipLaunchKernelGGL(swiglu_kernel<float>, grid, block, 0, stream,
-                           static_cast<const float*>(gu), static_cast<float*>(out), ff, total);
+                           static_cast<const float*>(gu), static_cast<float*>(out), ff, total, limit, alpha);
     else
         hipLaunchKernelGGL(swiglu_kernel<bf16>, grid, block, 0, stream,
-                           static_cast<const bf16*>(gu), static_cast<bf16*>(out), ff, total);
+                           static_cast<const bf16*>(gu), static_cast<bf16*>(out), ff, total, limit, alpha);
     return CELEG_LAUNCH_RESULT();
 }
 

@@ -1519,6 +1519,289 @@ ModelSpec minilorn_build_spec(const Json& c) {
 
 }  // namespace
 
+// ---------------------------------------------------------------------------- Nosalorn
+// A pre-norm decoder (RMS norms, plain sums) of three kinds of mixer (windowed attention with kept first keys, stretched
+// rotations and values mixed with those of the first layer that mixes; linear attention with fixed decays; Mamba-2),
+// dense or routed feed-forwards, a scaled embedding and scaled logits.  config.json describes every layer by itself:
+//   {"architecture": "Nosalorn", "vocab", "width", "norm": {"eps"}, "embedding": {"scale"} (absent: 1),
+//    "logit_scale" (absent: 1), "max_context" (an engine limit; optional),
+//    "layers": [{"type": "attention",
+//                "mixer": {"heads", "kv_heads" (absent: heads), "dim", "vdim" (absent: dim), "scale", "v_mix" (absent: false),
+//                          "rot": {"base", "dims", "scaling": {"factor", "original", "fast", "slow"} (absent: none)} (absent, or
+//                          dims 0: no rotation; the halves of the rotated part pair),
+//                          "mask": {"size", "keep_first" (absent: 0)} (absent: every earlier key)},
+//                "mlp": null | {"kind": "dense", "ff"}
+//                            | {"kind": "moe", "expert": {"ff", "limit"}, "shared": {"ff", "limit"} (absent or null: none),
+//                               "router": {"experts", "top", "scale" (absent: 1), "identity" (absent: 0),
+//                                          "groups": {"count", "keep"} (absent: one group)}}},
+//               {"type": "lightning", "mixer": {"heads", "dim", "vdim" (absent: dim), "decay": [a number per head]}, "mlp": ...},
+//               {"type": "mamba2", "mixer": {"heads", "vdim", "state", "groups" (absent: 1), "conv", "norm_groups" (absent: 1)},
+//                "mlp": ...}]}
+// Tensors: embed, head, final.norm, l<i>.norm1, l<i>.norm2; attention: l<i>.mix.{q, k, v, q.b, k.b, v.b, o, vmix}; lightning:
+// l<i>.mix.{q, k, v, g, norm, o}; mamba2: l<i>.mix.{in, conv, conv.b, dt_bias, A_log, D, norm, o}; l<i>.mlp.{gate, up, down} or
+// l<i>.mlp.{router, correction}, l<i>.mlp.e<j>.{gate, up, down}, l<i>.mlp.shared.{gate, up, down, sg}.
+namespace {
+
+constexpr double NOSALORN_SWISH = 1.702;       // what a clamped gate is multiplied by inside its sigmoid
+
+Json nosalorn_read_config(const Json& raw, const TensorShapes* shapes) {
+    if (!raw.is_object()) throw ConfigError("config.json is not an object");
+    Json out = Json::object();
+    out.set("architecture", "Nosalorn");
+    out.set("vocab", regipel_int(raw, "vocab", ""));
+    out.set("width", regipel_int(raw, "width", ""));
+    const double eps = regipel_number(regipel_object(raw, "norm", ""), "eps", "norm.");
+    if (!(eps > 0)) throw ConfigError("config.json: 'norm.eps' must be positive");
+    out.set("norm", Json::object().set("eps", eps));
+    double embedding_scale = 1.0;
+    if (!raw["embedding"].is_null()) {
+        const Json& e = regipel_object(raw, "embedding", "");
+        if (!e["scale"].is_null()) embedding_scale = regipel_number(e, "scale", "embedding.");
+    }
+    out.set("embedding", Json::object().set("scale", embedding_scale));
+    out.set("logit_scale", raw["logit_scale"].is_null() ? 1.0 : regipel_number(raw, "logit_scale", ""));
+    out.set("max_context", raw["max_context"].is_null() ? 131072LL : regipel_int(raw, "max_context", ""));
+    if (!raw["layers"].is_array() || raw["layers"].size() == 0) throw ConfigError("config.json: 'layers' must be a list of layers");
+    Json layers = Json::array();
+    int i = 0;
+    long long mixed_width = 0;       // values a token of the layers that mix theirs
+    for (const Json& l : raw["layers"].items()) {
+        const std::string where = "layers[" + std::to_string(i++) + "].";
+        if (!l.is_object()) throw ConfigError("config.json: " + where + " must be an object");
+        const std::string type = l.get_string("type", "");
+        if (type != "attention" && type != "lightning" && type != "mamba2")
+            throw ConfigError("config.json: " + where + "'type' is '" + type + "'; known types are ['attention', 'lightning', 'mamba2']");
+        const Json& m = regipel_object(l, "mixer", where);
+        const std::string mw = where + "mixer.";
+        const long long heads = regipel_int(m, "heads", mw);
+        Json mixer = Json::object().set("heads", heads);
+        if (type == "attention") {
+            const long long dim = regipel_int(m, "dim", mw), vdim = m["vdim"].is_null() ? dim : regipel_int(m, "vdim", mw);
+            const long long kv_heads = m["kv_heads"].is_null() ? heads : regipel_int(m, "kv_heads", mw);
+            if (heads % kv_heads) throw ConfigError("config.json: " + mw + "'heads' must be a multiple of 'kv_heads'");
+            if (vdim > 256) throw ConfigError("config.json: " + mw + "'vdim' may be at most 256");
+            if (dim > 1024) throw ConfigError("config.json: " + mw + "'dim' may be at most 1024");
+            mixer.set("kv_heads", kv_heads).set("dim", dim).set("vdim", vdim).set("scale", regipel_number(m, "scale", mw));
+            Json rot = vabuzen_rot(m, mw, dim, "dim");
+            if (!rot.is_null()) {
+                Json scaling;
+                const Json& given = m["rot"]["scaling"];
+                if (!given.is_null()) {
+                    const Json& sc = regipel_object(m["rot"], "scaling", mw + "rot.");
+                    const std::string sw = mw + "rot.scaling.";
+                    scaling = Json::object();
+                    for (const char* key : {"factor", "original", "fast", "slow"}) {
+                        const double v = regipel_number(sc, key, sw);
+                        if (!(v > 0)) throw ConfigError("config.json: " + sw + "'" + key + "' must be positive");
+                        scaling.set(key, v);
+                    }
+                    if (!(rot["base"].as_double() > 1)) throw ConfigError("config.json: " + mw + "'rot.base' must be above 1 where frequencies are scaled");
+                }
+                rot.set("scaling", scaling);
+            }
+            mixer.set("rot", rot);
+            Json mask;
+            if (!m["mask"].is_null()) {
+                const Json& k = regipel_object(m, "mask", mw);
+                mask = Json::object().set("size", regipel_int(k, "size", mw + "mask."))
+                           .set("keep_first", k["keep_first"].is_null() ? 0LL : regipel_int(k, "keep_first", mw + "mask.", 0));
+            }
+            mixer.set("mask", mask);
+            // the first layer that mixes keeps its values, the later ones mix theirs with them
+            std::string v_mix = "none";
+            if (m.get_bool("v_mix", false)) {
+                v_mix = mixed_width == 0 ? "keep" : "mix";
+                if (mixed_width != 0 && mixed_width != kv_heads * vdim)
+                    throw ConfigError("config.json: " + mw + "'v_mix': all layers that mix values must have as many of them ('kv_heads' times 'vdim')");
+                mixed_width = kv_heads * vdim;
+            }
+            const bool stored = v_mix == "mix" || (v_mix == "keep" && (!shapes || shapes->count("l" + std::to_string(i - 1) + ".mix.vmix")));
+            mixer.set("v_mix", v_mix).set("vmix_stored", stored);
+        } else if (type == "lightning") {
+            const long long dim = regipel_int(m, "dim", mw), vdim = m["vdim"].is_null() ? dim : regipel_int(m, "vdim", mw);
+            if (dim > 256) throw ConfigError("config.json: " + mw + "'dim' may be at most 256");
+            if (vdim > 4096) throw ConfigError("config.json: " + mw + "'vdim' may be at most 4096");
+            if (!m["decay"].is_array() || static_cast<long long>(m["decay"].size()) != heads)
+                throw ConfigError("config.json: " + mw + "'decay' must list a number per head");
+            for (const Json& d : m["decay"].items())
+                if (!d.is_number() || !(d.as_double() > 0) || d.as_double() > 1)
+                    throw ConfigError("config.json: " + mw + "'decay' holds numbers above 0 and at most 1");
+            mixer.set("dim", dim).set("vdim", vdim).set("decay", m["decay"]);
+        } else {
+            const long long vdim = regipel_int(m, "vdim", mw), state = regipel_int(m, "state", mw);
+            const long long groups = m["groups"].is_null() ? 1LL : regipel_int(m, "groups", mw);
+            const long long norm_groups = m["norm_groups"].is_null() ? 1LL : regipel_int(m, "norm_groups", mw);
+            if (heads % groups) throw ConfigError("config.json: " + mw + "'heads' must be a multiple of 'groups'");
+            if ((heads * vdim) % norm_groups) throw ConfigError("config.json: " + mw + "'norm_groups' must divide 'heads' times 'vdim'");
+            if (state > 256) throw ConfigError("config.json: " + mw + "'state' may be at most 256");
+            if (vdim > 4096) throw ConfigError("config.json: " + mw + "'vdim' may be at most 4096");
+            mixer.set("vdim", vdim).set("state", state).set("groups", groups).set("norm_groups", norm_groups)
+                .set("conv", regipel_int(m, "conv", mw));
+        }
+        Json mlp;
+        if (!l["mlp"].is_null()) {
+            const Json& f = regipel_object(l, "mlp", where);
+            const std::string fw = where + "mlp.", kind = f.get_string("kind", "");
+            // an expert's sizes and constants
+            auto expert = [&](const char* key) {
+                const Json& e = regipel_object(f, key, fw);
+                const std::string ew = fw + key + ".";
+                const double limit = regipel_number(e, "limit", ew);
+                if (!(limit > 0)) throw ConfigError("config.json: " + ew + "'limit' must be positive");
+                return Json::object().set("ff", regipel_int(e, "ff", ew)).set("limit", limit);
+            };
+            if (kind == "dense") {
+                mlp = Json::object().set("kind", kind).set("ff", regipel_int(f, "ff", fw));
+            } else if (kind == "moe") {
+                const Json& router = regipel_object(f, "router", fw);
+                const std::string rw = fw + "router.";
+                const long long experts = regipel_int(router, "experts", rw), top = regipel_int(router, "top", rw);
+                const long long identity = router["identity"].is_null() ? 0LL : regipel_int(router, "identity", rw, 0);
+                const long long outputs = experts + identity;
+                if (top > outputs) throw ConfigError("config.json: " + rw + "'top' exceeds 'experts' and 'identity' together");
+                if (outputs > 512) throw ConfigError("config.json: " + rw + "'experts' and 'identity' may be at most 512 together");
+                long long count = 1, keep = 1;
+                if (!router["groups"].is_null()) {
+                    const Json& g = regipel_object(router, "groups", rw);
+                    count = regipel_int(g, "count", rw + "groups.");
+                    keep = regipel_int(g, "keep", rw + "groups.");
+                    if (count > 64 || outputs % count || keep > count)
+                        throw ConfigError("config.json: " + rw + "'groups.count' (at most 64) must divide 'experts' and 'identity' together, and 'groups.keep' may be at most 'groups.count'");
+                    if (top > keep * (outputs / count)) throw ConfigError("config.json: " + rw + "the kept groups hold fewer experts than 'top'");
+                }
+                mlp = Json::object().set("kind", kind).set("expert", expert("expert"))
+                          .set("router", Json::object().set("experts", experts).set("top", top).set("identity", identity)
+                                             .set("scale", router["scale"].is_null() ? 1.0 : regipel_number(router, "scale", rw))
+                                             .set("groups", Json::object().set("count", count).set("keep", keep)))
+                          .set("shared", f["shared"].is_null() ? Json() : expert("shared"));
+            } else {
+                throw ConfigError("config.json: " + fw + "'kind' is '" + kind + "'; known kinds are ['dense', 'moe']");
+            }
+        }
+        layers.push(Json::object().set("type", type).set("mixer", mixer).set("mlp", mlp));
+    }
+    out.set("layers", layers);
+    for (const char* key : {"bos_token_id", "eos_token_id"})
+        if (!raw[key].is_null()) out.set(key, raw[key]);
+    return out;
+}
+
+ModelSpec nosalorn_build_spec(const Json& c) {
+    const long long W = c["width"].as_int();
+    const double eps = c["norm"]["eps"].as_double();
+    auto norm = [&](const std::string& name) {
+        PartSpec p;
+        p.kind = "rmsnorm";
+        p.params = Json::object().set("width", W).set("eps", eps);
+        p.tensors = {{"weight", name}};
+        return p;
+    };
+    ModelSpec spec;
+    int i = 0;
+    for (const Json& l : c["layers"].items()) {
+        const std::string p = "l" + std::to_string(i) + ".", type = l["type"].as_string();
+        const Json& m = l["mixer"];
+        LayerSpec layer;
+        layer.arrangement = "pre_norm";
+        layer.mixer.params = Json::object().set("width", W).set("heads", m["heads"]);
+        auto tensors = [&](std::initializer_list<const char*> roles) {
+            for (const char* role : roles) layer.mixer.tensors.emplace_back(role, p + "mix." + role);
+        };
+        if (type == "attention") {
+            layer.mixer.kind = "biased_attention";
+            layer.mixer.params.set("kv_heads", m["kv_heads"]).set("head_dim", m["dim"]).set("v_dim", m["vdim"]).set("scale", m["scale"])
+                .set("bias", true).set("value_mix", m["v_mix"]);
+            if (!m["mask"].is_null()) layer.mixer.params.set("window", m["mask"]["size"]).set("keep_first", m["mask"]["keep_first"]);
+            if (!m["rot"].is_null()) {
+                PartSpec rope;
+                rope.kind = "rope";
+                rope.params = Json::object().set("theta", m["rot"]["base"]).set("rotary_dim", m["rot"]["dims"])
+                                  .set("head_dim", m["dim"]).set("pairing", "halves");
+                if (!m["rot"]["scaling"].is_null()) {
+                    Json scaling = m["rot"]["scaling"];
+                    rope.params.set("scaling", scaling.set("kind", "yarn"));
+                }
+                layer.mixer.params.set("position", rope.to_json());
+            }
+            tensors({"q", "k", "v", "o"});
+            for (const char* t : {"q", "k", "v"}) layer.mixer.tensors.emplace_back(std::string(t) + "_bias", p + "mix." + t + ".b");
+            if (m["vmix_stored"].as_bool()) layer.mixer.tensors.emplace_back("mix", p + "mix.vmix");
+        } else if (type == "lightning") {
+            layer.mixer.kind = "fixed_decay_attention";
+            layer.mixer.params.set("dim", m["dim"]).set("vdim", m["vdim"]).set("decay", m["decay"]).set("eps", eps);
+            tensors({"q", "k", "v", "g", "norm", "o"});
+        } else {
+            layer.mixer.kind = "state_space";
+            layer.mixer.params.set("vdim", m["vdim"]).set("state", m["state"]).set("groups", m["groups"]).set("taps", m["conv"])
+                .set("norm_groups", m["norm_groups"]).set("eps", eps);
+            tensors({"in", "conv", "dt_bias", "A_log", "D", "norm", "o"});
+            layer.mixer.tensors.emplace_back("conv_bias", p + "mix.conv.b");
+        }
+        layer.mixer_norm = norm(p + "norm1");
+        if (l["mlp"].is_null()) {
+            layer.ffn.kind = "none";
+            layer.ffn_norm.kind = "identity";
+        } else {
+            const Json& f = l["mlp"];
+            if (f["kind"].as_string() == "dense") {
+                layer.ffn.kind = "swiglu";
+                layer.ffn.params = Json::object().set("width", W).set("ff", f["ff"]);
+                for (const char* t : {"gate", "up", "down"}) layer.ffn.tensors.emplace_back(t, p + "mlp." + t);
+            } else {
+                const Json& r = f["router"];
+                const long long experts = r["experts"].as_int();
+                layer.ffn.kind = "routed_experts";
+                layer.ffn.params = Json::object().set("width", W).set("ff", f["expert"]["ff"]).set("experts", experts)
+                                       .set("identity", r["identity"]).set("top", r["top"]).set("score", "softmax")
+                                       .set("renormalize", false).set("route_scale", r["scale"]).set("groups", r["groups"])
+                                       .set("group_score", "best").set("correction", true).set("weight_on", "output")
+                                       .set("activation", "clamped").set("limit", f["expert"]["limit"]).set("alpha", NOSALORN_SWISH);
+                layer.ffn.tensors = {{"router", p + "mlp.router"}, {"correction", p + "mlp.correction"}};
+                for (long long e = 0; e < experts; ++e) {
+                    const std::string ep = p + "mlp.e" + std::to_string(e) + ".", n = std::to_string(e);
+                    layer.ffn.tensors.emplace_back("gate." + n, ep + "gate");
+                    layer.ffn.tensors.emplace_back("up." + n, ep + "up");
+                    layer.ffn.tensors.emplace_back("down." + n, ep + "down");
+                }
+                if (!f["shared"].is_null()) {
+                    PartSpec shared;
+                    shared.kind = "swiglu";
+                    shared.params = Json::object().set("width", W).set("ff", f["shared"]["ff"]).set("activation", "clamped")
+                                        .set("limit", f["shared"]["limit"]).set("alpha", NOSALORN_SWISH);
+                    layer.ffn.params.set("shared", shared.to_json()).set("shared_gate", true);
+                    for (const char* t : {"gate", "up", "down"})
+                        layer.ffn.tensors.emplace_back(std::string("shared.") + t, p + "mlp.shared." + t);
+                    layer.ffn.tensors.emplace_back("shared_gate", p + "mlp.shared.sg");
+                }
+            }
+            layer.ffn_norm = norm(p + "norm2");
+        }
+        spec.layers.push_back(std::move(layer));
+        spec.order.push_back(RunStep{i, {}, false, 0});
+        ++i;
+    }
+    spec.architecture = "Nosalorn";
+    spec.vocab_size = static_cast<int>(c["vocab"].as_int());
+    spec.hidden_size = static_cast<int>(W);
+    spec.max_context = static_cast<int>(c["max_context"].as_int());
+    spec.embedding.kind = "embedding";
+    spec.embedding.params = Json::object().set("vocab", c["vocab"]).set("width", W).set("scale", c["embedding"]["scale"]);
+    spec.embedding.tensors = {{"table", "embed"}};
+    spec.head.kind = "linear_head";
+    spec.head.params = Json::object().set("vocab", c["vocab"]).set("width", W).set("scale", c["logit_scale"]);
+    spec.head.tensors = {{"weight", "head"}};
+    spec.final_norm = norm("final.norm");
+    if (c["eos_token_id"].is_array())
+        for (const Json& e : c["eos_token_id"].items()) spec.eos_token_ids.push_back(static_cast<int>(e.as_int()));
+    else if (c["eos_token_id"].is_int())
+        spec.eos_token_ids.push_back(static_cast<int>(c["eos_token_id"].as_int()));
+    if (c["bos_token_id"].is_int()) spec.bos_token_id = static_cast<int>(c["bos_token_id"].as_int());
+    spec.validate();
+    return spec;
+}
+
+}  // namespace
+
 namespace {
 void register_builtin() {
     Architecture lfm2;
@@ -1564,6 +1847,13 @@ void register_builtin() {
     minilorn.build_spec = minilorn_build_spec;
     table()["Minilorn"] = minilorn;
     table()["minilorn"] = minilorn;
+    Architecture nosalorn;
+    nosalorn.name = "Nosalorn";
+    nosalorn.aliases = {"nosalorn"};
+    nosalorn.read_config = nosalorn_read_config;
+    nosalorn.build_spec = nosalorn_build_spec;
+    table()["Nosalorn"] = nosalorn;
+    table()["nosalorn"] = nosalorn;
 }
 
 }  // namespace

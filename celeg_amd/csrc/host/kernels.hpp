@@ -23,7 +23,7 @@ int celeg_embed_pairs(const void* table, const void* pairs, int table_dtype, con
                       float* stats, int stats_ld, int rows, int width, int vocab, hipStream_t stream);
 int celeg_rmsnorm(void* x, int x_dtype, const void* delta, int delta_dtype, const float* w, void* out, int out_dtype,
                   const int* rows, int n_rows, int width, float eps, int write_back, hipStream_t stream);
-int celeg_swiglu(const void* gu, void* out, int dtype, int rows, int ff, hipStream_t stream);
+int celeg_swiglu(const void* gu, void* out, int dtype, int rows, int ff, float limit, float alpha, hipStream_t stream);
 int celeg_add_bias(void* x, int dtype, const float* bias, int rows, int width, hipStream_t stream);
 int celeg_cast(const void* src, int src_dtype, void* dst, int dst_dtype, size_t total, hipStream_t stream);
 int celeg_table_update(int* table, int stride, int n_slots, const int* updates, int capacity, hipStream_t stream);
@@ -62,20 +62,21 @@ int celeg_latent_attention_fast(int form, const void* q, int ldq, const void* po
                                 hipStream_t stream);
 // moe.hip
 int celeg_moe_route(const float* logits, int rows, int experts, int top, int score, int renorm, int groups, int keep,
-                    float renorm_eps, float scale, int* ids, float* weights, hipStream_t stream);
+                    float renorm_eps, float scale, const float* correction, int group_best, float* gate_out, int* ids, float* weights,
+                    hipStream_t stream);
 int celeg_moe_router(const void* x, int x_dtype, const float* w, int rows, int width, int experts, int top, int score,
-                     int renorm, int groups, int keep, float renorm_eps, float scale, int* ids, float* weights,
-                     hipStream_t stream);
+                     int renorm, int groups, int keep, float renorm_eps, float scale, const float* correction, int group_best,
+                     float* gate_out, int* ids, float* weights, hipStream_t stream);
 int celeg_moe_tile_rows(int matrix_cores);
 int celeg_moe_plan(const int* ids, int n, int experts, int tile_rows, int* offsets, int* place_of, int* entry_at, int* tile_expert,
                    int* tile_row0, int* n_tiles, hipStream_t stream);
-int celeg_moe_gather(const void* x, int dtype, const int* entry_at, const float* weights, void* a, int n, int top, int width,
-                     hipStream_t stream);
-int celeg_moe_product(const void* a, const void* w, void* out, int dtype, int N, int K, int gated, int act, const int* offsets,
-                      const int* tile_expert, const int* tile_row0, const int* n_tiles, int max_tiles, int tile_rows, int wide,
+int celeg_moe_gather(const void* x, int dtype, const int* entry_at, const int* n_places, const float* weights, void* a, int n, int top,
+                     int width, hipStream_t stream);
+int celeg_moe_product(const void* a, const void* w, void* out, int dtype, int N, int K, int gated, int act, float limit, float alpha,
+                      const int* offsets, const int* tile_expert, const int* tile_row0, const int* n_tiles, int max_tiles, int tile_rows, int wide,
                       hipStream_t stream);
-int celeg_moe_combine(const void* y, int dtype, const int* place_of, const float* weights, const void* base, void* out, int rows,
-                      int top, int width, hipStream_t stream);
+int celeg_moe_combine(const void* y, int dtype, const int* place_of, const float* weights, const void* base,
+                      const float* base_weight, const void* x, void* out, int rows, int top, int width, hipStream_t stream);
 // gemm_f32.hip
 int celeg_gemm_f32(const float* X, int ldx, const float* W, int ldw, const float* bias, float* Y, int ldy, int M,
                    int N, int K, hipStream_t stream);
@@ -194,7 +195,7 @@ int celeg_conv_rope_store(const void* proj, int ld, int dtype, const float* conv
                           const int* positions, const int* token_seq, const int* seq_start, const int* token_slot,
                           const float* inv_freq, int rotary_dim, int pairing, void* q_out, int ldq, void* k_pool, void* v_pool,
                           const int* table, int table_stride, int n_tokens, int H, int G, int D, int V, int taps, int page_tokens,
-                          int n_layers, int layer, hipStream_t stream);
+                          int n_layers, int layer, const float* bias, float amplitude, void* kept, const float* mix, hipStream_t stream);
 // biased_attention.hip
 int celeg_kv_store(const void* k, int ldk, const void* v, int ldv, int dtype, void* k_pool, void* v_pool, const int* table,
                    int table_stride, const int* token_slot, const int* positions, int n_tokens, int kv_heads, int head_dim, int v_dim,
@@ -218,6 +219,16 @@ int celeg_matrix_memory(const void* proj, int ld, int dtype, int col_q, int col_
                         float* m, size_t ldm, const int* cu_seqlens, const int* seq_slot, const int* token_slot, float* planes,
                         float* chunk_s, float* chunk_n, void* out, int ldo, int n_rows, int n_seqs, int n_single, int max_chunks,
                         int H, int D, int V, float cap, float eps, hipStream_t stream);
+// decay_scan.hip
+int celeg_decay_scan(const void* q, int ldq, const void* k, int ldk, const void* v, int ldv, int dtype, const void* dt, int ld_dt,
+                     const float* a_log, const float* dt_bias, const float* log_decay, const float* skip, int silu, float* S, size_t ldS,
+                     const int* cu_seqlens, const int* seq_slot, const int* token_slot, float* chunk_s, float* chunk_decay, float* out,
+                     int ldo, int n_rows, int n_seqs, int n_single, int max_chunks, int H, int G, int D, int V, hipStream_t stream);
+int celeg_conv_act(const void* u, int ldu, int dtype, const float* w, const float* bias, float* state, size_t state_stride,
+                   const int* token_seq, const int* cu_seqlens, const int* seq_slot, void* out, int ldo, int n_rows, int channels,
+                   int taps, hipStream_t stream);
+int celeg_gated_norm(const float* o, int ldo, const void* gate, int ldg, int dtype, const float* weight, void* out, int ld, int rows,
+                     int parts, int size, float eps, int mode, hipStream_t stream);
 // linear_scan.hip
 int celeg_lru_gates(const void* x, int ldx, int dtype, const float* conv_w, const float* conv_b, const float* ra_t, const float* ra_b,
                     const float* ri_t, const float* ri_b, const float* lam, const float* conv_state, size_t state_stride,

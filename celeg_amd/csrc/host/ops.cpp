@@ -66,6 +66,9 @@ const char* path_name(Path p) {
         case Path::MatrixMemoryRows: return "matrix_memory_rows";
         case Path::MatrixMemoryStep: return "matrix_memory_step";
         case Path::LinearRecurrentUnit: return "linear_recurrent_unit";
+        case Path::DecayScan: return "decay_scan";
+        case Path::DecayScanRows: return "decay_scan_rows";
+        case Path::DecayScanStep: return "decay_scan_step";
         case Path::RoutedExperts: return "routed_experts";
         case Path::LinearF32: return "linear_f32";
         case Path::LinearLibrary: return "linear_library";
@@ -325,13 +328,26 @@ void Ops::latent_attention(const Tensor& q_lat, const Tensor& out, const LatentS
 }
 
 // ---------------------------------------------------------------------------- routed experts
-static Ops::RoutePlan new_route_plan(long long rows, long long experts, int top, bool matrix_cores, Workspace& ws) {
-    need(experts > 0 && experts <= 512, "moe_route: between 1 and 512 experts");
-    need(top > 0 && top <= experts, "moe_route: `top` must be between 1 and the number of experts");
+static Ops::RoutePlan new_route_plan(long long rows, long long outputs, const Ops::RouteRule& rule, bool matrix_cores, Workspace& ws,
+                                     const char* who) {
+    const std::string w = std::string(who) + ": ";
+    const long long total = outputs - (rule.row_gate ? 1 : 0), experts = total - rule.identity;
+    const int top = rule.top;
+    need(rule.identity >= 0 && experts > 0 && total <= 512, w + "between 1 and 512 experts, at least one of them with weights");
+    need(top > 0 && top <= total, w + "`top` must be between 1 and the number of experts");
+    need(rule.score == 0 || rule.score == 1, w + "score is sigmoid (0) or softmax (1)");
+    need(rule.groups >= 1 && rule.groups <= 64 && total % rule.groups == 0 && rule.keep >= 1 && rule.keep <= rule.groups,
+         w + "up to 64 groups that divide the experts evenly, of which 1 to all are kept");
+    need(top <= rule.keep * (total / rule.groups), w + "the kept groups hold fewer experts than a row uses");
+    if (rule.correction) {
+        dev(*rule.correction, "correction", DType::F32);
+        need(rule.correction->numel() == total, w + "one correction per expert");
+    }
     Ops::RoutePlan p;
     p.n = static_cast<int>(rows * top);
     p.top = top;
     p.experts = static_cast<int>(experts);
+    p.identity = rule.identity;
     const int tile = p.tile_rows = celeg_moe_tile_rows(matrix_cores ? 1 : 0);
     p.max_tiles = static_cast<int>(std::min<long long>(p.n, p.n / tile + experts));
     const long long n = std::max(p.n, 1), tiles = std::max(p.max_tiles, 1);
@@ -343,6 +359,7 @@ static Ops::RoutePlan new_route_plan(long long rows, long long experts, int top,
     p.tile_expert = ws.buf("moe_tile_expert", DType::I32, {tiles});
     p.tile_row0 = ws.buf("moe_tile_row0", DType::I32, {tiles});
     p.n_tiles = ws.buf("moe_n_tiles", DType::I32, {4});
+    if (rule.row_gate) p.row_gate = ws.buf("moe_row_gate", DType::F32, {std::max<long long>(rows, 1)});
     return p;
 }
 
@@ -351,21 +368,15 @@ static void plan_of(const Ops::RoutePlan& p, hipStream_t stream) {
                                 p.tile_expert.as<int>(), p.tile_row0.as<int>(), p.n_tiles.as<int>(), stream), "moe_plan");
 }
 
-static void check_route_rule(const Ops::RouteRule& r, long long experts, const char* who) {
-    need(r.score == 0 || r.score == 1, std::string(who) + ": score is sigmoid (0) or softmax (1)");
-    need(r.groups >= 1 && r.groups <= 64 && experts % r.groups == 0 && r.keep >= 1 && r.keep <= r.groups,
-         std::string(who) + ": up to 64 groups that divide the experts evenly, of which 1 to all are kept");
-    need(r.top <= r.keep * (experts / r.groups), std::string(who) + ": the kept groups hold fewer experts than a row uses");
-}
-
 Ops::RoutePlan Ops::moe_route(const Tensor& logits, const RouteRule& rule, bool matrix_cores, Workspace& ws) {
     dev(logits, "logits", DType::F32);
-    need(logits.ndim == 2, "moe_route: logits must be [rows, experts]");
-    RoutePlan p = new_route_plan(logits.shape[0], logits.shape[1], rule.top, matrix_cores, ws);
-    check_route_rule(rule, p.experts, "moe_route");
+    need(logits.ndim == 2 && logits.contiguous(), "moe_route: logits must be [rows, experts]");
+    RoutePlan p = new_route_plan(logits.shape[0], logits.shape[1], rule, matrix_cores, ws, "moe_route");
     took(Path::RoutedExperts);
-    kernel_check(celeg_moe_route(logits.as<float>(), static_cast<int>(logits.shape[0]), p.experts, rule.top, rule.score, rule.renorm ? 1 : 0,
-                                 rule.groups, rule.keep, rule.renorm_eps, rule.scale, p.ids.as<int>(), p.weights.as<float>(), stream),
+    kernel_check(celeg_moe_route(logits.as<float>(), static_cast<int>(logits.shape[0]), p.experts + p.identity, rule.top, rule.score,
+                                 rule.renorm ? 1 : 0, rule.groups, rule.keep, rule.renorm_eps, rule.scale,
+                                 rule.correction ? rule.correction->as<float>() : nullptr, rule.group_best ? 1 : 0,
+                                 rule.row_gate ? p.row_gate.as<float>() : nullptr, p.ids.as<int>(), p.weights.as<float>(), stream),
                  "moe_route");
     plan_of(p, stream);
     return p;
@@ -375,18 +386,19 @@ Ops::RoutePlan Ops::moe_route_rows(const Tensor& x, const Tensor& router, const 
     dev(x, "x");
     dev(router, "router", DType::F32);
     need(x.ndim == 2 && x.contiguous() && router.ndim == 2 && router.shape[1] == x.shape[1], "moe_route_rows: x [rows, width], router [experts, width]");
-    const long long rows = x.shape[0], width = x.shape[1], experts = router.shape[0];
-    if (!use_router_kernel || 4 * (width + experts) * 4 > 64 * 1024) {
-        Tensor logits = ws.buf("moe_logits", DType::F32, {rows, experts});
+    const long long rows = x.shape[0], width = x.shape[1], outputs = router.shape[0];
+    if (!use_router_kernel || 4 * (width + outputs + 1) * 4 > 64 * 1024) {
+        Tensor logits = ws.buf("moe_logits", DType::F32, {rows, outputs});
         linear(x, router, logits, nullptr, ws);
         return moe_route(logits, rule, matrix_cores, ws);
     }
-    RoutePlan p = new_route_plan(rows, experts, rule.top, matrix_cores, ws);
-    check_route_rule(rule, experts, "moe_route_rows");
+    RoutePlan p = new_route_plan(rows, outputs, rule, matrix_cores, ws, "moe_route_rows");
     took(Path::RoutedExperts);
-    kernel_check(celeg_moe_router(x.data, dt(x, "x"), router.as<float>(), static_cast<int>(rows), static_cast<int>(width), p.experts,
-                                  rule.top, rule.score, rule.renorm ? 1 : 0, rule.groups, rule.keep, rule.renorm_eps, rule.scale,
-                                  p.ids.as<int>(), p.weights.as<float>(), stream), "moe_router");
+    kernel_check(celeg_moe_router(x.data, dt(x, "x"), router.as<float>(), static_cast<int>(rows), static_cast<int>(width),
+                                  p.experts + p.identity, rule.top, rule.score, rule.renorm ? 1 : 0, rule.groups, rule.keep,
+                                  rule.renorm_eps, rule.scale, rule.correction ? rule.correction->as<float>() : nullptr,
+                                  rule.group_best ? 1 : 0, rule.row_gate ? p.row_gate.as<float>() : nullptr, p.ids.as<int>(),
+                                  p.weights.as<float>(), stream), "moe_router");
     plan_of(p, stream);
     return p;
 }
@@ -396,12 +408,14 @@ void Ops::moe_gather(const Tensor& x, const RoutePlan& p, bool weighted, const T
     dev(a, "a", x.dtype);
     need(x.ndim == 2 && x.contiguous() && a.ndim == 2 && a.shape[0] == p.n && a.shape[1] == x.shape[1] &&
              x.shape[0] * p.top == p.n, "moe_gather: a must be [rows * top, width]");
-    kernel_check(celeg_moe_gather(x.data, dt(x, "x"), p.entry_at.as<int>(), weighted ? p.weights.as<float>() : nullptr, a.data,
-                                  p.n, p.top, static_cast<int>(x.shape[1]), stream), "moe_gather");
+    kernel_check(celeg_moe_gather(x.data, dt(x, "x"), p.entry_at.as<int>(), p.offsets.as<int>() + p.experts,
+                                  weighted ? p.weights.as<float>() : nullptr, a.data, p.n, p.top, static_cast<int>(x.shape[1]), stream),
+                 "moe_gather");
 }
 
-void Ops::moe_product(const Tensor& a, const Tensor& w, const Tensor& out, bool gated, const RoutePlan& p, int act) {
-    need(act == 0 || (act == 1 && !gated), "moe_product: act is 0, or 1 (square of relu) where the product is not gated");
+void Ops::moe_product(const Tensor& a, const Tensor& w, const Tensor& out, bool gated, const RoutePlan& p, int act, float limit, float alpha) {
+    need(act == 0 || (act == 1 && !gated) || (act == 2 && gated && limit > 0.f),
+         "moe_product: act is 0, 1 (square of relu) where the product is not gated, or 2 (clamped, with a positive limit) where it is");
     dev(a, "a");
     dev(w, "w", a.dtype);
     dev(out, "out", a.dtype);
@@ -412,24 +426,27 @@ void Ops::moe_product(const Tensor& a, const Tensor& w, const Tensor& out, bool 
     need(p.tile_rows == celeg_moe_tile_rows(0) || moe_matrix_cores_ok(a.dtype, out.shape[1], a.shape[1]),
          "moe_product: the plan was made for the matrix cores, which do not take this product");
     kernel_check(celeg_moe_product(a.data, w.data, out.data, dt(a, "a"), static_cast<int>(out.shape[1]),
-                                   static_cast<int>(a.shape[1]), gated ? 1 : 0, act, p.offsets.as<int>(), p.tile_expert.as<int>(),
-                                   p.tile_row0.as<int>(), p.n_tiles.as<int>(), p.max_tiles, p.tile_rows,
+                                   static_cast<int>(a.shape[1]), gated ? 1 : 0, act, limit, alpha, p.offsets.as<int>(),
+                                   p.tile_expert.as<int>(), p.tile_row0.as<int>(), p.n_tiles.as<int>(), p.max_tiles, p.tile_rows,
                                    p.n >= 8 * p.experts ? 1 : 0, stream), "moe_product");
 }
 
-void Ops::moe_combine(const Tensor& y, const RoutePlan& p, bool weighted, const Tensor& out, const Tensor* base) {
+void Ops::moe_combine(const Tensor& y, const RoutePlan& p, bool weighted, const Tensor& out, const Tensor* base, const Tensor* x) {
     dev(y, "y");
     dev(out, "out", y.dtype);
     need(y.ndim == 2 && out.ndim == 2 && y.shape[0] == p.n && out.shape[0] * p.top == p.n && y.shape[1] == out.shape[1],
          "moe_combine: y [rows * top, width], out [rows, width]");
-    if (base) {
-        dev(*base, "base", y.dtype);
-        need(base->ndim == 2 && base->shape[0] == out.shape[0] && base->shape[1] == out.shape[1] && base->contiguous(),
-             "moe_combine: base must have the shape of out");
-    }
+    for (const Tensor* r : {base, x})
+        if (r) {
+            dev(*r, "base or x", y.dtype);
+            need(r->ndim == 2 && r->shape[0] == out.shape[0] && r->shape[1] == out.shape[1] && r->contiguous(),
+                 "moe_combine: base and x must have the shape of out");
+        }
+    need(p.identity == 0 || x, "moe_combine: identity experts need the rows themselves");
     kernel_check(celeg_moe_combine(y.data, dt(y, "y"), p.place_of.as<int>(), weighted ? p.weights.as<float>() : nullptr,
-                                   base ? base->data : nullptr, out.data,
-                                   static_cast<int>(out.shape[0]), p.top, static_cast<int>(y.shape[1]), stream), "moe_combine");
+                                   base ? base->data : nullptr, p.row_gate.defined() ? p.row_gate.as<float>() : nullptr,
+                                   x ? x->data : nullptr, out.data, static_cast<int>(out.shape[0]), p.top, static_cast<int>(y.shape[1]),
+                                   stream), "moe_combine");
 }
 
 void Ops::rmsnorm(const Tensor& x, const Tensor& weight, float eps, const Tensor& out, const Tensor* delta, const int* rows) {
@@ -509,13 +526,13 @@ void Ops::concat_rows(const Tensor& a, const Tensor& b, const Tensor& out) {
                                    static_cast<int>(a.shape[1]), stream), "concat_rows");
 }
 
-void Ops::swiglu(const Tensor& gate_up, const Tensor& out) {
+void Ops::swiglu(const Tensor& gate_up, const Tensor& out, float limit, float alpha) {
     dev(gate_up, "gate_up");
     dev(out, "out", gate_up.dtype);
     need(out.ndim == 2 && gate_up.ndim == 2 && gate_up.shape[0] == out.shape[0] && gate_up.shape[1] == 2 * out.shape[1] &&
              gate_up.contiguous() && out.contiguous(), "swiglu: gate_up must be [rows, 2*ff]");
     kernel_check(celeg_swiglu(gate_up.data, out.data, dt(out, "out"), static_cast<int>(out.shape[0]),
-                              static_cast<int>(out.shape[1]), stream), "swiglu");
+                              static_cast<int>(out.shape[1]), limit, alpha, stream), "swiglu");
 }
 
 void Ops::add_bias(const Tensor& x, const Tensor& bias) {
@@ -1042,6 +1059,88 @@ void Ops::matrix_memory(const Tensor& proj, const MemoryColumns& at, const Memor
                  "matrix_memory");
 }
 
+// ---------------------------------------------------------------------------- linear attention with a decay per head
+void Ops::decay_scan(const Tensor& q, const Tensor& k, const Tensor& v, const DecayGates& g, const DecayShape& s, const Tensor& S,
+                     const Tensor& out, const StepBatch& batch, Workspace& ws) {
+    dev(q, "q");
+    dev(k, "k", q.dtype, false);
+    dev(v, "v", q.dtype, false);
+    dev(out, "out", DType::F32, false);
+    const long long T = batch.n_tokens, H = s.heads, G = s.groups, D = s.dim, V = s.vdim;
+    need(H > 0 && G > 0 && H % G == 0 && D > 0 && V > 0 && D <= 256 && V <= 4096,
+         "decay_scan: heads a positive multiple of groups, dim up to 256, vdim up to 4,096");
+    need(q.ndim == 2 && k.ndim == 2 && v.ndim == 2 && out.ndim == 2 && q.shape[0] == T && k.shape[0] == T && v.shape[0] == T &&
+             out.shape[0] == T && q.shape[1] == G * D && k.shape[1] == G * D && v.shape[1] == H * V && out.shape[1] == H * V,
+         "decay_scan: q and k [rows, groups * dim], v and out [rows, heads * vdim]");
+    need((g.dt != nullptr) != (g.log_decay != nullptr), "decay_scan: decays come from dt or are fixed");
+    auto per_head = [&](const Tensor* t, const char* name, long long n) {
+        if (!t) return;
+        dev(*t, name, DType::F32);
+        need(t->numel() == n, std::string("decay_scan: ") + name + " has one entry per head");
+    };
+    if (g.dt) {
+        dev(*g.dt, "dt", q.dtype, false);
+        need(g.dt->ndim == 2 && g.dt->shape[0] == T && g.dt->shape[1] == H && g.a_log && g.dt_bias, "decay_scan: dt [rows, heads], with a_log and dt_bias");
+    }
+    per_head(g.a_log, "a_log", H);
+    per_head(g.dt_bias, "dt_bias", H);
+    per_head(g.log_decay, "log_decay", 2 * H);
+    per_head(g.skip, "skip", H);
+    dev(S, "S", DType::F32, false);
+    need(S.ndim >= 2 && S.numel() / S.shape[0] == H * D * V && S.stride[S.ndim - 1] == 1, "decay_scan: the states do not fit");
+    const int n_single = std::min(batch.single_rows, batch.n_seqs), portions = batch.n_seqs - n_single;
+    float *chunk_s = nullptr, *chunk_decay = nullptr;
+    int max_chunks = 0;
+    took(Path::DecayScan);
+    if (n_single > 0) took(Path::DecayScanStep);
+    if (portions > 0) {
+        took(Path::DecayScanRows);
+        max_chunks = static_cast<int>(T - n_single) / 64 + portions;
+        chunk_s = static_cast<float*>(ws.raw("decay_chunks", static_cast<size_t>(max_chunks) * H * D * V * sizeof(float)));
+        chunk_decay = static_cast<float*>(ws.raw("decay_chunk_decays", static_cast<size_t>(max_chunks) * H * sizeof(float)));
+    }
+    kernel_check(celeg_decay_scan(q.data, rows_of(q, "q"), k.data, rows_of(k, "k"), v.data, rows_of(v, "v"), dt(q, "q"),
+                                  g.dt ? g.dt->data : nullptr, g.dt ? rows_of(*g.dt, "dt") : 0, g.a_log ? g.a_log->as<float>() : nullptr,
+                                  g.dt_bias ? g.dt_bias->as<float>() : nullptr, g.log_decay ? g.log_decay->as<float>() : nullptr,
+                                  g.skip ? g.skip->as<float>() : nullptr, s.silu ? 1 : 0, S.as<float>(), static_cast<size_t>(S.stride[0]),
+                                  batch.cu_seqlens, batch.seq_slot, batch.token_slot, chunk_s, chunk_decay, out.as<float>(),
+                                  rows_of(out, "out"), static_cast<int>(T), batch.n_seqs, n_single, max_chunks, s.heads, s.groups, s.dim,
+                                  s.vdim, stream), "decay_scan");
+}
+
+void Ops::conv_act(const Tensor& x, const Tensor& w, const Tensor* bias, const Tensor& saved, const Tensor& out, const StepBatch& batch) {
+    dev(x, "x");
+    dev(w, "w", DType::F32);
+    dev(saved, "saved", DType::F32, false);
+    dev(out, "out", x.dtype, false);
+    need(x.ndim == 2 && w.ndim == 2 && out.ndim == 2 && x.shape[0] == batch.n_tokens && out.shape[0] == x.shape[0] &&
+             out.shape[1] == x.shape[1] && w.shape[1] == x.shape[1] && w.shape[0] >= 1 && w.contiguous(),
+         "conv_act: x and out [rows, channels], w [taps, channels]");
+    const long long channels = x.shape[1], taps = w.shape[0];
+    if (bias) {
+        dev(*bias, "bias", DType::F32);
+        need(bias->numel() == channels, "conv_act: one bias per channel");
+    }
+    need(saved.ndim == 3 && saved.shape[1] == std::max<long long>(taps - 1, 1) && saved.shape[2] == channels && saved.stride[2] == 1 &&
+             saved.stride[1] == channels, "conv_act: the saved inputs must be [slots, taps - 1, channels]");
+    kernel_check(celeg_conv_act(x.data, rows_of(x, "x"), dt(x, "x"), w.as<float>(), bias ? bias->as<float>() : nullptr, saved.as<float>(),
+                                static_cast<size_t>(saved.stride[0]), batch.token_seq, batch.cu_seqlens, batch.seq_slot, out.data,
+                                rows_of(out, "out"), batch.n_tokens, static_cast<int>(channels), static_cast<int>(taps), stream), "conv_act");
+}
+
+void Ops::gated_norm(const Tensor& o, const Tensor& gate, const Tensor& weight, int parts, float eps, bool gate_first, const Tensor& out) {
+    dev(o, "o", DType::F32, false);
+    dev(gate, "gate");
+    dev(weight, "weight", DType::F32);
+    dev(out, "out", gate.dtype, false);
+    need(o.ndim == 2 && gate.ndim == 2 && out.ndim == 2 && gate.shape[0] == o.shape[0] && gate.shape[1] == o.shape[1] &&
+             out.shape[0] == o.shape[0] && out.shape[1] == o.shape[1] && weight.numel() == o.shape[1], "gated_norm: o, gate and out of one shape, a weight per column");
+    need(parts > 0 && parts <= 65535 && o.shape[1] % parts == 0 && eps > 0.f, "gated_norm: parts must divide the row, eps positive");
+    kernel_check(celeg_gated_norm(o.as<float>(), rows_of(o, "o"), gate.data, rows_of(gate, "gate"), dt(gate, "gate"), weight.as<float>(),
+                                  out.data, rows_of(out, "out"), static_cast<int>(o.shape[0]), parts, static_cast<int>(o.shape[1] / parts),
+                                  eps, gate_first ? 1 : 0, stream), "gated_norm");
+}
+
 // ---------------------------------------------------------------------------- linear recurrent unit
 void Ops::lru_gates(const Tensor& x, const Tensor& conv_w, const Tensor* conv_b, const Tensor& ra_t, const Tensor& ra_b,
                     const Tensor& ri_t, const Tensor& ri_b, const Tensor& lam, const Tensor& conv_state, const Tensor& decay,
@@ -1179,7 +1278,8 @@ void Ops::biased_attention(const Tensor& q, const Tensor& out, const ScoreShape&
 }
 
 void Ops::conv_rope_store(const Tensor& proj, const Tensor* conv_w, const Tensor* conv_state, int taps, const Tensor* inv_freq,
-                          int rotary_dim, int pairing, const Tensor& q_out, int heads, const StepBatch& batch, const KVView& kv) {
+                          int rotary_dim, int pairing, const Tensor& q_out, int heads, const StepBatch& batch, const KVView& kv,
+                          const StoreExtras& extras) {
     dev(proj, "proj");
     dev(q_out, "q_out", proj.dtype, false);
     check_kv_wide(kv, kv.kv_heads, kv.head_dim, kv.v_head_dim, proj.dtype, "conv_rope_store");
@@ -1205,13 +1305,30 @@ void Ops::conv_rope_store(const Tensor& proj, const Tensor* conv_w, const Tensor
         need(rotary_dim > 0 && rotary_dim % 2 == 0 && rotary_dim <= D && inv_freq->numel() == rotary_dim / 2 && (pairing == 0 || pairing == 1),
              "conv_rope_store: an even number of turned values, at most a head's, with a frequency a pair");
     }
+    if (extras.bias) {
+        dev(*extras.bias, "bias", DType::F32);
+        need(!conv_w && extras.bias->numel() >= channels, "conv_rope_store: one bias per projected column, and no convolution");
+    }
+    need(!extras.mix || extras.kept, "conv_rope_store: mixing needs the kept values");
+    if (extras.mix) {
+        dev(*extras.mix, "mix", DType::F32);
+        need(extras.mix->numel() == 1, "conv_rope_store: mix is one number");
+    }
+    if (extras.kept) {
+        dev(*extras.kept, "kept", proj.dtype);
+        need(extras.kept->ndim == 2 && extras.kept->contiguous() && extras.kept->shape[0] == T && extras.kept->shape[1] == G * V,
+             "conv_rope_store: kept values are [rows, kv_heads * v_dim]");
+    }
     const size_t state_stride = conv_state ? static_cast<size_t>(conv_state->stride[0]) : 0;
     kernel_check(celeg_conv_rope_store(proj.data, rows_of(proj, "proj"), dt(proj, "proj"), conv_w ? conv_w->as<float>() : nullptr,
                                        conv_state ? conv_state->as<float>() : nullptr, state_stride, batch.positions, batch.token_seq,
                                        batch.seq_start, batch.token_slot, inv_freq ? inv_freq->as<float>() : nullptr,
                                        inv_freq ? rotary_dim : 0, pairing, q_out.data, rows_of(q_out, "q_out"), kv.k, kv.v, kv.table,
                                        kv.table_stride, static_cast<int>(T), heads, static_cast<int>(G), static_cast<int>(D),
-                                       static_cast<int>(V), taps, kv.page_tokens, kv.n_layers, kv.layer, stream), "conv_rope_store");
+                                       static_cast<int>(V), taps, kv.page_tokens, kv.n_layers, kv.layer,
+                                       extras.bias ? extras.bias->as<float>() : nullptr, extras.amplitude,
+                                       extras.kept ? extras.kept->data : nullptr, extras.mix ? extras.mix->as<float>() : nullptr, stream),
+                 "conv_rope_store");
     // (after every row has read the old saved inputs)
     if (conv_w && taps > 1)
         kernel_check(celeg_delta_conv_state(proj.data, rows_of(proj, "proj"), dt(proj, "proj"), conv_state->as<float>(), state_stride,

@@ -102,7 +102,7 @@ struct StepPrologue {
 // graph records; a replay counts nothing): what tests and tools ask to see that a size took the
 // path it was meant to take.
 enum class Path : int {
-    AttentionDecode = 0, AttentionDecodeFresh, AttentionRows, AttentionGeneral, AttentionSigmoid, AttentionSigmoidRows, AttentionSigmoidDecode, DeltaRule, AttentionLatent, AttentionLatentRows, AttentionLatentDecode, AttentionBiased, AttentionBiasedRows, AttentionBiasedDecode, ChannelScan, MatrixMemory, MatrixMemoryRows, MatrixMemoryStep, LinearRecurrentUnit, RoutedExperts, LinearF32, LinearLibrary, LinearStandIn,
+    AttentionDecode = 0, AttentionDecodeFresh, AttentionRows, AttentionGeneral, AttentionSigmoid, AttentionSigmoidRows, AttentionSigmoidDecode, DeltaRule, AttentionLatent, AttentionLatentRows, AttentionLatentDecode, AttentionBiased, AttentionBiasedRows, AttentionBiasedDecode, ChannelScan, MatrixMemory, MatrixMemoryRows, MatrixMemoryStep, DecayScan, DecayScanRows, DecayScanStep, LinearRecurrentUnit, RoutedExperts, LinearF32, LinearLibrary, LinearStandIn,
     FusedSliced, FusedRows, FusedStaged, Tiled, TiledQkv, ArgmaxMerged, Count
 };
 const char* path_name(Path p);
@@ -180,7 +180,8 @@ public:
     void softcap(const Tensor& x, float cap);
     // out [rows, 2 * width] = (a | b), both 32-bit [rows, width]
     void concat_rows(const Tensor& a, const Tensor& b, const Tensor& out);
-    void swiglu(const Tensor& gate_up, const Tensor& out);
+    // silu(gate) * up; limit > 0: the clamped form g sigmoid(alpha g) (u + 1), g = min(gate, limit), u = clamp(up, -limit, limit)
+    void swiglu(const Tensor& gate_up, const Tensor& out, float limit = 0.f, float alpha = 1.f);
     void add_bias(const Tensor& x, const Tensor& bias);
     void cast(const Tensor& src, const Tensor& dst);
     void apply_table_updates(int* table, int stride, int rows, const int* updates, int capacity);
@@ -259,8 +260,15 @@ public:
     // conv_w [channels, taps] 32-bit continues from conv_state [slots, taps - 1, channels] 32-bit (both null: no
     // convolution), which is moved on afterwards; q and k heads turn by the rows' positions (inv_freq null: not);
     // the queries go to q_out [rows, heads * head_dim], keys and values to the rows' places in the pages.
+    struct StoreExtras {
+        const Tensor* bias = nullptr;      // one number per column of proj, 32-bit (not with a convolution)
+        float amplitude = 1.f;             // cosine and sine times this
+        const Tensor* kept = nullptr;      // [rows, kv_heads * v_dim]: the rows' values are left there,
+        const Tensor* mix = nullptr;       // or, with one number lambda, become (1 - lambda) v + lambda kept
+    };
     void conv_rope_store(const Tensor& proj, const Tensor* conv_w, const Tensor* conv_state, int taps, const Tensor* inv_freq,
-                         int rotary_dim, int pairing, const Tensor& q_out, int heads, const StepBatch& batch, const KVView& kv);
+                         int rotary_dim, int pairing, const Tensor& q_out, int heads, const StepBatch& batch, const KVView& kv,
+                         const StoreExtras& extras);
     // a step's keys [rows, kv_heads * head_dim] and values [rows, kv_heads * v_dim] to their places in the pages;
     // v_eps > 0: every head's value divided by sqrt(mean(v^2) + v_eps)
     void kv_store(const Tensor& k, const Tensor& v, const StepBatch& batch, const KVView& kv, float v_eps = 0.f);
@@ -274,6 +282,20 @@ public:
     void matrix_memory(const Tensor& proj, const MemoryColumns& at, const MemoryShape& shape, const Tensor& bias_i, const Tensor& bias_f,
                        const Tensor& norm, const Tensor& S, const Tensor& n, const Tensor& m, const Tensor& out, const StepBatch& batch,
                        Workspace& ws);
+    // Linear attention with one decay per head and token: S <- exp(f) S + w k v^T, o = S^T q (+ skip v) from and into S
+    // [slots, heads, dim, vdim].  q, k [rows, groups * dim] and v [rows, heads * vdim] (views with dense rows); either dt
+    // [rows, heads] (w = softplus(dt + dt_bias), f = -exp(a_log) w) or log_decay [heads, 2] (two numbers whose sum is f; w = 1);
+    // skip [heads] or null; silu: q, k and v pass it as they are read; out [rows, heads * vdim] 32-bit.
+    struct DecayShape { int heads = 0, groups = 0, dim = 0, vdim = 0; bool silu = false; };
+    struct DecayGates { const Tensor *dt = nullptr, *dt_bias = nullptr, *a_log = nullptr, *log_decay = nullptr, *skip = nullptr; };
+    void decay_scan(const Tensor& q, const Tensor& k, const Tensor& v, const DecayGates& gates, const DecayShape& shape, const Tensor& S,
+                    const Tensor& out, const StepBatch& batch, Workspace& ws);
+    // out = silu(bias + causal convolution of x per channel); w [taps, channels] and bias [channels] 32-bit; saved
+    // [slots, max(taps - 1, 1), channels] 32-bit holds the requests' last inputs and is moved on
+    void conv_act(const Tensor& x, const Tensor& w, const Tensor* bias, const Tensor& saved, const Tensor& out, const StepBatch& batch);
+    // RMS norm over `parts` equal parts of a row of o (32-bit), with a gate: out = norm(o) * weight * sigmoid(gate), or, with
+    // gate_first, norm(o * silu(gate)) * weight
+    void gated_norm(const Tensor& o, const Tensor& gate, const Tensor& weight, int parts, float eps, bool gate_first, const Tensor& out);
     // layer glue (32-bit arithmetic; rows of the run's dtype)
     // out = act(x + bias): act 0 gelu (tanh form), 1 square of relu, 2 none, 3 p0 z^2 + z / 2 for z > 0 and
     // p1 (exp(z) - 1 - z) + z / 2 else; x and out views with dense rows
@@ -316,17 +338,25 @@ public:
         Tensor ids, weights;                       // [rows * top]: expert and score of every (row, choice)
         Tensor offsets, place_of, entry_at;        // rows sorted by expert
         Tensor tile_expert, tile_row0, n_tiles;
-        int n = 0, top = 0, experts = 0, max_tiles = 0, tile_rows = 0;
+        Tensor row_gate;                           // [rows], where the rule asks for one
+        int n = 0, top = 0, experts = 0, max_tiles = 0, tile_rows = 0;   // (experts: without the identity ones)
+        int identity = 0;
     };
     // How a row's experts are chosen and weighted: score "sigmoid" (0) or "softmax" (1); with groups > 1 the experts
     // form that many equal runs of neighbours, a run's score is the sum of its two largest scores, and only the experts
     // of the `keep` best runs can be chosen; the `top` largest scores are the weights, with `renorm` divided by their
-    // sum plus renorm_eps, then times `scale`.
+    // sum plus renorm_eps, then times `scale`.  correction [experts] 32-bit is added to the scores for the choice of runs and
+    // experts only; group_best: a run's score is its largest one; the last `identity` of the router's outputs are experts whose
+    // result is the row itself; row_gate: the router has one output more, whose sigmoid is a number of the row (plan.row_gate).
     struct RouteRule {
         int top = 1, score = 0;
         bool renorm = false;
         float renorm_eps = 0.f, scale = 1.f;
         int groups = 1, keep = 1;
+        const Tensor* correction = nullptr;
+        bool group_best = false;
+        int identity = 0;
+        bool row_gate = false;
     };
     // logits [rows, experts] 32-bit -> the plan; matrix_cores: the plan's products all run on the matrix cores
     // (moe_matrix_cores_ok for each of them)
@@ -340,10 +370,13 @@ public:
     }
     void moe_gather(const Tensor& x, const RoutePlan& plan, bool weighted, const Tensor& a);
     // out[p] = a[p] w[expert of p]^T; w [experts * N, K], or [experts * 2N, K] if gated (silu(gate) * up)
-    // (not gated, act 1: the square of relu of the product)
-    void moe_product(const Tensor& a, const Tensor& w, const Tensor& out, bool gated, const RoutePlan& plan, int act = 0);
-    // base: rows [rows, width] added to every row's sum (what all rows get besides their experts), or null
-    void moe_combine(const Tensor& y, const RoutePlan& plan, bool weighted, const Tensor& out, const Tensor* base = nullptr);
+    // (not gated, act 1: the square of relu of the product; gated, act 2: the clamped form with limit and alpha, see swiglu)
+    void moe_product(const Tensor& a, const Tensor& w, const Tensor& out, bool gated, const RoutePlan& plan, int act = 0,
+                     float limit = 0.f, float alpha = 1.f);
+    // base: rows [rows, width] added to every row's sum (what all rows get besides their experts; times the plan's row gates
+    // where it has them), or null; x: the rows themselves, where the plan has identity experts
+    void moe_combine(const Tensor& y, const RoutePlan& plan, bool weighted, const Tensor& out, const Tensor* base = nullptr,
+                     const Tensor* x = nullptr);
     // sampling
     void sample(const Tensor& logits, const float* fparams, const int* iparams, uint8_t* seen,
                 size_t seen_stride, int* out_tokens, int* last_tokens, bool all_greedy, Workspace& ws,

@@ -257,6 +257,22 @@ public:
             if (!sc.is_object()) throw SpecError("rope: scaling must be an object");
             scaled_ = true;
             factor_ = sc.get_double("factor", 1.0);
+            const std::string kind = sc.get_string("kind", "wavelength");
+            if (kind == "yarn") {
+                yarn_ = true;
+                original_ = sc.get_double("original", 0.0);
+                const double fast = sc.get_double("fast", 0.0), slow = sc.get_double("slow", 0.0);
+                if (!(factor_ > 0) || !(original_ > 0) || !(fast > 0) || !(slow > 0) || !(theta_ > 1))
+                    throw SpecError("rope: yarn scaling needs positive factor, original, fast and slow, and theta above 1");
+                auto pair_of = [&](double turns) {
+                    return rotary_dim_ * std::log(original_ / (2.0 * 3.14159265358979323846 * turns)) / (2.0 * std::log(theta_));
+                };
+                low_ = std::max(std::floor(pair_of(fast)), 0.0);
+                high_ = std::min(std::ceil(pair_of(slow)), rotary_dim_ - 1.0);
+                amplitude_ = 0.1 * std::log(factor_) + 1.0;
+                return;
+            }
+            if (kind != "wavelength") throw SpecError("rope: scaling is 'wavelength' or 'yarn', not '" + kind + "'");
             low_ = sc.get_double("low", 1.0);
             high_ = sc.get_double("high", 1.0);
             original_ = sc.get_double("original", 0.0);
@@ -269,18 +285,25 @@ public:
         if (!table_) {
             std::vector<float> freq(static_cast<size_t>(rotary_dim_ / 2));
             for (int i = 0; i < rotary_dim_ / 2; ++i)
-                freq[static_cast<size_t>(i)] = static_cast<float>(scaled(std::pow(theta_, -2.0 * i / rotary_dim_)));
+                freq[static_cast<size_t>(i)] = static_cast<float>(scaled(std::pow(theta_, -2.0 * i / rotary_dim_), i));
             table_ = from_host_floats(freq, DType::F32, {rotary_dim_ / 2});
         }
-        return Tables{table_->view, rotary_dim_, pairing_};
+        return Tables{table_->view, rotary_dim_, pairing_, static_cast<float>(amplitude_)};
     }
 
 private:
     // "scaling" {factor, low, high, original}: frequencies whose wavelength 2 pi / f is below
     // original / high stay, above original / low become f / factor, and between the two
-    // (1 - s) f / factor + s f with s = (original / wavelength - low) / (high - low)
-    double scaled(double f) const {
+    // (1 - s) f / factor + s f with s = (original / wavelength - low) / (high - low).
+    // "kind": "yarn" {factor, original, fast, slow}: with d(t) the pair (a fraction) whose wavelength fits t times into
+    // `original`, pairs up to floor(d(fast)) keep their frequency, those from ceil(d(slow)) on have f / factor, and
+    // between the two lies a line in the pair's number; cosine and sine are multiplied by 0.1 ln(factor) + 1.
+    double scaled(double f, int i) const {
         if (!scaled_) return f;
+        if (yarn_) {
+            const double ramp = std::min(std::max((i - low_) / std::max(high_ - low_, 0.001), 0.0), 1.0);
+            return f / factor_ * ramp + f * (1.0 - ramp);
+        }
         const double wavelength = 2.0 * 3.14159265358979323846 / f;
         if (wavelength < original_ / high_) return f;
         if (wavelength > original_ / low_) return f / factor_;
@@ -288,11 +311,19 @@ private:
         return (1.0 - t) * f / factor_ + t * f;
     }
     double theta_;
-    bool scaled_ = false;
+    bool scaled_ = false, yarn_ = false;
+    double amplitude_ = 1.0;
     double factor_ = 1.0, low_ = 1.0, high_ = 1.0, original_ = 0.0;
     int head_dim_, rotary_dim_, pairing_ = 0;
     std::shared_ptr<DeviceTensor> table_;
 };
+
+// the tables of a mixer whose kernels know no amplitude
+PositionEncoding::Tables plain_tables(PositionEncoding& position, Runtime& rt, const char* who) {
+    const PositionEncoding::Tables t = position.tables(rt);
+    if (t.amplitude != 1.f) throw SpecError(std::string(who) + ": a position encoding that scales cosine and sine is not supported here");
+    return t;
+}
 
 class NoPosition final : public PositionEncoding {
 public:
@@ -405,7 +436,7 @@ private:
             if (norm) fused::norm_linear(rt, x, *norm, w->view, out, Epilogue::Store);
             else rt.ops.linear(x, w->view, out, nullptr, rt.ws);
         };
-        const PositionEncoding::Tables tables = position_->tables(rt);
+        const PositionEncoding::Tables tables = plain_tables(*position_, rt, "gqa_attention");
         const Tensor* inv_freq = tables.inv_freq.defined() ? &tables.inv_freq : nullptr;
         Tensor q, k, v;
         bool finished = false;      // norm, rotation and cache write made by the product's own kernel
@@ -597,7 +628,7 @@ private:
         Tensor proj = rt.ws.buf("latent_proj", rt.dtype, {T, w_in_->view.shape[0]});
         if (norm) fused::norm_linear(rt, x, *norm, w_in_->view, proj, Epilogue::Store);
         else rt.ops.linear(x, w_in_->view, proj, nullptr, rt.ws);
-        const PositionEncoding::Tables tables = position_->tables(rt);
+        const PositionEncoding::Tables tables = plain_tables(*position_, rt, "latent_attention");
         const Tensor* inv_freq = tables.inv_freq.defined() ? &tables.inv_freq : nullptr;
         Tensor q_lat = rt.ws.buf("latent_q", rt.dtype, {T, H * D});
         if (q_rank_ > 0) {
@@ -751,10 +782,21 @@ private:
 // (src/backend/cpu/model_forward_token.cpp:163-172; kernels/elementwise.cpp:101-119).  Gate and
 // up projections run as one matrix product on the concatenation [W1; W3] (rows [0,ff) gate,
 // [ff,2ff) up), as the reference's w13 (src/backend/cuda/model/weight_setup.cpp:289-306).
+// "activation": "clamped" with "limit" c and "alpha": gate and up become g = min(gate, c), u = clamp(up, -c, c), and
+// the product's place takes g sigmoid(alpha g) (u + 1).
+void read_clamp(const Json& p, const char* who, float& limit, float& alpha) {
+    limit = static_cast<float>(p.get_double("limit", 0.0));
+    alpha = static_cast<float>(p.get_double("alpha", 1.0));
+    if (!(limit > 0.f)) throw SpecError(std::string(who) + ": a clamped activation needs a positive limit");
+}
+
 class SwiGlu final : public FeedForward {
 public:
     explicit SwiGlu(const PartSpec& s) : FeedForward(s), width_(s.params.get_int("width", 0)), ff_(s.params.get_int("ff", 0)) {
         if (width_ <= 0 || ff_ <= 0) throw SpecError("swiglu: width and ff must be positive");
+        const std::string act = s.params.get_string("activation", "silu");
+        if (act != "silu" && act != "clamped") throw SpecError("swiglu: activation is 'silu' or 'clamped', not '" + act + "'");
+        if (act == "clamped") read_clamp(s.params, "swiglu", limit_, alpha_);
     }
     bool graph_safe() const override { return true; }
     WeightSpecs weight_specs() const override {
@@ -771,7 +813,7 @@ public:
         Tensor gate_up = rt.ws.buf("ffn_gate_up", rt.dtype, {T, 2 * ff_});
         rt.ops.linear(x, w_gate_up_->view, gate_up, nullptr, rt.ws);
         Tensor act = rt.ws.buf("ffn_act", rt.dtype, {T, ff_});
-        rt.ops.swiglu(gate_up, act);
+        rt.ops.swiglu(gate_up, act, limit_, alpha_);
         Tensor out = rt.ws.buf("ffn_out", rt.dtype, {T, width_});
         rt.ops.linear(act, w_down_->view, out, nullptr, rt.ws);
         return out;
@@ -779,7 +821,8 @@ public:
     // h += ffn(norm(h)): the norm and the SwiGLU folded into the first product, the residual
     // addition into the second
     bool forward_fused(const Tensor& h, const Norm::Foldable& norm, const StepBatch& batch, Runtime& rt) override {
-        if (!fused::fused_rows_ok(rt, batch, {width_, ff_}) || w_gate_up_->view.dtype != rt.dtype || w_down_->view.dtype != rt.dtype)
+        if (limit_ > 0.f || !fused::fused_rows_ok(rt, batch, {width_, ff_}) || w_gate_up_->view.dtype != rt.dtype ||
+            w_down_->view.dtype != rt.dtype)
             return false;
         Tensor act = fused::operand_rows(rt, "ffn_act_fused", batch.n_tokens, ff_, {width_});
         fused::norm_linear(rt, h, norm, w_gate_up_->view, act, Epilogue::Swiglu);
@@ -789,6 +832,7 @@ public:
 
 private:
     long long width_, ff_;
+    float limit_ = 0.f, alpha_ = 1.f;
     std::shared_ptr<DeviceTensor> w_gate_up_, w_down_;
 };
 
@@ -802,7 +846,12 @@ private:
 // "groups": {"count", "keep"}: the experts form `count` equal groups of neighbours, a group's score is the
 // sum of its two largest scores, and only experts of the `keep` best groups can be chosen.  "renormalize_eps"
 // is added to the sum the chosen scores are divided by; "route_scale" multiplies the weights afterwards.
-// "shared": a feed-forward part that every row passes as well; its output is added to the experts'.
+// "shared": a feed-forward part that every row passes as well; its output is added to the experts', times
+// sigmoid(W_sg x), one number a row, with "shared_gate" (tensor "shared_gate" [1, width]).
+// "correction": a number per router output (tensor "correction") added to the scores for the choice of groups and
+// experts, not to the weights.  "group_score": "two" (the default) or "best" (a group's largest score).
+// "identity" n: the router has n outputs more, the last ones, for experts whose output is the row itself.
+// "activation": "clamped" with "limit" and "alpha" as for swiglu.
 class RoutedExperts final : public FeedForward {
 public:
     explicit RoutedExperts(const PartSpec& s) : FeedForward(s) {
@@ -826,12 +875,28 @@ public:
         if (PartSpec::is_part(p["shared"])) shared_ = build_as<FeedForward>("ffn", PartSpec::from_json(p["shared"], "routed_experts.shared"));
         gated_ = p.get_bool("gated", true);
         const std::string act = p.get_string("activation", gated_ ? "silu" : "relu2");
-        if (act != (gated_ ? "silu" : "relu2"))
-            throw SpecError("routed_experts: activation is 'silu' for gated experts and 'relu2' for experts without a gate, not '" + act + "'");
-        if (width_ <= 0 || ff_ <= 0 || experts_ <= 0 || top_ <= 0 || top_ > experts_)
+        if (act == "clamped" && gated_) {
+            act_ = 2;
+            read_clamp(p, "routed_experts", limit_, alpha_);
+        } else if (act != (gated_ ? "silu" : "relu2")) {
+            throw SpecError("routed_experts: activation is 'silu' or 'clamped' for gated experts and 'relu2' for experts without a gate, not '" + act + "'");
+        } else {
+            act_ = gated_ ? 0 : 1;
+        }
+        rule_.identity = static_cast<int>(p.get_int("identity", 0));
+        corrected_ = p.get_bool("correction", false);
+        const std::string group_score = p.get_string("group_score", "two");
+        if (group_score != "two" && group_score != "best") throw SpecError("routed_experts: group_score is 'two' or 'best', not '" + group_score + "'");
+        rule_.group_best = group_score == "best";
+        rule_.row_gate = p.get_bool("shared_gate", false);
+        if (rule_.row_gate && !shared_) throw SpecError("routed_experts: shared_gate goes with a shared part");
+        const int outputs = experts_ + rule_.identity;
+        if (rule_.identity < 0 || (rule_.identity > 0 && on_input_))
+            throw SpecError("routed_experts: identity is not negative, and goes with weights on the output");
+        if (width_ <= 0 || ff_ <= 0 || experts_ <= 0 || top_ <= 0 || top_ > outputs)
             throw SpecError("routed_experts: width, ff and experts must be positive and top between 1 and experts");
-        if (rule_.groups < 1 || rule_.groups > 64 || experts_ % rule_.groups || rule_.keep < 1 || rule_.keep > rule_.groups ||
-            top_ > rule_.keep * (experts_ / rule_.groups))
+        if (rule_.groups < 1 || rule_.groups > 64 || outputs % rule_.groups || rule_.keep < 1 || rule_.keep > rule_.groups ||
+            top_ > rule_.keep * (outputs / rule_.groups))
             throw SpecError("routed_experts: groups.count (up to 64) must divide experts, and the groups.keep kept groups must hold at least top experts");
         rule_.top = top_;
         rule_.score = score_;
@@ -842,7 +907,10 @@ public:
     }
     static std::string role(const char* what, int e) { return std::string(what) + "." + std::to_string(e); }
     WeightSpecs weight_specs() const override {
-        WeightSpecs specs{{"router", WeightSpec{{experts_, width_}, "vector", "normal", {}}}};
+        const long long outputs = experts_ + rule_.identity;
+        WeightSpecs specs{{"router", WeightSpec{{outputs, width_}, "vector", "normal", {}}}};
+        if (corrected_) specs.push_back({"correction", vec(outputs)});
+        if (rule_.row_gate) specs.push_back({"shared_gate", WeightSpec{{1, width_}, "vector", "normal", {}}});
         for (int e = 0; e < experts_; ++e) {
             if (gated_) specs.push_back({role("gate", e), matrix(ff_, width_)});
             specs.push_back({role("up", e), matrix(ff_, width_)});
@@ -855,6 +923,11 @@ public:
     }
     void load(const PartTensors& t, Runtime& rt) override {
         router_ = get(t, "router");
+        if (rule_.row_gate) router_ = concat_rows({router_, get(t, "shared_gate")});     // (one product for both)
+        if (corrected_) {
+            correction_ = get(t, "correction");
+            rule_.correction = &correction_->view;
+        }
         if (shared_) {
             PartTensors mine;
             for (const auto& ws : shared_->weight_specs()) mine[ws.first] = get(t, "shared." + ws.first);
@@ -883,21 +956,23 @@ public:
         Tensor a = rt.ws.buf("moe_in", rt.dtype, {T * top_, width_});
         rt.ops.moe_gather(x, plan, on_input_, a);
         Tensor act = rt.ws.buf("moe_act", rt.dtype, {T * top_, ff_});
-        rt.ops.moe_product(a, w_gate_up_->view, act, gated_, plan, gated_ ? 0 : 1);
+        rt.ops.moe_product(a, w_gate_up_->view, act, gated_, plan, act_, limit_, alpha_);
         Tensor y = rt.ws.buf("moe_y", rt.dtype, {T * top_, width_});
         rt.ops.moe_product(act, w_down_->view, y, false, plan);
         Tensor out = rt.ws.buf(shared_ ? "moe_out" : "ffn_out", rt.dtype, {T, width_});
-        rt.ops.moe_combine(y, plan, !on_input_, out, shared_ ? &base : nullptr);
+        rt.ops.moe_combine(y, plan, !on_input_, out, shared_ ? &base : nullptr, rule_.identity > 0 ? &x : nullptr);
         return out;
     }
 
 private:
     long long width_ = 0, ff_ = 0;
     int experts_ = 0, top_ = 0, score_ = 0;
-    bool on_input_ = false, gated_ = true;
+    bool on_input_ = false, gated_ = true, corrected_ = false;
+    int act_ = 0;
+    float limit_ = 0.f, alpha_ = 1.f;
     Ops::RouteRule rule_;
     std::unique_ptr<FeedForward> shared_;
-    std::shared_ptr<DeviceTensor> router_, w_gate_up_, w_down_;
+    std::shared_ptr<DeviceTensor> router_, correction_, w_gate_up_, w_down_;
 };
 
 // a layer without a feed-forward (the reference's LayerSpec may hold none,
@@ -1440,7 +1515,7 @@ public:
         Tensor q = proj.cols(0, qw), k = proj.cols(qw, kvw);
         Tensor v = values_are_keys_ ? k : proj.cols(qw + kvw, kvw);
         Tensor gate = head_gate_ ? proj.cols(gate_col_, heads_) : Tensor();
-        const PositionEncoding::Tables tables = position_->tables(rt);
+        const PositionEncoding::Tables tables = plain_tables(*position_, rt, "sigmoid_attention");
         const Tensor* inv_freq = tables.inv_freq.defined() ? &tables.inv_freq : nullptr;
         // (q is normed and turned in place; the keys go to their pages normed and turned, the values as they are)
         rt.ops.qk_norm_rope_store(q, &k, &v, q_norm_ ? &q_norm_->view : nullptr, k_norm_ ? &k_norm_->view : nullptr, eps_, inv_freq,
@@ -1731,7 +1806,11 @@ private:
 // "taps" n > 0: every channel of q, k and v passes a causal convolution over time of n taps right behind its
 // projection (tensors q_conv, k_conv, v_conv [channels, taps], no bias; y_t = sum_j w[:, j] u_(t - n + 1 + j),
 // zeros before the sequence starts); the last n - 1 projected rows are the request's state.  "position": a
-// position encoding part (rope) that turns q and k heads behind the convolution.
+// position encoding part (rope) that turns q and k heads behind the convolution.  "bias": q, k and v have biases
+// (tensors q_bias, k_bias, v_bias; not with taps).  "value_mix": "keep" leaves the rows' values for later layers of the same
+// step; "mix" makes them (1 - lambda) v + lambda kept before they are cached (lambda: tensor "mix", one number).  The kept
+// rows are a buffer of the run's workspace that mixers of one model share under the name "value_mix_rows"; which layer keeps
+// and which layers mix is the architecture's business.
 class BiasedAttention final : public Mixer {
 public:
     explicit BiasedAttention(const PartSpec& s) : Mixer(s) {
@@ -1777,7 +1856,15 @@ public:
         if (PartSpec::is_part(p["position"]))
             position_ = build_as<PositionEncoding>("position", PartSpec::from_json(p["position"], "biased_attention.position"));
         distance_bias_ = p.get_bool("distance_bias", false);
-        if (v_eps_ > 0.f && (taps_ > 0 || position_)) throw SpecError("biased_attention: value_norm does not go with taps or a position part");
+        bias_ = p.get_bool("bias", false);
+        const std::string value_mix = p.get_string("value_mix", "none");
+        if (value_mix != "none" && value_mix != "keep" && value_mix != "mix")
+            throw SpecError("biased_attention: value_mix is 'none', 'keep' or 'mix', not '" + value_mix + "'");
+        keeps_values_ = value_mix == "keep";
+        mixes_values_ = value_mix == "mix";
+        if (bias_ && taps_ > 0) throw SpecError("biased_attention: bias does not go with taps");
+        if (v_eps_ > 0.f && (taps_ > 0 || position_ || bias_ || value_mix != "none"))
+            throw SpecError("biased_attention: value_norm does not go with taps, a position part, bias or value_mix");
         const std::string gate = p.get_string("gate", "none");
         if (gate != "none" && gate != "sigmoid") throw SpecError("biased_attention: gate is 'none' or 'sigmoid', not '" + gate + "'");
         gated_ = gate == "sigmoid";
@@ -1809,6 +1896,13 @@ public:
         }
         if (sink_) specs.push_back({"sink", vec(shape_.heads)});
         if (gated_) specs.push_back({"g", matrix(o_width(), width_)});
+        if (bias_) {
+            specs.push_back({"q_bias", vec(q_width())});
+            specs.push_back({"k_bias", vec(k_width())});
+            specs.push_back({"v_bias", vec(v_width())});
+        }
+        // (a checkpoint may store the number of a layer that keeps its values too; it is bound and not used)
+        if (mixes_values_ || (keeps_values_ && spec.tensor("mix"))) specs.push_back({"mix", WeightSpec{{}, "vector", "normal", {{1}}}});
         if (taps_ > 0) {
             auto taps = [&](long long n) { return WeightSpec{{n, taps_}, "vector", "normal", {}}; };
             specs.push_back({"q_conv", taps(q_width())});
@@ -1830,6 +1924,15 @@ public:
         r1_ = maybe(t, "r1");
         r2_ = maybe(t, "r2");
         sink_w_ = maybe(t, "sink");
+        if (bias_) {
+            std::vector<float> b;
+            for (const char* role : {"q_bias", "k_bias", "v_bias"}) {
+                const std::vector<float> piece = to_host_floats(get(t, role)->view);
+                b.insert(b.end(), piece.begin(), piece.end());
+            }
+            bias_w_ = from_host_floats(b, DType::F32, {static_cast<long long>(b.size())});
+        }
+        if (mixes_values_) mix_ = from_host_floats(to_host_floats(get(t, "mix")->view), DType::F32, {1});
     }
     Tensor forward(const Tensor& x, const StepBatch& batch, const LayerCache& cache, Runtime& rt) override {
         Tensor attended = project_and_attend(x, nullptr, batch, cache, rt);
@@ -1857,15 +1960,24 @@ private:
         else rt.ops.linear(x, w_in_->view, proj, nullptr, rt.ws);
         // every row's keys and values are in their pages before any row attends
         Tensor q = proj.cols(0, q_width());
-        if (taps_ > 0 || position_) {
+        if (taps_ > 0 || position_ || bias_ || keeps_values_ || mixes_values_) {
             // convolutions continuing from the request's saved rows, rotation, queries to a buffer of their own
             PositionEncoding::Tables tables;
             if (position_) tables = position_->tables(rt);
             const Tensor* inv_freq = tables.inv_freq.defined() ? &tables.inv_freq : nullptr;
             q = rt.ws.buf("battn_q", rt.dtype, {T, q_width()});
             const Tensor* state = taps_ > 0 ? &cache.states.at("conv") : nullptr;
+            Ops::StoreExtras extras;
+            extras.amplitude = tables.amplitude;
+            if (bias_) extras.bias = &bias_w_->view;
+            Tensor kept;
+            if (keeps_values_ || mixes_values_) {
+                kept = rt.ws.buf("value_mix_rows", rt.dtype, {T, v_width()});
+                extras.kept = &kept;
+                if (mixes_values_) extras.mix = &mix_->view;
+            }
             rt.ops.conv_rope_store(proj, taps_ > 0 ? &conv_w_->view : nullptr, state, taps_, inv_freq, tables.rotary_dim, tables.pairing,
-                                   q, shape_.heads, batch, *cache.kv);
+                                   q, shape_.heads, batch, *cache.kv, extras);
         } else {
             rt.ops.kv_store(proj.cols(col_k_, k_width()), proj.cols(col_v_, v_width()), batch, *cache.kv, v_eps_);
         }
@@ -1878,11 +1990,11 @@ private:
 
     long long width_ = 0, col_k_ = 0, col_v_ = 0, col_g_ = 0;
     Ops::ScoreShape shape_;
-    bool distance_bias_ = false, gated_ = false, sink_ = false;
+    bool distance_bias_ = false, gated_ = false, sink_ = false, bias_ = false, keeps_values_ = false, mixes_values_ = false;
     float v_eps_ = 0.f;
     int taps_ = 0;
     std::unique_ptr<PositionEncoding> position_;
-    std::shared_ptr<DeviceTensor> w_in_, w_o_, r1_, r2_, conv_w_, sink_w_;
+    std::shared_ptr<DeviceTensor> w_in_, w_o_, r1_, r2_, conv_w_, sink_w_, bias_w_, mix_;
 };
 
 // ---------------------------------------------------------------------------- real-gated linear recurrent unit
@@ -2206,6 +2318,193 @@ private:
     std::shared_ptr<DeviceTensor> w_in_, b_i_, b_f_, norm_, w_o_;
 };
 
+// ---------------------------------------------------------------------------- linear attention with fixed decays
+// q = silu(W_q h), k = silu(W_k h) (heads x dim), v = silu(W_v h) (heads x vdim); per head, with a number "decay" of its own,
+//     S <- decay S + k v^T;   o = S^T q                 from S = 0, no other scale
+// The heads side by side are divided by their common sqrt(mean(o^2) + eps), times a weight, times sigmoid(W_g h), through
+// W_o.  State per request: S [heads, dim, vdim], 32-bit like everything behind the projections.
+class FixedDecayAttention final : public Mixer {
+public:
+    explicit FixedDecayAttention(const PartSpec& s) : Mixer(s) {
+        const Json& p = s.params;
+        width_ = p.get_int("width", 0);
+        shape_.heads = shape_.groups = static_cast<int>(p.get_int("heads", 0));
+        shape_.dim = static_cast<int>(p.get_int("dim", 0));
+        shape_.vdim = static_cast<int>(p.get_int("vdim", shape_.dim));
+        shape_.silu = true;
+        eps_ = static_cast<float>(p.get_double("eps", 1e-6));
+        if (width_ <= 0 || shape_.heads <= 0 || shape_.dim <= 0 || shape_.vdim <= 0)
+            throw SpecError("fixed_decay_attention: width, heads, dim and vdim must be positive");
+        if (shape_.dim > 256 || shape_.vdim > 4096) throw SpecError("fixed_decay_attention: dim may be at most 256 and vdim at most 4096");
+        if (!(eps_ > 0.f)) throw SpecError("fixed_decay_attention: eps must be positive");
+        if (!p["decay"].is_array() || static_cast<int>(p["decay"].size()) != shape_.heads)
+            throw SpecError("fixed_decay_attention: decay lists a number per head");
+        for (const Json& d : p["decay"].items()) {
+            const double x = d.as_double();
+            if (!(x > 0) || x > 1) throw SpecError("fixed_decay_attention: a decay lies above 0 and is at most 1");
+            const double log_x = std::log(x);
+            const float hi = static_cast<float>(log_x);
+            decays_.push_back(hi);                                        // (two 32-bit numbers that add up to the log)
+            decays_.push_back(static_cast<float>(log_x - hi));
+        }
+    }
+    bool graph_safe() const override { return true; }
+    long long qk_width() const { return static_cast<long long>(shape_.heads) * shape_.dim; }
+    long long v_width() const { return static_cast<long long>(shape_.heads) * shape_.vdim; }
+    std::vector<StateNeed> state_needs() const override { return {StateNeed{"S", {shape_.heads, shape_.dim, shape_.vdim}, DType::F32}}; }
+    WeightSpecs weight_specs() const override {
+        return {{"q", matrix(qk_width(), width_)}, {"k", matrix(qk_width(), width_)}, {"v", matrix(v_width(), width_)},
+                {"g", matrix(v_width(), width_)},  {"norm", vec(v_width(), "around_one")}, {"o", matrix(width_, v_width())}};
+    }
+    void load(const PartTensors& t, Runtime&) override {
+        const Stacked in = stack_projections({{get(t, "q"), false}, {get(t, "k"), false}, {get(t, "v"), false}, {get(t, "g"), false}},
+                                             "fixed_decay_attention");
+        w_in_ = in.weight;
+        col_k_ = in.at[1];
+        col_v_ = in.at[2];
+        col_g_ = in.at[3];
+        norm_ = get(t, "norm");
+        w_o_ = get(t, "o");
+        log_decay_ = from_host_floats(decays_, DType::F32, {shape_.heads, 2});
+    }
+    Tensor forward(const Tensor& x, const StepBatch& batch, const LayerCache& cache, Runtime& rt) override {
+        Tensor read = project_and_read(x, nullptr, batch, cache, rt);
+        Tensor out = rt.ws.buf("decay_mixer_out", rt.dtype, {x.shape[0], width_});
+        rt.ops.linear(read, w_o_->view, out, nullptr, rt.ws);
+        return out;
+    }
+    // h += mixer(norm(h)) with the norm folded into the one product in front and the sum into the one behind
+    bool forward_fused(const Tensor& h, const Norm::Foldable& norm, const StepBatch& batch, const LayerCache& cache,
+                       Runtime& rt) override {
+        if (!fused::fused_rows_ok(rt, batch, {width_, v_width()}) || w_in_->view.dtype != rt.dtype || w_o_->view.dtype != rt.dtype) return false;
+        Tensor read = project_and_read(h, &norm, batch, cache, rt);
+        fused::linear_into_stream(rt, read, w_o_->view, h);
+        return true;
+    }
+
+private:
+    // norm null: x are normalised rows; else x is the stream and the norm is applied inside the product
+    Tensor project_and_read(const Tensor& x, const Norm::Foldable* norm, const StepBatch& batch, const LayerCache& cache, Runtime& rt) {
+        const long long T = x.shape[0];
+        Tensor proj = rt.ws.buf("decay_proj", rt.dtype, {T, w_in_->view.shape[0]});
+        if (norm) fused::norm_linear(rt, x, *norm, w_in_->view, proj, Epilogue::Store);
+        else rt.ops.linear(x, w_in_->view, proj, nullptr, rt.ws);
+        Tensor o = rt.ws.buf("decay_o", DType::F32, {T, v_width()});
+        Ops::DecayGates gates;
+        gates.log_decay = &log_decay_->view;
+        rt.ops.decay_scan(proj.cols(0, qk_width()), proj.cols(col_k_, qk_width()), proj.cols(col_v_, v_width()), gates, shape_,
+                          cache.states.at("S"), o, batch, rt.ws);
+        Tensor read = rt.ws.buf("decay_read", rt.dtype, {T, v_width()});
+        rt.ops.gated_norm(o, proj.cols(col_g_, v_width()), norm_->view, 1, eps_, false, read);
+        return read;
+    }
+
+    long long width_ = 0, col_k_ = 0, col_v_ = 0, col_g_ = 0;
+    Ops::DecayShape shape_;
+    float eps_ = 1e-6f;
+    std::vector<float> decays_;
+    std::shared_ptr<DeviceTensor> w_in_, norm_, w_o_, log_decay_;
+};
+
+// ---------------------------------------------------------------------------- state space with decays from the input
+// Mamba-2.  With inner = heads * vdim and N = "state", W_in h = [z: inner | x: inner | B: groups * N | C: groups * N | dt: heads].
+// x, B and C pass a causal convolution per channel ("taps", with bias) and silu; w = softplus(dt + dt_bias); per head (heads of
+// a group share its B and C)
+//     S <- exp(-exp(A_log) w) S + w B x^T;   y = S^T C + D x             S [N, vdim] from 0
+// y times silu(z), RMS-normed in "norm_groups" equal parts, times a weight, through W_o.  State per request: S and the
+// convolution's last taps - 1 inputs, 32-bit like everything behind the convolutions.
+class StateSpace final : public Mixer {
+public:
+    explicit StateSpace(const PartSpec& s) : Mixer(s) {
+        const Json& p = s.params;
+        width_ = p.get_int("width", 0);
+        shape_.heads = static_cast<int>(p.get_int("heads", 0));
+        shape_.groups = static_cast<int>(p.get_int("groups", 1));
+        shape_.dim = static_cast<int>(p.get_int("state", 0));
+        shape_.vdim = static_cast<int>(p.get_int("vdim", 0));
+        taps_ = p.get_int("taps", 1);
+        norm_groups_ = static_cast<int>(p.get_int("norm_groups", 1));
+        eps_ = static_cast<float>(p.get_double("eps", 1e-6));
+        if (width_ <= 0 || shape_.heads <= 0 || shape_.groups <= 0 || shape_.heads % shape_.groups || shape_.dim <= 0 || shape_.vdim <= 0)
+            throw SpecError("state_space: width, state and vdim must be positive and heads a positive multiple of groups");
+        if (shape_.dim > 256 || shape_.vdim > 4096) throw SpecError("state_space: state may be at most 256 and vdim at most 4096");
+        if (taps_ <= 0 || norm_groups_ <= 0 || inner() % norm_groups_ || !(eps_ > 0.f))
+            throw SpecError("state_space: taps and eps must be positive, and norm_groups must divide heads * vdim");
+    }
+    bool graph_safe() const override { return true; }
+    long long inner() const { return static_cast<long long>(shape_.heads) * shape_.vdim; }
+    long long bc_width() const { return static_cast<long long>(shape_.groups) * shape_.dim; }
+    long long channels() const { return inner() + 2 * bc_width(); }
+    std::vector<StateNeed> state_needs() const override {
+        return {StateNeed{"S", {shape_.heads, shape_.dim, shape_.vdim}, DType::F32},
+                StateNeed{"conv", {std::max<long long>(taps_ - 1, 1), channels()}, DType::F32}};
+    }
+    WeightSpecs weight_specs() const override {
+        return {{"in", matrix(inner() + channels() + shape_.heads, width_)},
+                {"conv", WeightSpec{{channels(), taps_}, "vector", "normal", {}}}, {"conv_bias", vec(channels())},
+                {"dt_bias", vec(shape_.heads)}, {"A_log", vec(shape_.heads)}, {"D", vec(shape_.heads)},
+                {"norm", vec(inner(), "around_one")}, {"o", matrix(width_, inner())}};
+    }
+    void load(const PartTensors& t, Runtime&) override {
+        w_in_ = stack_projections({{get(t, "in"), false}}, "state_space").weight;
+        const std::vector<float> w = to_host_floats(get(t, "conv")->view);
+        std::vector<float> by_tap(w.size());
+        const size_t C = static_cast<size_t>(channels()), taps = static_cast<size_t>(taps_);
+        for (size_t c = 0; c < C; ++c)
+            for (size_t j = 0; j < taps; ++j) by_tap[j * C + c] = w[c * taps + j];
+        conv_w_ = from_host_floats(by_tap, DType::F32, {taps_, channels()});
+        conv_b_ = get(t, "conv_bias");
+        dt_bias_ = get(t, "dt_bias");
+        a_log_ = get(t, "A_log");
+        skip_ = get(t, "D");
+        norm_ = get(t, "norm");
+        w_o_ = get(t, "o");
+    }
+    Tensor forward(const Tensor& x, const StepBatch& batch, const LayerCache& cache, Runtime& rt) override {
+        Tensor read = project_and_read(x, nullptr, batch, cache, rt);
+        Tensor out = rt.ws.buf("space_mixer_out", rt.dtype, {x.shape[0], width_});
+        rt.ops.linear(read, w_o_->view, out, nullptr, rt.ws);
+        return out;
+    }
+    // h += mixer(norm(h)) with the norm folded into the one product in front and the sum into the one behind
+    bool forward_fused(const Tensor& h, const Norm::Foldable& norm, const StepBatch& batch, const LayerCache& cache,
+                       Runtime& rt) override {
+        if (!fused::fused_rows_ok(rt, batch, {width_, inner()}) || w_in_->view.dtype != rt.dtype || w_o_->view.dtype != rt.dtype) return false;
+        Tensor read = project_and_read(h, &norm, batch, cache, rt);
+        fused::linear_into_stream(rt, read, w_o_->view, h);
+        return true;
+    }
+
+private:
+    // norm null: x are normalised rows; else x is the stream and the norm is applied inside the product
+    Tensor project_and_read(const Tensor& x, const Norm::Foldable* norm, const StepBatch& batch, const LayerCache& cache, Runtime& rt) {
+        const long long T = x.shape[0];
+        Tensor proj = rt.ws.buf("space_proj", rt.dtype, {T, w_in_->view.shape[0]});
+        if (norm) fused::norm_linear(rt, x, *norm, w_in_->view, proj, Epilogue::Store);
+        else rt.ops.linear(x, w_in_->view, proj, nullptr, rt.ws);
+        Tensor xbc = rt.ws.buf("space_xbc", rt.dtype, {T, channels()});
+        rt.ops.conv_act(proj.cols(inner(), channels()), conv_w_->view, &conv_b_->view, cache.states.at("conv"), xbc, batch);
+        Tensor y = rt.ws.buf("space_y", DType::F32, {T, inner()});
+        const Tensor dt = proj.cols(inner() + channels(), shape_.heads);
+        Ops::DecayGates gates;
+        gates.dt = &dt;
+        gates.dt_bias = &dt_bias_->view;
+        gates.a_log = &a_log_->view;
+        gates.skip = &skip_->view;
+        rt.ops.decay_scan(xbc.cols(inner() + bc_width(), bc_width()), xbc.cols(inner(), bc_width()), xbc.cols(0, inner()), gates, shape_,
+                          cache.states.at("S"), y, batch, rt.ws);
+        Tensor read = rt.ws.buf("space_read", rt.dtype, {T, inner()});
+        rt.ops.gated_norm(y, proj.cols(0, inner()), norm_->view, norm_groups_, eps_, true, read);
+        return read;
+    }
+
+    long long width_ = 0, taps_ = 1;
+    int norm_groups_ = 1;
+    Ops::DecayShape shape_;
+    float eps_ = 1e-6f;
+    std::shared_ptr<DeviceTensor> w_in_, conv_w_, conv_b_, dt_bias_, a_log_, skip_, norm_, w_o_;
+};
+
 // ---------------------------------------------------------------------------- dense feed-forward with biases
 // mlp: W_down act(W_up x + b_up) + b_down; "activation": "gelu_tanh" (0.5 z (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3))))
 // or "relu2" (the square of relu) or "xielu" (for z > 0 softplus(p) z^2 + z / 2, else (1/2 + softplus(q)) (e^z - 1 - z) + z / 2
@@ -2405,6 +2704,8 @@ void register_builtin_parts() {
     r.parts["mixer"]["normed_pair"] = factory_of<NormedPair>();
     r.parts["mixer"]["gated_linear_attention"] = factory_of<GatedLinearAttention>();
     r.parts["mixer"]["matrix_memory"] = factory_of<MatrixMemory>();
+    r.parts["mixer"]["fixed_decay_attention"] = factory_of<FixedDecayAttention>();
+    r.parts["mixer"]["state_space"] = factory_of<StateSpace>();
     r.parts["ffn"]["mlp"] = factory_of<DenseMlp>();
     r.parts["token_input"]["gated_table"] = factory_of<GatedTableInput>();
     r.parts["depth_mix"]["weighted_history"] = factory_of<WeightedHistory>();

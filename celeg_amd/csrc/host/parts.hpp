@@ -101,7 +101,8 @@ public:
     using Part::Part;
     // inv_freq undefined: no rotation.  Pair i of the first rotary_dim values of a head turns by
     // position * inv_freq[i]; pairing 0: the pair is (i, i + rotary_dim/2), 1: (2i, 2i + 1).
-    struct Tables { Tensor inv_freq; int rotary_dim = 0; int pairing = 0; };
+    // amplitude: what cosine and sine are both multiplied by (a mixer that cannot refuses anything but 1).
+    struct Tables { Tensor inv_freq; int rotary_dim = 0; int pairing = 0; float amplitude = 1.f; };
     virtual Tables tables(Runtime& rt) = 0;
 };
 

@@ -1,4 +1,6 @@
-// A routed feed-forward: every row goes to `top` of E expert feed-forwards.
+// A routed feed-forward: every row goes to `top` of E expert feed-forwards.  Of a router's outputs the last ones
+// may be identity experts, whose result is the row itself: they take part in the choice, have no place in the
+// plan (place -1), and are added by `combine`.
 //   route:   scores from the router's 32-bit logits, the `top` largest chosen per row;
 //   plan:    rows sorted by expert (a row's place among its expert's rows is its order in the
 //            batch), and the list of row tiles that the products walk;
@@ -16,10 +18,15 @@
 // experts.  groups > 1: the experts form `groups` equal runs of neighbours, a run's score is the sum of
 // its two largest scores, and only experts of the `keep` best runs (the lower run among equal ones) can be
 // chosen.  The chosen experts' scores are the weights; with `renorm` they are divided by their sum plus
-// renorm_eps; then times `scale`.
+// renorm_eps; then times `scale`.  correction [experts] (or null) is added to the scores for the choice, of runs and
+// of experts, and not to the weights; group_best: a run's score is its largest one.  gate_out (or null): a row has one
+// logit more behind those of the experts, whose sigmoid goes to gate_out[row].
 struct MoeRule {
     int experts, top, score, renorm, groups, keep;
     float renorm_eps, scale;
+    const float* correction;
+    int group_best;
+    float* gate_out;
 };
 
 __device__ __forceinline__ float route_score(float z, int score, float zmax, float denom) {
@@ -47,8 +54,16 @@ __device__ __forceinline__ void route_row(const float* z, const MoeRule& rule, i
             if (lane + j * CELEG_WAVE < experts) s += expf(v[j] - zmax);
         denom = wave_sum(s);
     }
+    // what is compared: logits (the order of scores is that of logits), or corrected scores
+    const bool corrected = rule.correction != nullptr;
+    if (corrected)
+#pragma unroll
+        for (int j = 0; j < MOE_MAX_PER_LANE; ++j) {
+            const int e = lane + j * CELEG_WAVE;
+            if (e < experts) v[j] = route_score(v[j], score, zmax, denom) + rule.correction[e];
+        }
     if (rule.groups > 1) {
-        // every run's two largest scores (the largest logits give them), their sum in lane g of `mine`
+        // every run's two largest scores, their sum (or the larger one) in lane g of `mine`
         const int per = experts / rule.groups;
         float mine = -INFINITY;
         for (int g = 0; g < rule.groups; ++g) {
@@ -68,8 +83,8 @@ __device__ __forceinline__ void route_row(const float* z, const MoeRule& rule, i
                 second = fmaxf(lo, fmaxf(second, os));
                 first = hi;
             }
-            float sum = route_score(first, score, zmax, denom);
-            if (per > 1) sum += route_score(second, score, zmax, denom);
+            float sum = corrected ? first : route_score(first, score, zmax, denom);
+            if (per > 1 && !rule.group_best) sum += corrected ? second : route_score(second, score, zmax, denom);
             if (lane == g) mine = sum;
         }
         // the `keep` best runs stay; the experts of the others leave the choice
@@ -112,7 +127,7 @@ __device__ __forceinline__ void route_row(const float* z, const MoeRule& rule, i
 #pragma unroll
         for (int j = 0; j < MOE_MAX_PER_LANE; ++j)
             if (lane + j * CELEG_WAVE == best_e) v[j] = -INFINITY;
-        const float s = route_score(best, score, zmax, denom);
+        const float s = route_score(corrected ? z[min(best_e, experts - 1)] : best, score, zmax, denom);
         total += s;
         if (lane == 0) {
             ids[k] = best_e;
@@ -125,7 +140,9 @@ __device__ __forceinline__ void route_row(const float* z, const MoeRule& rule, i
 
 __global__ void moe_route_kernel(const float* __restrict__ logits, MoeRule rule, int* __restrict__ ids, float* __restrict__ weights) {
     const size_t t = blockIdx.x;
-    route_row(logits + t * rule.experts, rule, ids + t * rule.top, weights + t * rule.top);
+    const int ld = rule.experts + (rule.gate_out ? 1 : 0);
+    route_row(logits + t * ld, rule, ids + t * rule.top, weights + t * rule.top);
+    if (rule.gate_out && threadIdx.x == 0) rule.gate_out[t] = route_score(logits[t * ld + rule.experts], 0, 0.f, 1.f);
 }
 
 // The router's product and the choice in one kernel: a workgroup takes four rows, keeps them in LDS
@@ -135,7 +152,7 @@ __global__ void moe_route_kernel(const float* __restrict__ logits, MoeRule rule,
 template <typename TX>
 __global__ __launch_bounds__(256) void moe_router_kernel(const TX* __restrict__ x, const float* __restrict__ w, int rows,
                                                          int width, MoeRule rule, int* __restrict__ ids, float* __restrict__ weights) {
-    const int experts = rule.experts, top = rule.top;
+    const int top = rule.top, outs = rule.experts + (rule.gate_out ? 1 : 0);
     extern __shared__ float router_lds[];        // ROUTE_ROWS rows of width, then ROUTE_ROWS rows of logits
     float* xs = router_lds;
     float* zs = router_lds + ROUTE_ROWS * width;
@@ -146,7 +163,7 @@ __global__ __launch_bounds__(256) void moe_router_kernel(const TX* __restrict__ 
         xs[i] = row0 + r < rows ? to_float(x[static_cast<size_t>(row0) * width + i]) : 0.f;
     }
     __syncthreads();
-    for (int e = wave; e < experts; e += 4) {
+    for (int e = wave; e < outs; e += 4) {
         const float* we = w + static_cast<size_t>(e) * width;
         float acc[ROUTE_ROWS] = {0.f, 0.f, 0.f, 0.f};
         if ((width & 3) == 0) {
@@ -171,18 +188,20 @@ __global__ __launch_bounds__(256) void moe_router_kernel(const TX* __restrict__ 
 #pragma unroll
         for (int r = 0; r < ROUTE_ROWS; ++r) {
             const float total = wave_sum(acc[r]);
-            if (lane == 0) zs[r * experts + e] = total;
+            if (lane == 0) zs[r * outs + e] = total;
         }
     }
     __syncthreads();
     const int t = row0 + wave;
-    if (t < rows)
-        route_row(zs + wave * experts, rule, ids + static_cast<size_t>(t) * top, weights + static_cast<size_t>(t) * top);
+    if (t < rows) {
+        route_row(zs + wave * outs, rule, ids + static_cast<size_t>(t) * top, weights + static_cast<size_t>(t) * top);
+        if (rule.gate_out && lane == 0) rule.gate_out[t] = route_score(zs[wave * outs + rule.experts], 0, 0.f, 1.f);
+    }
 }
 
 // ---------------------------------------------------------------- plan
-// One workgroup.  ids [n] -> offsets [E + 1], place_of [n] (entry -> place), entry_at [n] (place ->
-// entry), and the tiles of `tile_rows` rows: tile_expert, tile_row0 [max_tiles], n_tiles.
+// One workgroup.  ids [n] -> offsets [E + 1], place_of [n] (entry -> place; -1 for ids from E on, which have
+// none), entry_at [n] (place -> entry, for the first offsets[E] places), and the tiles of `tile_rows` rows: tile_expert, tile_row0 [max_tiles], n_tiles.
 __global__ __launch_bounds__(1024) void moe_plan_kernel(const int* __restrict__ ids, int n, int experts, int tile_rows,
                                                         int* __restrict__ offsets, int* __restrict__ place_of,
                                                         int* __restrict__ entry_at, int* __restrict__ tile_expert,
@@ -223,7 +242,11 @@ __global__ __launch_bounds__(1024) void moe_plan_kernel(const int* __restrict__ 
     __syncthreads();
     for (int i = threadIdx.x; i < n; i += blockDim.x) {
         const int e = ids[i];
-        const int place = (e >= 0 && e < experts ? starts[e] : 0) + place_of[i];
+        if (e < 0 || e >= experts) {
+            place_of[i] = -1;
+            continue;
+        }
+        const int place = starts[e] + place_of[i];
         place_of[i] = place;
         entry_at[place] = i;
     }
@@ -232,9 +255,10 @@ __global__ __launch_bounds__(1024) void moe_plan_kernel(const int* __restrict__ 
 // ---------------------------------------------------------------- gather
 // a[p, :] = x[entry_at[p] / top, :] (* weight of the entry)
 template <typename T>
-__global__ void moe_gather_kernel(const T* __restrict__ x, const int* __restrict__ entry_at,
+__global__ void moe_gather_kernel(const T* __restrict__ x, const int* __restrict__ entry_at, const int* __restrict__ n_places,
                                   const float* __restrict__ weights, T* __restrict__ a, int top, int width) {
     const int p = blockIdx.x;
+    if (p >= *n_places) return;
     const int entry = entry_at[p];
     const float wgt = weights ? weights[entry] : 1.f;
     const T* src = x + static_cast<size_t>(entry / top) * width;
@@ -244,11 +268,20 @@ __global__ void moe_gather_kernel(const T* __restrict__ x, const int* __restrict
 
 // ---------------------------------------------------------------- product over the tiles
 // w: [E, N, K]; a: [n, K]; out: [n, N].  gated: w holds, per expert, N gate rows then N up rows, and
-// out = silu(a gate^T) * (a up^T) (the two sums rounded to T first, as where they are tensors).  Not gated, with
+// out = silu(a gate^T) * (a up^T) (the two sums rounded to T first, as where they are tensors); with act 2 the clamped
+// form g sigmoid(alpha g) (u + 1), g = min(gate, limit), u = clamp(up, -limit, limit).  Not gated, with
 // act 1: the square of relu of the sum (rounded to T first); act 0: the sum itself.
+__device__ __forceinline__ float moe_gated(float g, float u, int act, float limit, float alpha) {
+    if (act == 2) {
+        g = fminf(g, limit);
+        u = fminf(fmaxf(u, -limit), limit);
+        return (g / (1.0f + expf(-alpha * g))) * (u + 1.0f);
+    }
+    return (g / (1.0f + expf(-g))) * u;
+}
 template <typename T>
 __global__ __launch_bounds__(256) void moe_product_kernel(const T* __restrict__ a, const T* __restrict__ w,
-                                                          T* __restrict__ out, int N, int K, int gated, int act,
+                                                          T* __restrict__ out, int N, int K, int gated, int act, float limit, float alpha,
                                                           const int* __restrict__ offsets,
                                                           const int* __restrict__ tile_expert,
                                                           const int* __restrict__ tile_row0,
@@ -276,7 +309,7 @@ __global__ __launch_bounds__(256) void moe_product_kernel(const T* __restrict__ 
             float v = sums.v[i][j];
             if (gated) {
                 const float g = to_float(from_float<T>(v)), u = to_float(from_float<T>(ups.v[i][j]));
-                v = (g / (1.0f + expf(-g))) * u;
+                v = moe_gated(g, u, act, limit, alpha);
             } else if (act == 1) {
                 const float z = fmaxf(to_float(from_float<T>(v)), 0.f);
                 v = z * z;
@@ -292,7 +325,7 @@ __global__ __launch_bounds__(256) void moe_product_kernel(const T* __restrict__ 
 // workgroups pull the weights).
 template <bool GATED, int MOE_CT>
 __global__ __launch_bounds__(256, 2) void moe_product_mfma_kernel(const __bf16* __restrict__ a, const __bf16* __restrict__ w,
-                                                                  __bf16* __restrict__ out, int N, int K, int act,
+                                                                  __bf16* __restrict__ out, int N, int K, int act, float limit, float alpha,
                                                                   const int* __restrict__ offsets,
                                                                   const int* __restrict__ tile_expert,
                                                                   const int* __restrict__ tile_row0,
@@ -332,7 +365,7 @@ __global__ __launch_bounds__(256, 2) void moe_product_mfma_kernel(const __bf16* 
                 if (GATED) {
                     const float g = static_cast<float>(static_cast<__bf16>(x));
                     const float u = static_cast<float>(static_cast<__bf16>(sums[S - 1][ct][rt][r]));
-                    x = (g / (1.0f + expf(-g))) * u;
+                    x = moe_gated(g, u, act, limit, alpha);
                 } else if (act == 1) {
                     const float z = fmaxf(static_cast<float>(static_cast<__bf16>(x)), 0.f);
                     x = z * z;
@@ -345,20 +378,25 @@ __global__ __launch_bounds__(256, 2) void moe_product_mfma_kernel(const __bf16* 
 }
 
 // ---------------------------------------------------------------- combine
-// out[t, :] = (base[t, :] +) sum_k (weight of entry (t, k)) * y[place_of[t * top + k], :], summed in 32-bit
+// out[t, :] = (base_weight[t] * base[t, :] +) sum_k (weight of entry (t, k)) * y[place_of[t * top + k], :], summed in
+// 32-bit; an entry without a place (an identity expert's) takes x[t, :]
 template <typename T>
 __global__ void moe_combine_kernel(const T* __restrict__ y, const int* __restrict__ place_of,
-                                   const float* __restrict__ weights, const T* __restrict__ base, T* __restrict__ out, int top,
-                                   int width) {
+                                   const float* __restrict__ weights, const T* __restrict__ base, const float* __restrict__ base_weight,
+                                   const T* __restrict__ x, T* __restrict__ out, int top, int width) {
     const int t = blockIdx.x;
     for (int i = threadIdx.x; i < width; i += blockDim.x) {
         float acc = 0.f;
         for (int k = 0; k < top; ++k) {
             const int entry = t * top + k;
-            const float v = to_float(y[static_cast<size_t>(place_of[entry]) * width + i]);
+            const int place = place_of[entry];
+            const float v = place >= 0 ? to_float(y[static_cast<size_t>(place) * width + i]) : x ? to_float(x[static_cast<size_t>(t) * width + i]) : 0.f;
             acc += weights ? weights[entry] * v : v;
         }
-        if (base) acc += to_float(base[static_cast<size_t>(t) * width + i]);
+        if (base) {
+            const float v = to_float(base[static_cast<size_t>(t) * width + i]);
+            acc += base_weight ? base_weight[t] * v : v;
+        }
         out[static_cast<size_t>(t) * width + i] = from_float<T>(acc);
     }
 }
@@ -373,22 +411,24 @@ static bool moe_rule_ok(const MoeRule& r) {
 }
 
 extern "C" int celeg_moe_route(const float* logits, int rows, int experts, int top, int score, int renorm, int groups, int keep,
-                               float renorm_eps, float scale, int* ids, float* weights, hipStream_t stream) {
+                               float renorm_eps, float scale, const float* correction, int group_best, float* gate_out, int* ids,
+                               float* weights, hipStream_t stream) {
     if (rows <= 0) return 0;
-    const MoeRule rule{experts, top, score, renorm, groups, keep, renorm_eps, scale};
+    const MoeRule rule{experts, top, score, renorm, groups, keep, renorm_eps, scale, correction, group_best, gate_out};
     if (!moe_rule_ok(rule)) return static_cast<int>(hipErrorInvalidValue);
     hipLaunchKernelGGL(moe_route_kernel, dim3(rows), dim3(CELEG_WAVE), 0, stream, logits, rule, ids, weights);
     return CELEG_LAUNCH_RESULT();
 }
 
 // rows of a tile: 64 where every product of the plan runs on the matrix cores, else 32
-// x [rows, width] (32-bit or bfloat16) times the router's 32-bit matrix w [experts, width], then the choice
+// x [rows, width] (32-bit or bfloat16) times the router's 32-bit matrix w [experts (+ 1 with gate_out), width], then
+// the choice
 extern "C" int celeg_moe_router(const void* x, int x_dtype, const float* w, int rows, int width, int experts, int top,
-                                int score, int renorm, int groups, int keep, float renorm_eps, float scale, int* ids,
-                                float* weights, hipStream_t stream) {
+                                int score, int renorm, int groups, int keep, float renorm_eps, float scale, const float* correction,
+                                int group_best, float* gate_out, int* ids, float* weights, hipStream_t stream) {
     if (rows <= 0) return 0;
-    const size_t lds = static_cast<size_t>(ROUTE_ROWS) * (width + experts) * sizeof(float);
-    const MoeRule rule{experts, top, score, renorm, groups, keep, renorm_eps, scale};
+    const size_t lds = static_cast<size_t>(ROUTE_ROWS) * (width + experts + 1) * sizeof(float);
+    const MoeRule rule{experts, top, score, renorm, groups, keep, renorm_eps, scale, correction, group_best, gate_out};
     if (!moe_rule_ok(rule) || lds > 64 * 1024) return static_cast<int>(hipErrorInvalidValue);
     dim3 grid((rows + ROUTE_ROWS - 1) / ROUTE_ROWS);
     if (x_dtype == CELEG_F32)
@@ -411,20 +451,21 @@ extern "C" int celeg_moe_plan(const int* ids, int n, int experts, int tile_rows,
     return CELEG_LAUNCH_RESULT();
 }
 
-extern "C" int celeg_moe_gather(const void* x, int dtype, const int* entry_at, const float* weights, void* a, int n,
+// n_places: on the device, how many of the n places hold an entry
+extern "C" int celeg_moe_gather(const void* x, int dtype, const int* entry_at, const int* n_places, const float* weights, void* a, int n,
                                 int top, int width, hipStream_t stream) {
     if (n <= 0) return 0;
     if (dtype == CELEG_F32)
         hipLaunchKernelGGL(moe_gather_kernel<float>, dim3(n), dim3(256), 0, stream, static_cast<const float*>(x), entry_at,
-                           weights, static_cast<float*>(a), top, width);
+                           n_places, weights, static_cast<float*>(a), top, width);
     else
         hipLaunchKernelGGL(moe_gather_kernel<bf16>, dim3(n), dim3(256), 0, stream, static_cast<const bf16*>(x), entry_at,
-                           weights, static_cast<bf16*>(a), top, width);
+                           n_places, weights, static_cast<bf16*>(a), top, width);
     return CELEG_LAUNCH_RESULT();
 }
 
-extern "C" int celeg_moe_product(const void* a, const void* w, void* out, int dtype, int N, int K, int gated, int act,
-                                 const int* offsets, const int* tile_expert, const int* tile_row0, const int* n_tiles,
+extern "C" int celeg_moe_product(const void* a, const void* w, void* out, int dtype, int N, int K, int gated, int act, float limit,
+                                 float alpha, const int* offsets, const int* tile_expert, const int* tile_row0, const int* n_tiles,
                                  int max_tiles, int tile_rows, int wide, hipStream_t stream) {
     if (max_tiles <= 0) return 0;
     if (tile_rows == MR_ROWS) {
@@ -433,7 +474,7 @@ extern "C" int celeg_moe_product(const void* a, const void* w, void* out, int dt
         dim3 grid(max_tiles, (N + MR_COLS * ct - 1) / (MR_COLS * ct));
 #define MOE_GO(GATED, CT)                                                                                                       \
     hipLaunchKernelGGL((moe_product_mfma_kernel<GATED, CT>), grid, dim3(256), 0, stream, static_cast<const __bf16*>(a),         \
-                       static_cast<const __bf16*>(w), static_cast<__bf16*>(out), N, K, act, offsets, tile_expert, tile_row0, n_tiles)
+                       static_cast<const __bf16*>(w), static_cast<__bf16*>(out), N, K, act, limit, alpha, offsets, tile_expert, tile_row0, n_tiles)
         if (gated && wide) MOE_GO(true, 2);
         else if (gated) MOE_GO(true, 1);
         else if (wide) MOE_GO(false, 4);
@@ -445,24 +486,26 @@ extern "C" int celeg_moe_product(const void* a, const void* w, void* out, int dt
     dim3 grid(max_tiles, (N + SG_COLS - 1) / SG_COLS);
     if (dtype == CELEG_F32)
         hipLaunchKernelGGL(moe_product_kernel<float>, grid, dim3(256), 0, stream, static_cast<const float*>(a),
-                           static_cast<const float*>(w), static_cast<float*>(out), N, K, gated, act, offsets, tile_expert,
+                           static_cast<const float*>(w), static_cast<float*>(out), N, K, gated, act, limit, alpha, offsets, tile_expert,
                            tile_row0, n_tiles);
     else
         hipLaunchKernelGGL(moe_product_kernel<bf16>, grid, dim3(256), 0, stream, static_cast<const bf16*>(a),
-                           static_cast<const bf16*>(w), static_cast<bf16*>(out), N, K, gated, act, offsets, tile_expert,
+                           static_cast<const bf16*>(w), static_cast<bf16*>(out), N, K, gated, act, limit, alpha, offsets, tile_expert,
                            tile_row0, n_tiles);
     return CELEG_LAUNCH_RESULT();
 }
 
-// base: rows [rows, width] added to the sum (what every row gets besides its experts), or null
-extern "C" int celeg_moe_combine(const void* y, int dtype, const int* place_of, const float* weights, const void* base, void* out,
-                                 int rows, int top, int width, hipStream_t stream) {
+// base: rows [rows, width] added to the sum (what every row gets besides its experts; times base_weight [rows] unless
+// null), or null; x: the rows themselves, for identity experts (null: there are none)
+extern "C" int celeg_moe_combine(const void* y, int dtype, const int* place_of, const float* weights, const void* base,
+                                 const float* base_weight, const void* x, void* out, int rows, int top, int width, hipStream_t stream) {
     if (rows <= 0) return 0;
     if (dtype == CELEG_F32)
         hipLaunchKernelGGL(moe_combine_kernel<float>, dim3(rows), dim3(256), 0, stream, static_cast<const float*>(y),
-                           place_of, weights, static_cast<const float*>(base), static_cast<float*>(out), top, width);
+                           place_of, weights, static_cast<const float*>(base), base_weight, static_cast<const float*>(x), static_cast<float*>(out), top,
+                           width);
     else
         hipLaunchKernelGGL(moe_combine_kernel<bf16>, dim3(rows), dim3(256), 0, stream, static_cast<const bf16*>(y), place_of,
-                           weights, static_cast<const bf16*>(base), static_cast<bf16*>(out), top, width);
+                           weights, static_cast<const bf16*>(base), base_weight, static_cast<const bf16*>(x), static_cast<bf16*>(out), top, width);
     return CELEG_LAUNCH_RESULT();
 }
