@@ -256,6 +256,47 @@ MINILORN_SHAPES = {
            minilorn_beside(2048, 16, 8, 128, 1024, 16, 8, 128, 128, 4096)),
 }
 
+# Nosalorn beside Kivorax, the closest existing design with attention, recurrences with a matrix state per head and routed
+# experts: Kivorax's pair of attention and recurrent unit where Nosalorn has windowed attention, gated linear attention with
+# as many state numbers where it has linear attention with fixed decays or the state space, and as many experts a token as
+# Nosalorn's chosen and shared ones together.
+NOSALORN_PATTERN = "maalmaal"
+
+
+def nosalorn_shape(width, heads, kv_heads, dim, window, l_heads, l_dim, l_vdim, m_heads, m_vdim, state, groups, experts, identity, top,
+                   expert_groups, ff, vocab=65536):
+    kinds = {"a": ("attention", {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "scale": dim ** -0.5, "v_mix": True,
+                                 "rot": {"base": 500000.0, "dims": dim // 2,
+                                         "scaling": {"factor": 4.0, "original": 2048, "fast": 32.0, "slow": 1.0}},
+                                 "mask": {"size": window, "keep_first": 4}}),
+             "l": ("lightning", {"heads": l_heads, "dim": l_dim, "vdim": l_vdim,
+                                 "decay": [1.0 - 0.5 ** (1.0 + 8.0 * i / l_heads) for i in range(l_heads)]}),
+             "m": ("mamba2", {"heads": m_heads, "vdim": m_vdim, "state": state, "groups": groups, "conv": 4, "norm_groups": groups})}
+    moe = {"kind": "moe", "expert": {"ff": ff, "limit": 7.0}, "shared": {"ff": ff, "limit": 7.0},
+           "router": {"experts": experts, "identity": identity, "top": top, "scale": 2.0,
+                      "groups": {"count": expert_groups[0], "keep": expert_groups[1]}}}
+    layers = [{"type": kinds[c][0], "mixer": kinds[c][1], "mlp": moe} for c in NOSALORN_PATTERN]
+    layers[0]["mlp"] = {"kind": "dense", "ff": ff * (top + 1)}
+    return {"architecture": "Nosalorn", "vocab": vocab, "width": width, "norm": {"eps": 1e-5}, "embedding": {"scale": 1.0},
+            "max_context": 8192, "layers": layers}
+
+
+def kivorax_beside(width, heads, kv_heads, dim, inner, blocks, l_heads, l_dim, l_vdim, m_heads, m_dim, m_vdim, experts, top, ff):
+    cfg = kivorax_shape(width, "".join("p" if c == "a" else "g" for c in NOSALORN_PATTERN), heads, kv_heads, dim, dim, inner, blocks,
+                        l_heads, l_heads, l_dim, l_vdim, experts, top, ff)
+    for c, layer in zip(NOSALORN_PATTERN, cfg["layers"]):
+        if c == "m":
+            layer["mixer"] = dict(layer["mixer"], heads=m_heads, dim=m_dim, vdim=m_vdim)
+    return cfg
+
+
+NOSALORN_SHAPES = {
+    "1k": (nosalorn_shape(1024, 16, 8, 64, 1024, 16, 64, 64, 32, 64, 128, 2, 14, 2, 2, (4, 2), 1024),
+           kivorax_beside(1024, 16, 8, 64, 1024, 8, 16, 64, 64, 16, 128, 128, 16, 3, 1024)),
+    "2k": (nosalorn_shape(2048, 16, 8, 128, 1024, 16, 128, 128, 64, 64, 128, 8, 28, 4, 4, (4, 2), 1024),
+           kivorax_beside(2048, 16, 8, 128, 2048, 8, 16, 128, 128, 32, 128, 128, 32, 5, 1024)),
+}
+
 DESIGN_SHAPES = {
     "1k": (regipel_shape(1024, 8, 16, 64, 32, 64, 256, 16, 2, 1024), lfm2_shape(1024, 16, 8, 2048, set(range(8)), 8, 8192)),
     "2k": (regipel_shape(2048, 8, 16, 128, 64, 128, 512, 32, 4, 1024), lfm2_shape(2048, 32, 8, 4096, set(range(8)), 8, 8192)),
@@ -273,7 +314,7 @@ def design(shapes, steps: int, warmup: int, batch: int, layers: int = 0, profile
     for shape in shapes:
         table, beside = {"kifetar": (KIFETAR_SHAPES, "lfm2_hybrid"), "kivorax": (KIVORAX_SHAPES, "kifetar_beside"),
                          "regipel": (DESIGN_SHAPES, "lfm2_attention"), "vabuzen": (VABUZEN_SHAPES, "regipel_beside"),
-                         "minilorn": (MINILORN_SHAPES, "kifetar_beside")}[which]
+                         "minilorn": (MINILORN_SHAPES, "kifetar_beside"), "nosalorn": (NOSALORN_SHAPES, "kivorax_beside")}[which]
         for label, cfg in zip((which, beside), table[shape]):
             if profile_only and label != profile_only:
                 continue
@@ -306,7 +347,8 @@ def design(shapes, steps: int, warmup: int, batch: int, layers: int = 0, profile
     title = {"kifetar": "Kifetar beside LFM2 convolution and attention layers", "regipel": "Regipel beside LFM2 attention layers",
              "kivorax": "Kivorax beside Kifetar attention and delta-rule layers",
              "vabuzen": "Vabuzen beside Regipel layers of one residual stream",
-             "minilorn": "Minilorn beside Kifetar attention and delta-rule layers"}[which]
+             "minilorn": "Minilorn beside Kifetar attention and delta-rule layers",
+             "nosalorn": "Nosalorn beside Kivorax attention and gated linear attention layers"}[which]
     print(json.dumps({"metric": title + " at equal size: prefill tok/s @ 2048 tokens, "
                                 f"decode tok/s @ batch {batch}, context 2048 (bf16, random weights)",
                       "phase": "design", "design": which, "batch": batch, "steps": steps, "warmup": warmup, "dtype": "bf16",
@@ -336,9 +378,9 @@ def main() -> int:
                          "(default 2048, the headline's); with --phase prefill: tokens of the same "
                          "prompt that the cache holds before the measured portion of 2,048 (default 0)")
     ap.add_argument("--design-shape", default="1k,2k", help="with --phase design: which sizes (1k, 2k)")
-    ap.add_argument("--design", default="regipel", choices=["regipel", "kifetar", "kivorax", "vabuzen", "minilorn"],
+    ap.add_argument("--design", default="regipel", choices=["regipel", "kifetar", "kivorax", "vabuzen", "minilorn", "nosalorn"],
                     help="with --phase design: which design is measured beside its closest LFM2 shape")
-    ap.add_argument("--design-model", default="", choices=["", "regipel", "lfm2_attention", "kifetar", "lfm2_hybrid", "kivorax", "kifetar_beside", "vabuzen", "regipel_beside", "minilorn"],
+    ap.add_argument("--design-model", default="", choices=["", "regipel", "lfm2_attention", "kifetar", "lfm2_hybrid", "kivorax", "kifetar_beside", "vabuzen", "regipel_beside", "minilorn", "nosalorn", "kivorax_beside"],
                     help="with --phase design: only this model (for profiling)")
     ap.add_argument("--phase", choices=["all", "prefill", "decode", "serve", "design"], default="all",
                     help="for profiling: run only the prefill measurement, or only the batch-8 "

@@ -1719,7 +1719,7 @@ ModelSpec nosalorn_build_spec(const Json& c) {
                                   .set("head_dim", m["dim"]).set("pairing", "halves");
                 if (!m["rot"]["scaling"].is_null()) {
                     Json scaling = m["rot"]["scaling"];
-                    rope.params.set("scaling", scaling.set("kind", "yarn"));
+                    rope.params.set("scaling", scaling.set("rule", "yarn"));
                 }
                 layer.mixer.params.set("position", rope.to_json());
             }

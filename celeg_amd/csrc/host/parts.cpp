@@ -257,8 +257,8 @@ public:
             if (!sc.is_object()) throw SpecError("rope: scaling must be an object");
             scaled_ = true;
             factor_ = sc.get_double("factor", 1.0);
-            const std::string kind = sc.get_string("kind", "wavelength");
-            if (kind == "yarn") {
+            const std::string rule = sc.get_string("rule", "wavelength");
+            if (rule == "yarn") {
                 yarn_ = true;
                 original_ = sc.get_double("original", 0.0);
                 const double fast = sc.get_double("fast", 0.0), slow = sc.get_double("slow", 0.0);
@@ -272,7 +272,7 @@ public:
                 amplitude_ = 0.1 * std::log(factor_) + 1.0;
                 return;
             }
-            if (kind != "wavelength") throw SpecError("rope: scaling is 'wavelength' or 'yarn', not '" + kind + "'");
+            if (rule != "wavelength") throw SpecError("rope: scaling.rule is 'wavelength' or 'yarn', not '" + rule + "'");
             low_ = sc.get_double("low", 1.0);
             high_ = sc.get_double("high", 1.0);
             original_ = sc.get_double("original", 0.0);
@@ -295,7 +295,7 @@ private:
     // "scaling" {factor, low, high, original}: frequencies whose wavelength 2 pi / f is below
     // original / high stay, above original / low become f / factor, and between the two
     // (1 - s) f / factor + s f with s = (original / wavelength - low) / (high - low).
-    // "kind": "yarn" {factor, original, fast, slow}: with d(t) the pair (a fraction) whose wavelength fits t times into
+    // "rule": "yarn" {factor, original, fast, slow}: with d(t) the pair (a fraction) whose wavelength fits t times into
     // `original`, pairs up to floor(d(fast)) keep their frequency, those from ceil(d(slow)) on have f / factor, and
     // between the two lies a line in the pair's number; cosine and sine are multiplied by 0.1 ln(factor) + 1.
     double scaled(double f, int i) const {
