@@ -324,15 +324,20 @@ def drawn_model(rng):
 @pytest.mark.parametrize("seed", range(8))
 def test_models_drawn_at_random(tmp_path, seed):
     """Eight models drawn at random, weights stored in bfloat16, four requests of 20 to 200 tokens,
-    in a mixed schedule and in long and short portions, in 32-bit and in bfloat16."""
+    in a mixed schedule and in long and short portions, in 32-bit and in bfloat16.  For bfloat16 the corrections lie
+    further apart than scores can, so that no choice of experts hangs on the rounding of a row (a changed choice moves the row
+    and, through states and keys, all later ones); the choices themselves are what the 32-bit runs hold."""
     rng = random.Random(4000 + seed)
     cfg = drawn_model(rng)
-    folder = write_model(tmp_path / "drawn", cfg, seed, torch.bfloat16, std=0.06)
-    c, W = plain.load_model_folder(folder)
     reqs = {f"r{i}": random_tokens(cfg["vocab"], rng.randint(20, 200), seed=seed * 10 + i) for i in range(4)}
-    ref = {rid: plain.model_logits(c, W, toks) for rid, toks in reqs.items()}
+    tail = rng.randint(3, 20)
     for dtype in ("float32", "bfloat16"):
-        for steps in (mixed_schedule(reqs, seed=seed, decode_tail=rng.randint(3, 20)), portions_schedule(reqs, sizes=(70, 2, 33, 1, 130, 16, 5))):
+        decided = {f"l{i}.mlp.correction": lambda w: 1.5 * w.argsort().argsort().float() for i, layer in enumerate(cfg["layers"])
+                   if layer["mlp"] and layer["mlp"]["kind"] == "moe" and dtype == "bfloat16"}
+        folder = write_model(tmp_path / dtype, cfg, seed, torch.bfloat16, std=0.06, change=decided)
+        c, W = plain.load_model_folder(folder)
+        ref = {rid: plain.model_logits(c, W, toks) for rid, toks in reqs.items()}
+        for steps in (mixed_schedule(reqs, seed=seed, decode_tail=tail), portions_schedule(reqs, sizes=(70, 2, 33, 1, 130, 16, 5))):
             lm, _ = load(folder, dtype, steps)
             got = EngineDriver(lm).run(steps)
             for rid in reqs:
