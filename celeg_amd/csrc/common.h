@@ -127,6 +127,31 @@ __device__ __forceinline__ float lanes_sum(float v) {
     return v;
 }
 
+// four neighbouring values, on a boundary of four, as 32-bit numbers
+template <typename T> struct Vec4;
+template <> struct Vec4<float> {
+    typedef float raw __attribute__((ext_vector_type(4)));
+    static __device__ __forceinline__ void load(const float* p, float (&v)[4]) {
+        const raw r = *reinterpret_cast<const raw*>(p);
+        v[0] = r[0]; v[1] = r[1]; v[2] = r[2]; v[3] = r[3];
+    }
+    static __device__ __forceinline__ void store(float* p, const float (&v)[4]) {
+        *reinterpret_cast<raw*>(p) = raw{v[0], v[1], v[2], v[3]};
+    }
+};
+template <> struct Vec4<bf16> {
+    typedef __bf16 raw __attribute__((ext_vector_type(4)));
+    static __device__ __forceinline__ void load(const bf16* p, float (&v)[4]) {
+        const raw r = *reinterpret_cast<const raw*>(p);
+        v[0] = static_cast<float>(r[0]); v[1] = static_cast<float>(r[1]);
+        v[2] = static_cast<float>(r[2]); v[3] = static_cast<float>(r[3]);
+    }
+    static __device__ __forceinline__ void store(bf16* p, const float (&v)[4]) {
+        *reinterpret_cast<raw*>(p) = raw{static_cast<__bf16>(v[0]), static_cast<__bf16>(v[1]),
+                                         static_cast<__bf16>(v[2]), static_cast<__bf16>(v[3])};
+    }
+};
+
 #define CELEG_LAUNCH_RESULT() static_cast<int>(hipGetLastError())
 
 enum CelegDtype { CELEG_F32 = 0, CELEG_BF16 = 1 };

@@ -471,11 +471,11 @@ int ds_rows(const DsArgs& a, int max_chunks, hipStream_t stream) {
 
 // ---------------------------------------------------------------- convolution with bias and silu
 // y_t[c] = silu(bias[c] + sum_j w[j, c] u_(t - taps + 1 + j)[c]); saved [slots][taps - 1][channels] keeps a
-// request's last inputs.  A thread owns VEC neighbouring channels of CONV_ROWS rows.  The first taps - 1 rows of
+// request's last inputs.  A thread owns VEC neighbouring channels of rows_each rows.  The first taps - 1 rows of
 // a portion, the only ones that read the saved inputs, are all computed by the block that holds the portion's
 // first row, whose threads then leave the new inputs.
 // TAPS: their number where it is known to the compiler (the inputs then move through registers), 0: any.
-#define CONV_ROWS 8
+// (also gated_norm's loads)
 template <typename T, int VEC>
 __device__ __forceinline__ void conv_load(const T* p, float (&x)[VEC]) {
     if (VEC == 4) {
@@ -488,8 +488,11 @@ __device__ __forceinline__ void conv_load(const T* p, float (&x)[VEC]) {
 }
 template <typename T, int VEC>
 __device__ __forceinline__ void conv_store(T* p, const float (&y)[VEC]) {
+    float z[VEC];
 #pragma unroll
-    for (int e = 0; e < VEC; ++e) p[e] = from_float<T>(ds_silu(y[e]));
+    for (int e = 0; e < VEC; ++e) z[e] = ds_silu(y[e]);
+    if constexpr (VEC == 4) Vec4<T>::store(p, z);
+    else p[0] = from_float<T>(z[0]);
 }
 
 template <typename T, int VEC, int TAPS>
@@ -497,11 +500,11 @@ __global__ __launch_bounds__(CELEG_WAVE) void conv_act_kernel(const T* __restric
                                                               const float* __restrict__ bias, float* __restrict__ state,
                                                               size_t state_stride, const int* __restrict__ token_seq,
                                                               const int* __restrict__ cu_seqlens, const int* __restrict__ seq_slot,
-                                                              T* __restrict__ out, int ldo, int n_rows, int channels, int n_taps) {
+                                                              T* __restrict__ out, int ldo, int n_rows, int channels, int n_taps, int rows_each) {
     const int taps = TAPS > 0 ? TAPS : n_taps;
     const int c = (blockIdx.x * CELEG_WAVE + threadIdx.x) * VEC;
     if (c >= channels) return;
-    const int r0 = blockIdx.y * CONV_ROWS, r1 = min(r0 + CONV_ROWS, n_rows);
+    const int r0 = blockIdx.y * rows_each, r1 = min(r0 + rows_each, n_rows);
     const T* mine = u + c;
     float held_w[TAPS > 0 ? TAPS : 1][VEC], b[VEC];
 #pragma unroll
@@ -584,46 +587,65 @@ __global__ __launch_bounds__(CELEG_WAVE) void conv_act_kernel(const T* __restric
 // ---------------------------------------------------------------- gate and norm
 // One workgroup per (row, part).  mode 0: o / rms(o) * weight * sigmoid(gate); mode 1: y = o * silu(gate), then
 // y / rms(y) * weight.  The mean of squares runs over the part's `size` values.
-template <typename T>
+// VEC neighbouring values a thread and turn.
+template <typename T, int VEC>
 __global__ __launch_bounds__(256) void gated_norm_kernel(const float* __restrict__ o, int ldo, const T* __restrict__ gate, int ldg,
                                                          const float* __restrict__ weight, T* __restrict__ out, int ld, int size,
                                                          float eps, int mode) {
     __shared__ float scratch[16];
-    constexpr int HELD = 8;
+    constexpr int HELD = VEC == 4 ? 4 : 8;
     const size_t t = blockIdx.x;
-    const int base = blockIdx.y * size;
+    const int base = blockIdx.y * size, first = threadIdx.x * VEC, step = blockDim.x * VEC;
     const float* x = o + t * ldo + base;
     const T* g = gate + t * ldg + base;
-    float held[HELD], sq = 0.f;
+    const float* w = weight + base;
+    auto fetch = [&](int i, float (&y)[VEC], float (&z)[VEC]) __attribute__((always_inline)) {     // values (gated in mode 1) and gates
+        conv_load<float, VEC>(x + i, y);
+        conv_load<T, VEC>(g + i, z);
+        if (mode == 1)
+#pragma unroll
+            for (int e = 0; e < VEC; ++e) y[e] *= ds_silu(z[e]);
+    };
+    float held[HELD][VEC], held_z[HELD][VEC], sq = 0.f;
 #pragma unroll
     for (int u = 0; u < HELD; ++u) {
-        const int i = threadIdx.x + u * blockDim.x;
-        held[u] = 0.f;
+        const int i = first + u * step;
         if (i < size) {
-            held[u] = x[i];
-            if (mode == 1) held[u] *= ds_silu(to_float(g[i]));
-            sq = fmaf(held[u], held[u], sq);
+            fetch(i, held[u], held_z[u]);
+#pragma unroll
+            for (int e = 0; e < VEC; ++e) sq = fmaf(held[u][e], held[u][e], sq);
         }
     }
-    for (int i = threadIdx.x + HELD * blockDim.x; i < size; i += blockDim.x) {
-        const float y = mode == 1 ? x[i] * ds_silu(to_float(g[i])) : x[i];
-        sq = fmaf(y, y, sq);
+    for (int i = first + HELD * step; i < size; i += step) {
+        float y[VEC], z[VEC];
+        fetch(i, y, z);
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) sq = fmaf(y[e], y[e], sq);
     }
     sq = block_sum(sq, scratch);
     const float unit = 1.0f / sqrtf(sq / static_cast<float>(size) + eps);
     T* dst = out + t * ld + base;
-    auto finish = [&](int i, float y) __attribute__((always_inline)) {
-        float z = y * unit * weight[base + i];
-        if (mode == 0) z *= ds_sigmoid(to_float(g[i]));
-        dst[i] = from_float<T>(z);
+    auto finish = [&](int i, float (&y)[VEC], const float (&z)[VEC]) __attribute__((always_inline)) {
+        float wv[VEC];
+        conv_load<float, VEC>(w + i, wv);
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) {
+            y[e] *= unit * wv[e];
+            if (mode == 0) y[e] *= ds_sigmoid(z[e]);
+        }
+        if constexpr (VEC == 4) Vec4<T>::store(dst + i, y);
+        else dst[i] = from_float<T>(y[0]);
     };
 #pragma unroll
     for (int u = 0; u < HELD; ++u) {
-        const int i = threadIdx.x + u * blockDim.x;
-        if (i < size) finish(i, held[u]);
+        const int i = first + u * step;
+        if (i < size) finish(i, held[u], held_z[u]);
     }
-    for (int i = threadIdx.x + HELD * blockDim.x; i < size; i += blockDim.x)
-        finish(i, mode == 1 ? x[i] * ds_silu(to_float(g[i])) : x[i]);
+    for (int i = first + HELD * step; i < size; i += step) {
+        float y[VEC], z[VEC];
+        fetch(i, y, z);
+        finish(i, y, z);
+    }
 }
 
 }  // namespace
@@ -698,13 +720,15 @@ extern "C" int celeg_conv_act(const void* u, int ldu, int dtype, const float* w,
     if (channels <= 0 || taps <= 0) return static_cast<int>(hipErrorInvalidValue);
     const uintptr_t four = dtype == CELEG_F32 ? 16 : 8;
     // (weights and saved inputs are read by fours as well)
-    const bool by_fours = ((channels | ldu) & 3) == 0 && (state_stride & 3) == 0 && (reinterpret_cast<uintptr_t>(u) & (four - 1)) == 0 &&
+    const bool by_fours = ((channels | ldu | ldo) & 3) == 0 && (state_stride & 3) == 0 &&
+                          ((reinterpret_cast<uintptr_t>(u) | reinterpret_cast<uintptr_t>(out)) & (four - 1)) == 0 &&
                           ((reinterpret_cast<uintptr_t>(w) | reinterpret_cast<uintptr_t>(state)) & 15) == 0;
     const int per_block = CELEG_WAVE * (by_fours ? 4 : 1);
-    dim3 grid((channels + per_block - 1) / per_block, (n_rows + CONV_ROWS - 1) / CONV_ROWS), block(CELEG_WAVE);
+    const int rows_each = n_rows <= 128 ? 1 : 8;         // (few rows: latency is what counts)
+    dim3 grid((channels + per_block - 1) / per_block, (n_rows + rows_each - 1) / rows_each), block(CELEG_WAVE);
 #define CONV_GO_TAPS(T, VEC, TAPS)                                                                                                   \
     hipLaunchKernelGGL((conv_act_kernel<T, VEC, TAPS>), grid, block, 0, stream, static_cast<const T*>(u), ldu, w, bias, state, state_stride, \
-                       token_seq, cu_seqlens, seq_slot, static_cast<T*>(out), ldo, n_rows, channels, taps)
+                       token_seq, cu_seqlens, seq_slot, static_cast<T*>(out), ldo, n_rows, channels, taps, rows_each)
 #define CONV_GO(T, VEC)                        \
     switch (taps) {                            \
         case 2: CONV_GO_TAPS(T, VEC, 2); break; \
@@ -731,12 +755,19 @@ extern "C" int celeg_gated_norm(const float* o, int ldo, const void* gate, int l
                                 int rows, int parts, int size, float eps, int mode, hipStream_t stream) {
     if (rows <= 0) return 0;
     if (parts <= 0 || parts > 65535 || size <= 0 || mode < 0 || mode > 1) return static_cast<int>(hipErrorInvalidValue);
-    dim3 grid(rows, parts), block(size <= 64 ? 64 : size <= 128 ? 128 : 256);
-    if (dtype == CELEG_F32)
-        hipLaunchKernelGGL(gated_norm_kernel<float>, grid, block, 0, stream, o, ldo, static_cast<const float*>(gate), ldg, weight,
-                           static_cast<float*>(out), ld, size, eps, mode);
-    else
-        hipLaunchKernelGGL(gated_norm_kernel<bf16>, grid, block, 0, stream, o, ldo, static_cast<const bf16*>(gate), ldg, weight,
-                           static_cast<bf16*>(out), ld, size, eps, mode);
+    const uintptr_t ends = reinterpret_cast<uintptr_t>(o) | reinterpret_cast<uintptr_t>(gate) | reinterpret_cast<uintptr_t>(weight) |
+                           reinterpret_cast<uintptr_t>(out);
+    const uintptr_t half = dtype == CELEG_F32 ? 15 : 7;
+    const bool by_fours = ((size | ldo | ldg | ld) & 3) == 0 && (ends & half) == 0 && ((reinterpret_cast<uintptr_t>(o) | reinterpret_cast<uintptr_t>(weight)) & 15) == 0;
+    const int turns = by_fours ? size / 4 : size;
+    dim3 grid(rows, parts), block(turns <= 64 ? 64 : turns <= 128 ? 128 : 256);
+#define NORM_GO(T, VEC)                                                                                                              \
+    hipLaunchKernelGGL((gated_norm_kernel<T, VEC>), grid, block, 0, stream, o, ldo, static_cast<const T*>(gate), ldg, weight,          \
+                       static_cast<T*>(out), ld, size, eps, mode)
+    if (dtype == CELEG_F32 && by_fours) NORM_GO(float, 4);
+    else if (dtype == CELEG_F32) NORM_GO(float, 1);
+    else if (by_fours) NORM_GO(bf16, 4);
+    else NORM_GO(bf16, 1);
+#undef NORM_GO
     return CELEG_LAUNCH_RESULT();
 }

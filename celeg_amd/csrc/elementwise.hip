@@ -140,30 +140,6 @@ __global__ void rmsnorm_kernel(TX* __restrict__ x, const TD* __restrict__ delta,
 // The same with the row kept in registers: groups of 4 values, up to RMS_NV groups a
 // thread (width <= 4 * RMS_NV * 256), every load of a row asked for before the first is used.
 #define RMS_NV 4
-template <typename T> struct Vec4;
-template <> struct Vec4<float> {
-    typedef float raw __attribute__((ext_vector_type(4)));
-    static __device__ __forceinline__ void load(const float* p, float (&v)[4]) {
-        const raw r = *reinterpret_cast<const raw*>(p);
-        v[0] = r[0]; v[1] = r[1]; v[2] = r[2]; v[3] = r[3];
-    }
-    static __device__ __forceinline__ void store(float* p, const float (&v)[4]) {
-        *reinterpret_cast<raw*>(p) = raw{v[0], v[1], v[2], v[3]};
-    }
-};
-template <> struct Vec4<bf16> {
-    typedef __bf16 raw __attribute__((ext_vector_type(4)));
-    static __device__ __forceinline__ void load(const bf16* p, float (&v)[4]) {
-        const raw r = *reinterpret_cast<const raw*>(p);
-        v[0] = static_cast<float>(r[0]); v[1] = static_cast<float>(r[1]);
-        v[2] = static_cast<float>(r[2]); v[3] = static_cast<float>(r[3]);
-    }
-    static __device__ __forceinline__ void store(bf16* p, const float (&v)[4]) {
-        *reinterpret_cast<raw*>(p) = raw{static_cast<__bf16>(v[0]), static_cast<__bf16>(v[1]),
-                                         static_cast<__bf16>(v[2]), static_cast<__bf16>(v[3])};
-    }
-};
-
 template <typename TX, typename TD, typename TO>
 __global__ __launch_bounds__(256) void rmsnorm_vec_kernel(
     TX* __restrict__ x, const TD* __restrict__ delta, const float* __restrict__ w,

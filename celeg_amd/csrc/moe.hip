@@ -147,10 +147,11 @@ __global__ void moe_route_kernel(const float* __restrict__ logits, MoeRule rule,
 
 // The router's product and the choice in one kernel: a workgroup takes four rows, keeps them in LDS
 // in 32-bit, its wavefronts share out the experts (a weight is read once for the four rows; a row's
-// sum runs over k in an order that depends on nothing else), then each wavefront routes one row.
+// sum runs over k in an order that depends on nothing else), then each wavefront routes one row.  THREADS: 256, or 1,024
+// where there are few workgroups and their latency is what counts.
 #define ROUTE_ROWS 4
-template <typename TX>
-__global__ __launch_bounds__(256) void moe_router_kernel(const TX* __restrict__ x, const float* __restrict__ w, int rows,
+template <typename TX, int THREADS>
+__global__ __launch_bounds__(THREADS) void moe_router_kernel(const TX* __restrict__ x, const float* __restrict__ w, int rows,
                                                          int width, MoeRule rule, int* __restrict__ ids, float* __restrict__ weights) {
     const int top = rule.top, outs = rule.experts + (rule.gate_out ? 1 : 0);
     extern __shared__ float router_lds[];        // ROUTE_ROWS rows of width, then ROUTE_ROWS rows of logits
@@ -158,12 +159,12 @@ __global__ __launch_bounds__(256) void moe_router_kernel(const TX* __restrict__ 
     float* zs = router_lds + ROUTE_ROWS * width;
     const int row0 = blockIdx.x * ROUTE_ROWS;
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-    for (int i = threadIdx.x; i < ROUTE_ROWS * width; i += 256) {
+    for (int i = threadIdx.x; i < ROUTE_ROWS * width; i += THREADS) {
         const int r = i / width;
         xs[i] = row0 + r < rows ? to_float(x[static_cast<size_t>(row0) * width + i]) : 0.f;
     }
     __syncthreads();
-    for (int e = wave; e < outs; e += 4) {
+    for (int e = wave; e < outs; e += THREADS / CELEG_WAVE) {
         const float* we = w + static_cast<size_t>(e) * width;
         float acc[ROUTE_ROWS] = {0.f, 0.f, 0.f, 0.f};
         if ((width & 3) == 0) {
@@ -193,7 +194,7 @@ __global__ __launch_bounds__(256) void moe_router_kernel(const TX* __restrict__ 
     }
     __syncthreads();
     const int t = row0 + wave;
-    if (t < rows) {
+    if (wave < ROUTE_ROWS && t < rows) {
         route_row(zs + wave * outs, rule, ids + static_cast<size_t>(t) * top, weights + static_cast<size_t>(t) * top);
         if (rule.gate_out && lane == 0) rule.gate_out[t] = route_score(zs[wave * outs + rule.experts], 0, 0.f, 1.f);
     }
@@ -380,25 +381,39 @@ __global__ __launch_bounds__(256, 2) void moe_product_mfma_kernel(const __bf16* 
 // ---------------------------------------------------------------- combine
 // out[t, :] = (base_weight[t] * base[t, :] +) sum_k (weight of entry (t, k)) * y[place_of[t * top + k], :], summed in
 // 32-bit; an entry without a place (an identity expert's) takes x[t, :]
-template <typename T>
-__global__ void moe_combine_kernel(const T* __restrict__ y, const int* __restrict__ place_of,
-                                   const float* __restrict__ weights, const T* __restrict__ base, const float* __restrict__ base_weight,
-                                   const T* __restrict__ x, T* __restrict__ out, int top, int width) {
-    const int t = blockIdx.x;
-    for (int i = threadIdx.x; i < width; i += blockDim.x) {
-        float acc = 0.f;
-        for (int k = 0; k < top; ++k) {
-            const int entry = t * top + k;
-            const int place = place_of[entry];
-            const float v = place >= 0 ? to_float(y[static_cast<size_t>(place) * width + i]) : x ? to_float(x[static_cast<size_t>(t) * width + i]) : 0.f;
-            acc += weights ? weights[entry] * v : v;
-        }
-        if (base) {
-            const float v = to_float(base[static_cast<size_t>(t) * width + i]);
-            acc += base_weight ? base_weight[t] * v : v;
-        }
-        out[static_cast<size_t>(t) * width + i] = from_float<T>(acc);
+// VEC neighbouring columns a thread.
+template <typename T, int VEC>
+__global__ __launch_bounds__(256) void moe_combine_kernel(const T* __restrict__ y, const int* __restrict__ place_of,
+                                                          const float* __restrict__ weights, const T* __restrict__ base,
+                                                          const float* __restrict__ base_weight, const T* __restrict__ x,
+                                                          T* __restrict__ out, int top, int width) {
+    const int t = blockIdx.x, i = (blockIdx.y * 256 + threadIdx.x) * VEC;
+    if (i >= width) return;
+    const size_t at = static_cast<size_t>(t) * width + i;
+    auto load = [](const T* p, float (&v)[VEC]) __attribute__((always_inline)) {
+        if constexpr (VEC == 4) Vec4<T>::load(p, v);
+        else v[0] = to_float(p[0]);
+    };
+    float acc[VEC], v[VEC];
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) acc[e] = 0.f;
+    for (int k = 0; k < top; ++k) {
+        const int entry = t * top + k;
+        const int place = place_of[entry];
+        if (place < 0 && !x) continue;
+        load(place >= 0 ? y + static_cast<size_t>(place) * width + i : x + at, v);
+        const float weight = weights ? weights[entry] : 1.f;
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) acc[e] += weight * v[e];
     }
+    if (base) {
+        load(base + at, v);
+        const float weight = base_weight ? base_weight[t] : 1.f;
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) acc[e] += weight * v[e];
+    }
+    if constexpr (VEC == 4) Vec4<T>::store(out + at, acc);
+    else out[at] = from_float<T>(acc[0]);
 }
 
 // ---------------------------------------------------------------- entry points
@@ -431,12 +446,15 @@ extern "C" int celeg_moe_router(const void* x, int x_dtype, const float* w, int 
     const MoeRule rule{experts, top, score, renorm, groups, keep, renorm_eps, scale, correction, group_best, gate_out};
     if (!moe_rule_ok(rule) || lds > 64 * 1024) return static_cast<int>(hipErrorInvalidValue);
     dim3 grid((rows + ROUTE_ROWS - 1) / ROUTE_ROWS);
-    if (x_dtype == CELEG_F32)
-        hipLaunchKernelGGL(moe_router_kernel<float>, grid, dim3(256), lds, stream, static_cast<const float*>(x), w, rows, width,
-                           rule, ids, weights);
-    else
-        hipLaunchKernelGGL(moe_router_kernel<bf16>, grid, dim3(256), lds, stream, static_cast<const bf16*>(x), w, rows, width,
-                           rule, ids, weights);
+#define ROUTER_GO(TX, THREADS)                                                                                                    \
+    hipLaunchKernelGGL((moe_router_kernel<TX, THREADS>), grid, dim3(THREADS), lds, stream, static_cast<const TX*>(x), w, rows, width, \
+                       rule, ids, weights)
+    const bool few = grid.x < 64;
+    if (x_dtype == CELEG_F32 && few) ROUTER_GO(float, 1024);
+    else if (x_dtype == CELEG_F32) ROUTER_GO(float, 256);
+    else if (few) ROUTER_GO(bf16, 1024);
+    else ROUTER_GO(bf16, 256);
+#undef ROUTER_GO
     return CELEG_LAUNCH_RESULT();
 }
 
@@ -500,12 +518,18 @@ extern "C" int celeg_moe_product(const void* a, const void* w, void* out, int dt
 extern "C" int celeg_moe_combine(const void* y, int dtype, const int* place_of, const float* weights, const void* base,
                                  const float* base_weight, const void* x, void* out, int rows, int top, int width, hipStream_t stream) {
     if (rows <= 0) return 0;
-    if (dtype == CELEG_F32)
-        hipLaunchKernelGGL(moe_combine_kernel<float>, dim3(rows), dim3(256), 0, stream, static_cast<const float*>(y),
-                           place_of, weights, static_cast<const float*>(base), base_weight, static_cast<const float*>(x), static_cast<float*>(out), top,
-                           width);
-    else
-        hipLaunchKernelGGL(moe_combine_kernel<bf16>, dim3(rows), dim3(256), 0, stream, static_cast<const bf16*>(y), place_of,
-                           weights, static_cast<const bf16*>(base), base_weight, static_cast<const bf16*>(x), static_cast<bf16*>(out), top, width);
+    const uintptr_t ends = reinterpret_cast<uintptr_t>(y) | reinterpret_cast<uintptr_t>(base) | reinterpret_cast<uintptr_t>(x) |
+                           reinterpret_cast<uintptr_t>(out);
+    const bool by_fours = width % 4 == 0 && (ends & 15) == 0;
+    const int columns = by_fours ? 1024 : 256;
+    dim3 grid(rows, (width + columns - 1) / columns);
+#define COMBINE_GO(T, VEC)                                                                                                          \
+    hipLaunchKernelGGL((moe_combine_kernel<T, VEC>), grid, dim3(256), 0, stream, static_cast<const T*>(y), place_of, weights,         \
+                       static_cast<const T*>(base), base_weight, static_cast<const T*>(x), static_cast<T*>(out), top, width)
+    if (dtype == CELEG_F32 && by_fours) COMBINE_GO(float, 4);
+    else if (dtype == CELEG_F32) COMBINE_GO(float, 1);
+    else if (by_fours) COMBINE_GO(bf16, 4);
+    else COMBINE_GO(bf16, 1);
+#undef COMBINE_GO
     return CELEG_LAUNCH_RESULT();
 }
