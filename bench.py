@@ -379,7 +379,7 @@ def main() -> int:
                          "prompt that the cache holds before the measured portion of 2,048 (default 0)")
     ap.add_argument("--design-shape", default="1k,2k", help="with --phase design: which sizes (1k, 2k)")
     ap.add_argument("--design", default="regipel", choices=["regipel", "kifetar", "kivorax", "vabuzen", "minilorn", "nosalorn"],
-                    help="with --phase design: which design is measured beside its closest LFM2 shape")
+                    help="with --phase design: which design is measured beside its closest existing model")
     ap.add_argument("--design-model", default="", choices=["", "regipel", "lfm2_attention", "kifetar", "lfm2_hybrid", "kivorax", "kifetar_beside", "vabuzen", "regipel_beside", "minilorn", "nosalorn", "kivorax_beside"],
                     help="with --phase design: only this model (for profiling)")
     ap.add_argument("--phase", choices=["all", "prefill", "decode", "serve", "design"], default="all",
